@@ -26,13 +26,12 @@ def _torch_lib() -> str:
     return str(Path(spec.origin).parent / "lib")
 
 
-# per-file hipcc flags: the prefill GEMM's dequant runs beside MFMAs, where the packed
-# v_pk_fma_f32 the SLP vectoriser forms issues slower than two scalar FMAs (profiles/r5_prefill_gemm.md)
-_NO_PK_F32 = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]   # scalar fp32 math only
-FILE_FLAGS = {"gemm_bs.hip": ["-fno-slp-vectorize"], "shortconv.hip": _NO_PK_F32, "attention_mix.hip": _NO_PK_F32,
-              "moe_dense.hip": _NO_PK_F32, "norm_chain.hip": _NO_PK_F32, "rope_pages.hip": _NO_PK_F32,
-              "retention.hip": _NO_PK_F32, "attention_latent.hip": _NO_PK_F32, "mamba2.hip": _NO_PK_F32, "delta_rule.hip": _NO_PK_F32,
-              "matrix_memory.hip": _NO_PK_F32}
+# scalar fp32 math only, in every source: some forms of the packed fp32 instructions the compiler makes
+# from ordinary float code have given wrong results on this hardware
+NO_PK_F32 = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
+# per-file hipcc flags: the prefill GEMM's dequant runs beside MFMAs, where code the SLP vectoriser
+# rearranges issues slower than plain scalar FMAs (profiles/r5_prefill_gemm.md)
+FILE_FLAGS = {"gemm_bs.hip": ["-fno-slp-vectorize"]}
 
 
 def _sources():
@@ -45,7 +44,7 @@ def _digest() -> str:
         h.update(p.name.encode())
         h.update(p.read_bytes())
     h.update(ARCH.encode())
-    h.update(repr(sorted(FILE_FLAGS.items())).encode())
+    h.update(repr((NO_PK_F32, sorted(FILE_FLAGS.items()))).encode())
     return h.hexdigest()[:16]
 
 
@@ -89,7 +88,7 @@ def _build_lib(LIB: Path, defines, force: bool, verbose: bool, jobs: int, source
         return LIB
     objdir = HERE / ("build" if not defines else "build_" + LIB.stem)
     objdir.mkdir(exist_ok=True)
-    flags = ["-O3", f"--offload-arch={ARCH}", "-fPIC", "-std=c++17", "-Wno-unused-result",
+    flags = ["-O3", f"--offload-arch={ARCH}", "-fPIC", "-std=c++17", "-Wno-unused-result", *NO_PK_F32,
              "-I", str(CSRC)] + [f"-D{d}" for d in defines]
 
     def compile_one(src: Path) -> Path:
