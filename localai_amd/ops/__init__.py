@@ -87,8 +87,8 @@ def lib():
             "la_embed": [I, P, P, P, P, I, I, P, I, P, F, P],
             "la_dequant": [I, P, P, P, P, I, I, P, P],
             "la_attn_decode": [P, P, P, P, I, P, I, I, I, I, I, F, I, I, P, P, P, P, P, LNG, I, P, P, P, P, F, I, I, P, I, P,
-                               P],
-            "la_attn_prefill": [P, P, P, P, I, P, P, P, I, I, I, I, I, F, P, F, I, P, I, P, P],
+                               P, I, P, LNG, P],
+            "la_attn_prefill": [P, P, P, P, I, P, P, P, I, I, I, I, I, F, P, F, I, P, I, P, P, I, P, LNG, P],
             "la_sample": [P, LNG, I, I, P, P, P, P, P],
             "la_penalties": [P, LNG, I, P, I, P, P, I, P, P],
             "la_penalties_cols": [P, LNG, I, P, I, P, P, I, P, I, I, P],
@@ -121,9 +121,9 @@ def lib():
             "la_bsmoe": [I, I, P, I, I, I, P, P, I, P, I, I, I, P, P, I, LNG, I, I, P],
             "la_decode_advance": [P, P, P, P, P, P, I, I, I, P, I, P, P, P],
             "la_shortconv_kv": [I, I, P, I, P, P, I, I, I, I, P, P, P, P, P, P, P, P, P, I, I, I, I, P, P, P, I, I, P],
-            "la_attn_mix_rows": [I, P, P, P, P, P, P, I, I, I, I, I, I, I, F, F, P, P, I, I, P, I, P, P, I, P, P],
-            "la_attn_mix_tiles": [P, P, P, P, I, P, P, P, I, I, I, I, I, I, F, F, P, P, I, I, P, I, P, I, P, P, I, P, I, P,
-                                  P],
+            "la_attn_mix_rows": [I, P, P, P, P, P, P, I, I, I, I, I, I, I, F, F, P, P, I, I, P, I, I, P, P, I, P, P, P],
+            "la_attn_mix_tiles": [P, P, P, P, I, P, P, P, I, I, I, I, I, I, F, F, P, P, I, I, P, I, I, P, I, P, P, I, P, I,
+                                  P, P, P],
             "la_router_sigmoid": [I, P, LNG, P, P, I, I, I, I, I, P, P, P],
             "la_router_topk": [I, I, P, LNG, P, P, I, I, I, I, I, P, P, P],
             "la_moe_pairs": [I, P, P, P, P, P, P, I, I, I, I, I, P, P, I, F, F, P],
@@ -137,6 +137,10 @@ def lib():
             "la_poly_norm_act": [P, I, LNG, I, I, I, P, F, P, I, P],
             "la_sigmoid_mul": [P, I, P, I, LNG, I, I, P, I, P],
             "la_qk_norm_rope_pages": [I, P, LNG, I, I, I, I, I, P, P, P, P, F, P, F, I, P, P, P, P, I, P],
+            "la_qk_row_norm_rope_pages": [I, P, LNG, I, I, I, I, P, P, P, P, P, F, P, I, P, P, P, I, P],
+            "la_stream_conv": [P, I, I, P, I, LNG, I, I, P, F, P, I, I, P, P, P, P, P, I, P, I, P],
+            "la_glu_act": [P, I, LNG, I, I, I, I, P, I, P],
+            "la_lightning": [I, P, I, I, I, I, I, I, P, P, P, P, I, P, P, F, P, P, P, I, P],
             "la_rotate_heads": [I, P, I, I, I, P, P, F, F, P, LNG, P],
             "la_delta_rule": [I, P, LNG, P, P, I, I, I, I, I, I, I, I, P, P, P, P, P, F, F, P, P, P, P, P, I, P, P, P, P,
                               P, P, P],
@@ -1532,27 +1536,40 @@ def decode_workspace(B: int, Hq: int, Hkv: int, Dh: int, max_len: int, device, b
             torch.zeros(max(1, B * Hkv), dtype=torch.int32, device=device))
 
 
+def _attn_extras(who: str, T: int, Hq: int, Dh: int, dist_bias, sink, sigmoid_bias, gate) -> int:
+    """Checks the optional operands of the decode / prefill attention kernels; the gate's row stride."""
+    for t in (dist_bias, sink, sigmoid_bias):
+        if t is not None and (t.dtype != torch.float32 or not t.is_contiguous() or not t.is_cuda or t.shape[-1] != Hq):
+            raise ValueError(f"{who}: dist_bias [N, Hq], sink [Hq] and sigmoid_bias [Hq] are contiguous fp32")
+    if gate is None:
+        return 0
+    if gate.dtype != torch.bfloat16 or tuple(gate.shape) != (T, Hq * Dh) or gate.stride(1) != 1 or not gate.is_cuda:
+        raise ValueError(f"{who}: the gate is a bf16 [T, Hq Dh] view with unit column stride")
+    return gate.stride(0)
+
+
 def attn_decode(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_tables: torch.Tensor,
                 seq_lens: torch.Tensor, scale: float, max_seq_len: int, out: Optional[torch.Tensor] = None,
                 workspace: Optional[Tuple[torch.Tensor, ...]] = None, softcap: float = 0.0,
                 window: int = 0, dist_bias: Optional[torch.Tensor] = None,
-                sink: Optional[torch.Tensor] = None) -> torch.Tensor:
+                sink: Optional[torch.Tensor] = None, sigmoid_bias: Optional[torch.Tensor] = None, chunk: int = 0,
+                gate: Optional[torch.Tensor] = None) -> torch.Tensor:
     """q [B,Hq,Dh] bf16; K cache [nblk,Hkv,BS,Dh]; V cache (grouped-transposed pages)
     [nblk,Hkv,BS/8,Dh,8]; block_tables [B,maxb] i32; seq_lens [B] i32.  softcap > 0: scores
     softcap * tanh(s / softcap); window > 0: only the last `window` keys are attended (Gemma-2).
     dist_bias (fp32 [N, Hq]) / sink (fp32 [Hq]): a bias per distance and head (constant from row
-    N - 1 on) and a logit without key or value in the softmax denominator, as in attn_mix."""
+    N - 1 on) and a logit without key or value in the softmax denominator, as in attn_mix.
+    sigmoid_bias (fp32 [Hq]), chunk, gate ([B, Hq Dh], any row stride): sigmoid weights instead of the
+    softmax, the chunked mask and a logit per output channel, as in attn_mix."""
     B, Hq, Dh = q.shape
     nblk, Hkv, BS, Dh2 = k_cache.shape
     if Dh2 != Dh or Hq % Hkv or tuple(v_cache.shape) != (nblk, Hkv, BS // 8, Dh, 8):
         raise ValueError("attn_decode: head/cache shape mismatch")
     if not q.is_cuda:
-        if dist_bias is not None or sink is not None:
-            raise ValueError("attn_decode: distance bias and sink have no CPU path here (attn_mix has)")
+        if dist_bias is not None or sink is not None or sigmoid_bias is not None or chunk or gate is not None:
+            raise ValueError("attn_decode: score extras, chunks and gates have no CPU path here (attn_mix has)")
         return _attn_ref_decode(q, k_cache, v_cache, block_tables, seq_lens, scale, softcap, window)
-    for t in (dist_bias, sink):
-        if t is not None and (t.dtype != torch.float32 or not t.is_contiguous() or not t.is_cuda or t.shape[-1] != Hq):
-            raise ValueError("attn_decode: dist_bias [N, Hq] and sink [Hq] are contiguous fp32")
+    ldg = _attn_extras("attn_decode", B, Hq, Dh, dist_bias, sink, sigmoid_bias, gate)
     P, PS = decode_partitions(B, Hkv, max_seq_len, BS)
     if out is None:
         out = torch.empty(B, Hq, Dh, dtype=torch.bfloat16, device=q.device)
@@ -1564,7 +1581,8 @@ def attn_decode(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, b
                                 block_tables.shape[1], seq_lens.data_ptr(), B, Hq, Hkv, Dh, BS, float(scale), P, PS,
                                 out.data_ptr(), po.data_ptr(), pml.data_ptr(), tk.data_ptr(), None, 0, 0, None, None,
                                 None, None, float(softcap), int(window), _dec_nw(B, Hkv), _ptr(dist_bias),
-                                dist_bias.shape[0] if dist_bias is not None else 0, _ptr(sink), _stream()),
+                                dist_bias.shape[0] if dist_bias is not None else 0, _ptr(sink), _ptr(sigmoid_bias),
+                                int(chunk), _ptr(gate), ldg, _stream()),
            "la_attn_decode")
     return out
 
@@ -1609,7 +1627,7 @@ def attn_decode_rope(qkv: Partial, pos: torch.Tensor, slots: torch.Tensor, cos_s
                                 block_tables.shape[1], seq_lens.data_ptr(), T, Hq, Hkv, Dh, BS, float(scale), P, PS,
                                 out.data_ptr(), po.data_ptr(), pml.data_ptr(), tk.data_ptr(), a[0], a[1], a[2], a[3],
                                 pos.data_ptr(), slots.data_ptr(), cos_sin.data_ptr(), float(softcap), int(window),
-                                _dec_nw(T, Hkv), None, 0, None, _stream()),
+                                _dec_nw(T, Hkv), None, 0, None, None, 0, None, 0, _stream()),
            "la_attn_decode(rope)")
     return out
 
@@ -1677,18 +1695,18 @@ def attn_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, 
                  ctx_lens: torch.Tensor, block_tables: torch.Tensor, scale: float,
                  tiles: Optional[torch.Tensor] = None, q_lens: Optional[Sequence[int]] = None,
                  out: Optional[torch.Tensor] = None, softcap: float = 0.0, window: int = 0,
-                 dist_bias: Optional[torch.Tensor] = None, sink: Optional[torch.Tensor] = None) -> torch.Tensor:
+                 dist_bias: Optional[torch.Tensor] = None, sink: Optional[torch.Tensor] = None,
+                 sigmoid_bias: Optional[torch.Tensor] = None, chunk: int = 0,
+                 gate: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Causal attention for new tokens. q [T,Hq,Dh]; cu_q [nseq+1]; ctx_lens [nseq] (cached+new).
-    dist_bias (fp32 [N, Hq]) / sink (fp32 [Hq]): as in attn_decode and attn_mix."""
+    dist_bias (fp32 [N, Hq]) / sink / sigmoid_bias (fp32 [Hq]) / chunk / gate: as in attn_decode and attn_mix."""
     T, Hq, Dh = q.shape
     Hkv = k_cache.shape[1]
     if not q.is_cuda:
-        if dist_bias is not None or sink is not None:
-            raise ValueError("attn_prefill: distance bias and sink have no CPU path here (attn_mix has)")
+        if dist_bias is not None or sink is not None or sigmoid_bias is not None or chunk or gate is not None:
+            raise ValueError("attn_prefill: score extras, chunks and gates have no CPU path here (attn_mix has)")
         return _attn_ref_prefill(q, k_cache, v_cache, cu_q, ctx_lens, block_tables, scale, softcap, window)
-    for t in (dist_bias, sink):
-        if t is not None and (t.dtype != torch.float32 or not t.is_contiguous() or not t.is_cuda or t.shape[-1] != Hq):
-            raise ValueError("attn_prefill: dist_bias [N, Hq] and sink [Hq] are contiguous fp32")
+    ldg = _attn_extras("attn_prefill", T, Hq, Dh, dist_bias, sink, sigmoid_bias, gate)
     if tiles is None:
         cq = cu_q.cpu().tolist()
         tiles = prefill_tiles([cq[i + 1] - cq[i] for i in range(len(cq) - 1)], q.device)
@@ -1698,7 +1716,8 @@ def attn_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, 
                                  tiles.shape[0], cu_q.data_ptr(), ctx_lens.data_ptr(), block_tables.data_ptr(),
                                  block_tables.shape[1], Hq, Hkv, Dh, k_cache.shape[2], float(scale),
                                  out.data_ptr(), float(softcap), int(window), _ptr(dist_bias),
-                                 dist_bias.shape[0] if dist_bias is not None else 0, _ptr(sink), _stream()), "la_attn_prefill")
+                                 dist_bias.shape[0] if dist_bias is not None else 0, _ptr(sink), _ptr(sigmoid_bias),
+                                 int(chunk), _ptr(gate), ldg, _stream()), "la_attn_prefill")
     return out
 
 
@@ -1879,7 +1898,7 @@ def attn_mix(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, row_
              window: int = 0, gate: Optional[torch.Tensor] = None, tiles: Optional[torch.Tensor] = None,
              tile_rows: int = 0, cu_q: Optional[torch.Tensor] = None, key_splits: int = 1,
              v_width: int = 0, dist_bias: Optional[torch.Tensor] = None,
-             sink: Optional[torch.Tensor] = None) -> torch.Tensor:
+             sink: Optional[torch.Tensor] = None, sigmoid_bias: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Attention with reshaped scores over paged K ([blocks, G, BS, Dk]) and V ([blocks, G, BS / 8,
     Dv, 8], transposed per 8 keys: the operand layout of the P.V matrix instruction); one
     query row per token, row r belonging to sequence row_seq[r] (block_tables row) at position
@@ -1887,7 +1906,7 @@ def attn_mix(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, row_
     minus slopes[g] * distance; then the heads' scores are mixed by talk [H, H]; keys are visible
     within the query's chunk of `chunk` positions and the last `window` positions (0: no limit);
     softmax; values of width Dv; each head's output times sigmoid(gate[r, h]) (gate: [T, H] view,
-    any row stride).  Returns [T, H * Dv] in q's dtype; scores and softmax in fp32.
+    any row stride), or, with a [T, H Dv] gate, every output channel times the sigmoid of its own logit.  Returns [T, H * Dv] in q's dtype; scores and softmax in fp32.
     tiles / tile_rows / cu_q (attn_mix_tiles): the first tile_rows rows are whole prompt portions,
     positions consecutive within each; in bf16 and where the shape allows (key width % 32, value
     width % 16 and <= 128, at most 32 heads) they run on the matrix-core tile kernel, every other
@@ -1901,7 +1920,9 @@ def attn_mix(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, row_
     dist_bias (fp32 [N, H]): dist_bias[min(i - j, N - 1), h] is added to head h's score of key j
     after scale and softcap (a learned bias per distance, constant from N - 1 on; see
     bucketed_bias).  sink (fp32 [H]): the softmax denominator of head h also holds exp(sink[h]),
-    a logit without key or value that counts once per query.  Both need talk None."""
+    a logit without key or value that counts once per query.  Both need talk None.
+    sigmoid_bias (fp32 [H]): no softmax; a visible key's weight is sigmoid(s + sigmoid_bias[h]), not
+    normalised over the keys."""
     T = q.shape[0]
     G, BS, Dk = k_cache.shape[1], k_cache.shape[2], k_cache.shape[3]
     if (dist_bias is not None or sink is not None) and (talk is not None or v_cache is None):
@@ -1910,6 +1931,8 @@ def attn_mix(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, row_
         raise ValueError("attn_mix: dist_bias is [N, H]")
     if sink is not None and sink.numel() != H:
         raise ValueError("attn_mix: sink is [H]")
+    if sigmoid_bias is not None and (sigmoid_bias.numel() != H or sink is not None or v_cache is None):
+        raise ValueError("attn_mix: sigmoid_bias is [H], without sinks and latent caches")
     if v_cache is None:
         if not 0 < v_width <= Dk:
             raise ValueError("attn_mix: without V pages v_width names the value columns of a key row")
@@ -1946,13 +1969,15 @@ def attn_mix(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, row_
                 s = talk.float() @ s
             if dist_bias is not None:
                 s = s + dist_bias.float()[(i - js).clamp(max=dist_bias.shape[0] - 1)].t()
-            if sink is not None:    # one more logit in the denominator, nothing in the numerator
+            if sigmoid_bias is not None:
+                pr = torch.sigmoid(s + sigmoid_bias.float().view(H, 1))
+            elif sink is not None:    # one more logit in the denominator, nothing in the numerator
                 pr = torch.softmax(torch.cat([s, sink.float().view(H, 1)], 1), -1)[:, :-1]
             else:
                 pr = torch.softmax(s, -1)
             o = torch.einsum("hn,nhd->hd", pr, vv)
             if gate is not None:
-                o = o * torch.sigmoid(gate[r].float()).view(H, 1)
+                o = o * torch.sigmoid(gate[r].float()).view(H, gate.shape[1] // H)
             out[r] = o
         return out.view(T, H * Dv).to(q.dtype)
     f32 = q.dtype == torch.float32
@@ -1964,15 +1989,17 @@ def attn_mix(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, row_
         raise ValueError("attn_mix: operands must be contiguous")
     for t in (row_seq, pos, block_tables):
         assert t.dtype == torch.int32 and t.is_cuda
-    for t in (slopes, talk, dist_bias, sink):
+    for t in (slopes, talk, dist_bias, sink, sigmoid_bias):
         assert t is None or (t.dtype == torch.float32 and t.is_contiguous() and t.is_cuda)
     assert slopes is None or slopes.numel() == H
     nbias = dist_bias.shape[0] if dist_bias is not None else 0
     assert talk is None or tuple(talk.shape) == (H, H)
-    ldg = 0
+    ldg, gch = 0, 0
     if gate is not None:
-        if gate.dtype != q.dtype or tuple(gate.shape) != (T, H) or gate.stride(1) != 1:
-            raise ValueError("attn_mix: gate must be a [T, H] view of q's dtype with unit column stride")
+        gch = int(gate.shape[1] != H)        # a logit per output channel
+        if (gate.dtype != q.dtype or tuple(gate.shape) not in ((T, H), (T, H * Dv)) or gate.stride(1) != 1
+                or (gch and v_cache is None)):
+            raise ValueError("attn_mix: gate must be a [T, H] or [T, H Dv] view of q's dtype with unit column stride")
         ldg = gate.stride(0)
     out = torch.empty(T, H * Dv, dtype=q.dtype, device=q.device)
     r0 = 0
@@ -2004,8 +2031,9 @@ def attn_mix(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, row_
         rc = lib().la_attn_mix_tiles(q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), tiles.data_ptr(),
                                      tiles.shape[0], cu_q.data_ptr(), pos.data_ptr(), block_tables.data_ptr(),
                                      block_tables.shape[1], H, G, Dk, Dv, BS, float(scale), float(softcap), _ptr(slopes),
-                                     _ptr(talk), int(chunk), int(window), _ptr(gate), ldg, out.data_ptr(), ns,
-                                     _ptr(po), _ptr(pml), tile_rows, _ptr(dist_bias), nbias, _ptr(sink), _stream())
+                                     _ptr(talk), int(chunk), int(window), _ptr(gate), ldg, gch, out.data_ptr(), ns,
+                                     _ptr(po), _ptr(pml), tile_rows, _ptr(dist_bias), nbias, _ptr(sink),
+                                     _ptr(sigmoid_bias), _stream())
         if rc == 0:
             r0 = tile_rows
         elif rc != 1:
@@ -2016,8 +2044,9 @@ def attn_mix(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, row_
                                       _ptr(v_cache), row_seq.data_ptr() + r0 * 4, pos.data_ptr() + r0 * 4,
                                       block_tables.data_ptr(), block_tables.shape[1], T - r0, H, G, Dk, Dv, BS,
                                       float(scale), float(softcap), _ptr(slopes), _ptr(talk), int(chunk), int(window),
-                                      None if gate is None else gate.data_ptr() + r0 * ldg * esz, ldg,
-                                      out.data_ptr() + r0 * H * Dv * esz, _ptr(dist_bias), nbias, _ptr(sink), _stream()),
+                                      None if gate is None else gate.data_ptr() + r0 * ldg * esz, ldg, gch,
+                                      out.data_ptr() + r0 * H * Dv * esz, _ptr(dist_bias), nbias, _ptr(sink),
+                                      _ptr(sigmoid_bias), _stream()),
                "la_attn_mix_rows")
     return out
 
@@ -2144,26 +2173,29 @@ def _ln_ref(y: torch.Tensor, w: torch.Tensor, eps: float) -> torch.Tensor:
     return d * torch.rsqrt(d.pow(2).mean(-1, keepdim=True) + eps) * w.float()
 
 
+def _rms_ref(y: torch.Tensor, w: torch.Tensor, eps: float) -> torch.Tensor:
+    return y * torch.rsqrt(y.pow(2).mean(-1, keepdim=True) + eps) * w.float()
+
+
 def norm_chain(res: torch.Tensor, branch=None, post: Optional[tuple] = None, pre: Optional[tuple] = None,
                add_vec: Optional[torch.Tensor] = None, replace: bool = False,
                out_dtype: torch.dtype = torch.bfloat16) -> Optional[torch.Tensor]:
     """One launch per sublayer boundary of a post-normed residual stream (fp32 [T, D], updated in
     place):  res <- (0 if replace else res) + post(branch) + add_vec, then returns pre(res).
     post / pre:  ("dyt", alpha, w, b): tanh(alpha x) * w + b, a norm without statistics (alpha a
-    Python float, w / b fp32 [D]);  ("rms", w, eps): x / sqrt(mean(x^2) + eps) * w (post only);
-    ("ln", w, eps): (x - mean) / sqrt(mean((x - mean)^2) + eps) * w, a layer norm without bias (post
-    and pre);  ("cast",): res in out_dtype (pre only);  None: identity for post, no output for pre.
+    Python float, w / b fp32 [D]);  ("rms", w, eps): x / sqrt(mean(x^2) + eps) * w;
+    ("ln", w, eps): (x - mean) / sqrt(mean((x - mean)^2) + eps) * w, a layer norm without bias;  ("cast",): res in out_dtype (pre only);  None: identity for post, no output for pre.
     branch: a Partial or dense [T, D] tensor (None: the stream is only read).  All arithmetic fp32."""
     T, D = res.shape
     pm = NORM_NONE if post is None else {"dyt": NORM_DYT, "rms": NORM_RMS, "ln": NORM_LN}[post[0]]
-    qm = NORM_NONE if pre is None else {"dyt": NORM_DYT, "cast": NORM_CAST, "ln": NORM_LN}[pre[0]]
+    qm = NORM_NONE if pre is None else {"dyt": NORM_DYT, "cast": NORM_CAST, "ln": NORM_LN, "rms": NORM_RMS}[pre[0]]
     if not res.is_cuda:
         if branch is not None:
             y = _branch_dense(branch)
             if pm == NORM_DYT:
                 y = torch.tanh(float(post[1]) * y) * post[2].float() + post[3].float()
             elif pm == NORM_RMS:
-                y = y * torch.rsqrt(y.pow(2).mean(-1, keepdim=True) + float(post[2])) * post[1].float()
+                y = _rms_ref(y, post[1], float(post[2]))
             elif pm == NORM_LN:
                 y = _ln_ref(y, post[1], float(post[2]))
             if add_vec is not None:
@@ -2176,6 +2208,8 @@ def norm_chain(res: torch.Tensor, branch=None, post: Optional[tuple] = None, pre
             return (torch.tanh(float(pre[1]) * res) * pre[2].float() + pre[3].float()).to(out_dtype)
         if qm == NORM_LN:
             return _ln_ref(res, pre[1], float(pre[2])).to(out_dtype)
+        if qm == NORM_RMS:
+            return _rms_ref(res, pre[1], float(pre[2])).to(out_dtype)
         return res.to(out_dtype) if qm == NORM_CAST else None
     if res.dtype != torch.float32 or not res.is_contiguous() or out_dtype not in (torch.float32, torch.bfloat16):
         raise ValueError("norm_chain: the stream is contiguous fp32; outputs are bf16 or fp32")
@@ -2186,7 +2220,7 @@ def norm_chain(res: torch.Tensor, branch=None, post: Optional[tuple] = None, pre
     elif pm in (NORM_RMS, NORM_LN):
         pw, eps = post[1], float(post[2])
     qa, qw_, qb = (float(pre[1]), pre[2], pre[3]) if qm == NORM_DYT else (0.0, None, None)
-    if qm == NORM_LN:       # the output norm's eps travels in the slot of the squashing norm's alpha
+    if qm in (NORM_LN, NORM_RMS):       # the output norm's eps travels in the slot of the squashing norm's alpha
         qa, qw_ = float(pre[2]), pre[1]
     for t in (pw, pb, qw_, qb, add_vec):
         if t is not None and (t.dtype != torch.float32 or t.numel() != D or not t.is_contiguous()):
@@ -2764,6 +2798,177 @@ def rotate_heads(x: torch.Tensor, H: int, Dv: int, pos: torch.Tensor, freqs: tor
     _check(lib().la_rotate_heads(int(x.dtype == torch.float32), x.data_ptr(), T, H, Dv, pos.data_ptr(), freqs.data_ptr(),
                                  float(sign), float(scale), out.data_ptr() + col0 * es, out.stride(0), _stream()),
            "la_rotate_heads")
+    return out
+
+
+def qk_row_norm_rope_pages(src: torch.Tensor, H: int, D: int, G: int, pos: torch.Tensor, slots: torch.Tensor,
+                           q_w: torch.Tensor, k_w: torch.Tensor, eps: float, freqs: torch.Tensor, rot: int,
+                           k_cache: torch.Tensor, v_cache: torch.Tensor,
+                           head_scale: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Queries and keys normed over their whole projections, keys that are also the values: of projection
+    rows src [T, >= H D + G D] (q | k, any row stride) all H D query columns are divided by
+    sqrt(mean x^2 + eps) over the row and multiplied by q_w (fp32 [H D]), the G D key columns likewise
+    (k_w [G D]); dims i and i + rot / 2 of every head's first `rot` dims are turned by the angle pos *
+    freqs[i]; queries are multiplied by head_scale[h] (fp32 [H]).  Returns q [T, H D]; the keys go to the
+    K pool [blocks, G, BS, D] and the raw keys, before norm and rotation, to the V pool [blocks, G,
+    BS / 8, D, 8] at `slots` (-1: nowhere).  Norms, angles and rotations fp32."""
+    T = src.shape[0]
+    Cq, Ck = H * D, G * D
+    if (src.dim() != 2 or src.shape[1] < Cq + Ck or pos.shape[0] != T or src.stride(1) != 1 or rot % 2 or rot > D
+            or freqs.numel() != rot // 2 or q_w.numel() != Cq or k_w.numel() != Ck or slots.shape[0] != T
+            or (head_scale is not None and head_scale.numel() != H)):
+        raise ValueError("qk_row_norm_rope_pages: operand shapes do not fit")
+    if (tuple(k_cache.shape[1:]) != (G, k_cache.shape[2], D)
+            or tuple(v_cache.shape[1:]) != (G, k_cache.shape[2] // 8, D, 8)):
+        raise ValueError("qk_row_norm_rope_pages: pools do not fit the key width")
+    if not src.is_cuda:
+        x = src.float()
+        q = _rotate_ref(_rms_ref(x[:, :Cq], q_w, eps).reshape(T, H, D), pos, freqs, 1.0, rot, 0, False)
+        k = _rotate_ref(_rms_ref(x[:, Cq:Cq + Ck], k_w, eps).reshape(T, G, D), pos, freqs, 1.0, rot, 0, False)
+        if head_scale is not None:
+            q = q * head_scale.float().view(1, H, 1)
+        _page_write_ref(k_cache, v_cache, slots, k, x[:, Cq:Cq + Ck].reshape(T, G, D))
+        return q.reshape(T, Cq).to(src.dtype)
+    if src.dtype not in (torch.float32, torch.bfloat16) or k_cache.dtype != src.dtype or v_cache.dtype != src.dtype:
+        raise ValueError("qk_row_norm_rope_pages: bf16 or fp32 rows, pools of the same dtype")
+    assert pos.dtype == torch.int32 and slots.dtype == torch.int32
+    for t in (q_w, k_w, freqs, head_scale):
+        assert t is None or (t.dtype == torch.float32 and t.is_contiguous() and t.is_cuda)
+    q = torch.empty(T, Cq, dtype=src.dtype, device=src.device)
+    _check(lib().la_qk_row_norm_rope_pages(int(src.dtype == torch.float32), src.data_ptr(), src.stride(0), T, H, D, G,
+                                           pos.data_ptr(), slots.data_ptr(), q_w.data_ptr(), k_w.data_ptr(), _ptr(head_scale),
+                                           float(eps), freqs.data_ptr() if rot else None, rot, q.data_ptr(),
+                                           k_cache.data_ptr(), v_cache.data_ptr(), k_cache.shape[2], _stream()),
+           "la_qk_row_norm_rope_pages")
+    return q
+
+
+def stream_conv(res: torch.Tensor, branch, post: Optional[tuple], w_t: torch.Tensor, row_seq: torch.Tensor,
+                cu_q: torch.Tensor, pos: torch.Tensor, sslots: torch.Tensor, tail: torch.Tensor, single: bool = False,
+                out_dtype: torch.dtype = torch.bfloat16) -> torch.Tensor:
+    """Sublayer boundary with a short convolution on the residual stream (fp32 [T, D], updated in place):
+    res <- res + post(branch) (branch None: only read; post None or ("rms", w, eps), as in norm_chain), then
+    returns res + conv(res), conv(x)_t = sum_j w_t[j] * x_(t - taps + 1 + j) per channel (w_t fp32 [taps, D],
+    zeros before position 0).  Rows of a sequence portion are consecutive (row_seq [T], cu_q [nseq + 1],
+    pos [T]); what precedes a portion comes from tail[sslots[seq]] (fp32 [slots, taps - 1, D]: the stream's
+    last rows), which advances to the portion's end.  single: one row per sequence -- norm, add,
+    convolution and tail in one launch.  All arithmetic fp32."""
+    T, D = res.shape
+    taps, nseq = w_t.shape[0], sslots.shape[0]
+    if (w_t.shape[1] != D or tuple(tail.shape[1:]) != (taps - 1, D) or pos.shape[0] != T
+            or (single and nseq != T) or (not single and (cu_q.shape[0] != nseq + 1 or row_seq.shape[0] != T))):
+        raise ValueError("stream_conv: operand shapes do not fit")
+    if not res.is_cuda:
+        if branch is not None:
+            norm_chain(res, branch, post, None)
+        out = res.clone()
+        cu = list(range(T + 1)) if single else cu_q.tolist()
+        for s in range(nseq):
+            a, b = cu[s], cu[s + 1]
+            if b <= a:
+                continue
+            ss = int(sslots[s])
+            hist = _conv_hist_ref(tail, ss, int(pos[a]), taps, D) if ss >= 0 else torch.zeros(taps - 1, D)
+            ext = torch.cat([hist, res[a:b]], 0)
+            for j in range(taps):
+                out[a:b] += w_t[j].float() * ext[j:j + (b - a)]
+            if ss >= 0 and taps > 1:
+                tail[ss] = ext[-(taps - 1):]
+        return out.to(out_dtype)
+    if res.dtype != torch.float32 or not res.is_contiguous() or out_dtype not in (torch.float32, torch.bfloat16):
+        raise ValueError("stream_conv: the stream is contiguous fp32; outputs are bf16 or fp32")
+    for t in (w_t, tail):
+        if t.dtype != torch.float32 or not t.is_contiguous() or not t.is_cuda:
+            raise ValueError("stream_conv: weights and tails are contiguous fp32 on the device")
+    for t in (pos, sslots) + (() if single else (row_seq, cu_q)):
+        assert t.dtype == torch.int32 and t.is_cuda and t.is_contiguous()
+    if branch is not None and not single:
+        norm_chain(res, branch, post, None)
+        branch = None
+    a = _branch_args(branch, T, D) if branch is not None else (None, 0, 0, 1)
+    pm, pw, eps = NORM_NONE, None, 0.0
+    if branch is not None and post is not None:
+        if post[0] != "rms":
+            raise ValueError("stream_conv: the branch norm is rms or none")
+        pm, pw, eps = NORM_RMS, post[1], float(post[2])
+        if pw.dtype != torch.float32 or pw.numel() != D or not pw.is_contiguous():
+            raise ValueError("stream_conv: the branch norm's weights are contiguous fp32 [D]")
+    out = torch.empty(T, D, dtype=out_dtype, device=res.device)
+    _check(lib().la_stream_conv(res.data_ptr(), T, D, a[0], a[1], a[2], a[3], pm, _ptr(pw), eps, w_t.data_ptr(), taps, nseq,
+                                None if single else row_seq.data_ptr(), None if single else cu_q.data_ptr(), pos.data_ptr(),
+                                sslots.data_ptr(), tail.data_ptr() if taps > 1 else None, int(single), out.data_ptr(),
+                                int(out_dtype == torch.float32), _stream()), "la_stream_conv")
+    return out
+
+
+def glu_act(src, F: int, mode: int, out_dtype: torch.dtype = torch.bfloat16) -> torch.Tensor:
+    """act(gate) * up of a projection [gate (F) | up (F)]: mode ACT_SWIGLU (silu) or ACT_GEGLU (the tanh form of
+    gelu), fp32 arithmetic, any width, [T, F] in out_dtype.  bf16 rows whose width `act` takes run its kernels."""
+    t = src.t if isinstance(src, Partial) else src
+    T = t.shape[-2]
+    if mode not in GLU_ACTS or t.shape[-1] != 2 * F:
+        raise ValueError("glu_act: [gate | up] rows of width 2 F, a gated activation")
+    if not t.is_cuda:
+        x = _branch_dense(src)
+        g = torch.nn.functional.silu(x[:, :F]) if mode == ACT_SWIGLU else torch.nn.functional.gelu(x[:, :F], approximate="tanh")
+        return (g * x[:, F:]).to(out_dtype)
+    if isinstance(src, Partial) and out_dtype == torch.bfloat16 and F % 4 == 0:
+        return act(src, F, mode)
+    a = _branch_args(src, T, 2 * F)
+    out = torch.empty(T, F, dtype=out_dtype, device=t.device)
+    _check(lib().la_glu_act(a[0], a[1], a[2], a[3], T, F, 0 if mode == ACT_SWIGLU else 1, out.data_ptr(),
+                            int(out_dtype == torch.float32), _stream()), "la_glu_act")
+    return out
+
+
+def lightning(src: torch.Tensor, H: int, Dk: int, Dv: int, pos: torch.Tensor, cu_q: torch.Tensor, sslots: torch.Tensor,
+              state: torch.Tensor, decay: torch.Tensor, norm_w: torch.Tensor, eps: float, max_rows: int = 0) -> torch.Tensor:
+    """Lightning attention over projection rows src [T, 2 H Dk + 2 H Dv] (q | k | v | gate): silu on q, k and v;
+    per head S <- decay_h S + k v^T, o = S^T q (no softmax, no scale, no rotation); the heads' outputs side by
+    side divided by the root mean square of the whole row (eps), times norm_w (fp32 [H Dv]), times
+    sigmoid(gate).  Portions, state slots (fp32, retention_state) and max_rows as in ops.retention; state,
+    activations, outputs and the norm are fp32.  Returns [T, H Dv] in src's dtype."""
+    T = src.shape[0]
+    nseq = cu_q.shape[0] - 1
+    Cq, Cv = H * Dk, H * Dv
+    if (src.dim() != 2 or src.shape[1] != 2 * Cq + 2 * Cv or tuple(state.shape[1:]) != (H, Dv, Dk) or decay.numel() != H
+            or norm_w.numel() != Cv or sslots.shape[0] != nseq or pos.shape[0] != T):
+        raise ValueError("lightning: operand shapes do not fit")
+    if not src.is_cuda:
+        x = src.float()
+        act3 = torch.nn.functional.silu(x[:, :2 * Cq + Cv])
+        q, k, v = act3[:, :Cq].reshape(T, H, Dk), act3[:, Cq:2 * Cq].reshape(T, H, Dk), act3[:, 2 * Cq:].reshape(T, H, Dv)
+        o = torch.zeros(T, H, Dv)
+        cu = cu_q.tolist()
+        d = decay.float().view(H, 1, 1)
+        for s in range(nseq):
+            a, b = cu[s], cu[s + 1]
+            if b <= a:
+                continue
+            ss = int(sslots[s])
+            S = torch.zeros(H, Dk, Dv) if int(pos[a]) == 0 else state[ss].float().transpose(1, 2).clone()
+            for t in range(a, b):
+                S = d * S + k[t].unsqueeze(2) * v[t].unsqueeze(1)
+                o[t] = torch.einsum("hkv,hk->hv", S, q[t])
+            state[ss] = S.transpose(1, 2)
+        return (_rms_ref(o.reshape(T, Cv), norm_w, eps) * torch.sigmoid(x[:, 2 * Cq + Cv:])).to(src.dtype)
+    if src.dtype not in (torch.float32, torch.bfloat16) or not src.is_contiguous():
+        raise ValueError("lightning: contiguous bf16 or fp32 rows")
+    if state.dtype != torch.float32 or not state.is_contiguous():
+        raise ValueError("lightning: the state pool is contiguous fp32")
+    for t in (pos, cu_q, sslots):
+        assert t.dtype == torch.int32 and t.is_cuda and t.is_contiguous()
+    for t in (decay, norm_w):
+        assert t.dtype == torch.float32 and t.is_contiguous() and t.is_cuda
+    o = torch.empty(T, Cv, dtype=torch.float32, device=src.device)
+    out = torch.empty(T, Cv, dtype=src.dtype, device=src.device)
+    max_rows = int(max_rows) if max_rows > 0 else T
+    seg = torch.empty((T // RETENTION_SEG + nseq) * H * Dv * Dk, dtype=torch.float32, device=src.device) \
+        if (T >= 8 * RETENTION_SEG and max_rows >= 4 * RETENTION_SEG) else None
+    _check(lib().la_lightning(int(src.dtype == torch.float32), src.data_ptr(), src.stride(0), T, nseq, H, Dk, Dv,
+                              pos.data_ptr(), cu_q.data_ptr(), sslots.data_ptr(), state.data_ptr(), state.shape[0],
+                              decay.data_ptr(), norm_w.data_ptr(), float(eps), o.data_ptr(), out.data_ptr(), _ptr(seg),
+                              max_rows, _stream()), "la_lightning")
     return out
 
 

@@ -115,16 +115,28 @@ LA_DEV void rope_src_load(const DecRope& R, int b, int col, float (&v)[N]) {
 // Score extras of designs without rotation: a bias per distance and head added to the scaled score
 // (table [n][Hq] fp32, constant from row n - 1 on) and a sink logit per head that joins the softmax
 // denominator once, without key or value (counted by wave 0 of the first partition).
+// sig: a bias per head that replaces the softmax: a visible key's weight is sigmoid(score + sig[head]),
+// not normalised over the keys (the running maximum stays 0, the running sum 1).  chunk: keys of the
+// query's chunk of that many positions only (0: all).  gate: a logit per output channel (row stride
+// ldg), the output times its sigmoid.
 struct DecExtra {
   const float* bias;
   int nbias;
   const float* sink;
+  const float* sig;
+  int chunk;
+  const bf16* gate;
+  long ldg;
 };
+
+LA_DEV float gate_at(const DecExtra& E, long row, int col) {
+  return 1.f / (1.f + __expf(-(float)E.gate[row * E.ldg + col]));
+}
 
 // K/V are streamed once per decode step: non-temporal loads (the default) read them 12-14 %
 // faster at batch 256 (5.05 -> 5.70 TB/s at 256 keys, 5.21 -> 5.98 at 384;
 // profiles/r4_attn_decode_nt.md).  VAR bit 0 = ordinary cached loads (A/B only); bit 1 = keys
-// two tiles ahead (measured no faster; kept for the A/B).
+// two tiles ahead (measured no faster; kept for the A/B); bit 2 = sigmoid weights (DecExtra sig).
 template <int DH, int GT, int NW, int VAR = 0>
 __global__ __launch_bounds__(NW * 64) __attribute__((amdgpu_waves_per_eu(2))) void attn_decode_kernel(
     const bf16* __restrict__ q, const bf16* __restrict__ kc, const bf16* __restrict__ vc,
@@ -147,7 +159,8 @@ __global__ __launch_bounds__(NW * 64) __attribute__((amdgpu_waves_per_eu(2))) vo
   const int PS = (L <= one_part && PS_grid < one_part) ? one_part : PS_grid;
   const int t0 = p * PS;
   if (t0 >= L) return;  // empty partition: the combiner only waits for ceil(L / PS) of them
-  const int wlo = window > 0 ? L - window : 0;  // first key inside the sliding window
+  int wlo = window > 0 ? L - window : 0;  // first key inside the sliding window / the chunk
+  if (E.chunk > 0) wlo = max(wlo, (L - 1) / E.chunk * E.chunk);
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int r = lane & 15, g = lane >> 4;
   const int kend = min(L, t0 + PS);
@@ -254,6 +267,13 @@ __global__ __launch_bounds__(NW * 64) __attribute__((amdgpu_waves_per_eu(2))) vo
     m = E.sink[hq_r] * 1.4426950408889634f;
     lsum = g == 0 ? 1.f : 0.f;                        // the lane groups' sums are added up at the end
   }
+  constexpr bool SIG = (VAR & 4) != 0;
+  float sig_l2 = 0.f;
+  if constexpr (SIG) {
+    sig_l2 = E.sig[hq_r] * 1.4426950408889634f;
+    m = 0.f;
+    lsum = (p == 0 && wave == 0 && g == 0) ? 1.f : 0.f;
+  }
 
   // register double buffer up to Dh 128; a Dh-256 tile (Gemma) is 128 VGPRs on its own, so it
   // is loaded at the top of each iteration instead (no prefetch, no spills)
@@ -261,6 +281,7 @@ __global__ __launch_bounds__(NW * 64) __attribute__((amdgpu_waves_per_eu(2))) vo
   // K2: keys two tiles ahead (V stays one ahead: a whole second tile does not fit in 256 VGPRs)
   constexpr bool K2 = (VAR & 2) != 0;
   int kb = t0 + 32 * wave;
+  if (wlo > kb) kb += (wlo - kb) / (32 * NW) * (32 * NW);   // this wave's tiles that end before the first visible key
   if (kb < kend) {
     DecTile<DH> cur, nxt;
     bf16x8 k2[2][(DH + 31) / 32];
@@ -300,6 +321,13 @@ __global__ __launch_bounds__(NW * 64) __attribute__((amdgpu_waves_per_eu(2))) vo
           s[t][i] = (key < kend && key >= wlo) ? sv : -INFINITY;
         }
       }
+      bf16x8 pa;
+      if constexpr (SIG) {
+#pragma unroll
+        for (int t = 0; t < 2; ++t)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) pa[4 * t + i] = (bf16)(1.f / (1.f + exp2f(-(s[t][i] + sig_l2))));
+      } else {
       // online softmax for head r over this 32-key tile
       float mx = fmaxf(fmaxf(fmaxf(s[0][0], s[0][1]), fmaxf(s[0][2], s[0][3])),
                        fmaxf(fmaxf(s[1][0], s[1][1]), fmaxf(s[1][2], s[1][3])));
@@ -308,7 +336,6 @@ __global__ __launch_bounds__(NW * 64) __attribute__((amdgpu_waves_per_eu(2))) vo
       const float mnew = fmaxf(m, mx);
       const float msafe = (mnew == -INFINITY) ? 0.f : mnew;
       const float alpha = exp2f(m - msafe);
-      bf16x8 pa;
       float ps = 0.f;
 #pragma unroll
       for (int t = 0; t < 2; ++t)
@@ -326,6 +353,7 @@ __global__ __launch_bounds__(NW * 64) __attribute__((amdgpu_waves_per_eu(2))) vo
         const float f = __shfl(alpha, 4 * g + i, 64);
 #pragma unroll
         for (int nd = 0; nd < ND; ++nd) o[nd][i] *= f;
+      }
       }
 #pragma unroll
       for (int nd = 0; nd < ND; ++nd) o[nd] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pa, cur.v[nd], o[nd], 0, 0, 0);
@@ -356,7 +384,11 @@ __global__ __launch_bounds__(NW * 64) __attribute__((amdgpu_waves_per_eu(2))) vo
         if (np == 1) {
           const float inv = lh > 0.f ? 1.f / lh : 0.f;
 #pragma unroll
-          for (int nd = 0; nd < ND; ++nd) out[((long)b * Hq + hq) * DH + 16 * nd + r] = (bf16)(o[nd][i] * inv);
+          for (int nd = 0; nd < ND; ++nd) {
+            const int d = 16 * nd + r;
+            const float gf = E.gate ? gate_at(E, b, hq * DH + d) : 1.f;
+            out[((long)b * Hq + hq) * DH + d] = (bf16)(o[nd][i] * inv * gf);
+          }
         } else {
 #pragma unroll
           for (int nd = 0; nd < ND; ++nd) part_o[(((long)b * Hq + hq) * P + p) * DH + 16 * nd + r] = o[nd][i];
@@ -395,7 +427,8 @@ __global__ __launch_bounds__(NW * 64) __attribute__((amdgpu_waves_per_eu(2))) vo
     }
     const int hq = kvh * G + h;
     if (np == 1) {
-      out[((long)b * Hq + hq) * DH + d] = (bf16)(den > 0.f ? num / den : 0.f);
+      const float gf = E.gate ? gate_at(E, b, hq * DH + d) : 1.f;
+      out[((long)b * Hq + hq) * DH + d] = (bf16)(den > 0.f ? num / den * gf : 0.f);
     } else {
       part_o[(((long)b * Hq + hq) * P + p) * DH + d] = num;
       if (d == 0) {
@@ -455,7 +488,8 @@ __global__ __launch_bounds__(NW * 64) __attribute__((amdgpu_waves_per_eu(2))) vo
       for (int j = 0; j < 8; ++j)
         if (j0 + j < np) num += wts[(j0 + j) * G + h] * v[j];
     }
-    out[((long)b * Hq + kvh * G + h) * DH + d] = (bf16)(num * wts[np * G + h]);
+    const float gf = E.gate ? gate_at(E, b, (kvh * G + h) * DH + d) : 1.f;
+    out[((long)b * Hq + kvh * G + h) * DH + d] = (bf16)(num * wts[np * G + h] * gf);
   }
 }
 
@@ -468,7 +502,7 @@ __global__ __launch_bounds__(NW * 64) __attribute__((amdgpu_waves_per_eu(2))) vo
 constexpr int PF_T = 256;
 constexpr int PF_KT = 32;  // keys per tile
 
-template <int DH, bool DENSE = false>
+template <int DH, bool DENSE = false, bool SIG = false>
 __global__ __launch_bounds__(PF_T) void attn_prefill_kernel(
     const bf16* __restrict__ q, const bf16* __restrict__ kc, const bf16* __restrict__ vc,
     const int* __restrict__ tiles,          // [ntiles][2] = (seq, first query row within seq)
@@ -476,7 +510,7 @@ __global__ __launch_bounds__(PF_T) void attn_prefill_kernel(
     const int* __restrict__ ctx_lens,       // [nseq] total keys (cached + new)
     const int* __restrict__ block_tables, int max_blocks, int Hq, int Hkv, int BS, float scale,
     bf16* __restrict__ out, float cap, int window, long ldq = 0, long ldk = 0, long ldv = 0, long ldo = 0,
-    DecExtra E = DecExtra{nullptr, 0, nullptr}) {
+    DecExtra E = DecExtra{nullptr, 0, nullptr, nullptr, 0, nullptr, 0}) {
   constexpr int DP = (DH + 31) / 32 * 32;  // padded head dim for the MFMA k loop
   constexpr int KC = DP / 32;               // k-chunks of 32
   constexpr int ND = DP / 16;               // 16-wide output column tiles
@@ -517,13 +551,21 @@ __global__ __launch_bounds__(PF_T) void attn_prefill_kernel(
   for (int i = 0; i < 4; ++i) {   // a sink: the softmax state starts at (sink, 1) instead of (-inf, 0)
     mrow[i] = E.sink ? E.sink[h] * 1.4426950408889634f : -INFINITY;
     lrow[i] = E.sink ? 1.f : 0.f;
+    if constexpr (SIG) { mrow[i] = 0.f; lrow[i] = 1.f; }
   }
+  const float sig_l2 = SIG ? E.sig[h] * 1.4426950408889634f : 0.f;
 
   const float sl2 = scale * 1.4426950408889634f;
   const int last_row = min(qlen, r0 + 64) - 1;
   const int kend = DENSE ? L : min(L, pos0 + last_row + 1);  // exclusive
 
-  for (int k0 = 0; k0 < kend; k0 += PF_KT) {
+  // first key any row of the tile sees (the first row's: the bounds grow with the position)
+  int kbeg = 0;
+  if constexpr (!DENSE) {
+    if (window > 0) kbeg = max(kbeg, pos0 + r0 - window + 1);
+    if (E.chunk > 0) kbeg = max(kbeg, (pos0 + r0) / E.chunk * E.chunk);
+  }
+  for (int k0 = kbeg / PF_KT * PF_KT; k0 < kend; k0 += PF_KT) {
     __syncthreads();
     // stage the K tile (row-major) and the V^T tile ([d][key], copied from the transposed cache)
     for (int cidx = tid; cidx < PF_KT * (DP / 8); cidx += PF_T) {
@@ -596,10 +638,16 @@ __global__ __launch_bounds__(PF_T) void attn_prefill_kernel(
         v0 = fmaf(E.bias[(long)min(max(qpos - key0, 0), E.nbias - 1) * Hq + h], 1.4426950408889634f, v0);
         v1 = fmaf(E.bias[(long)min(max(qpos - key1, 0), E.nbias - 1) * Hq + h], 1.4426950408889634f, v1);
       }
-      const int wlo = window > 0 ? qpos - window + 1 : 0;
+      int wlo = window > 0 ? qpos - window + 1 : 0;
+      if (!DENSE && E.chunk > 0) wlo = max(wlo, qpos / E.chunk * E.chunk);
       const bool causal = !DENSE;
       if ((causal && key0 > qpos) || key0 >= kend || qr >= qlen || key0 < wlo) v0 = -INFINITY;
       if ((causal && key1 > qpos) || key1 >= kend || qr >= qlen || key1 < wlo) v1 = -INFINITY;
+      if constexpr (SIG) {   // weights of their own, no softmax; hidden keys: -inf, weight 0
+        ps[wave][(4 * fq + i) * VS + fr] = (bf16)(1.f / (1.f + exp2f(-(v0 + sig_l2))));
+        ps[wave][(4 * fq + i) * VS + 16 + fr] = (bf16)(1.f / (1.f + exp2f(-(v1 + sig_l2))));
+        continue;
+      }
       float mx = group_max<16>(fmaxf(v0, v1));
       const float mnew = fmaxf(mrow[i], mx);
       const float msafe = (mnew == -INFINITY) ? 0.f : mnew;
@@ -610,10 +658,12 @@ __global__ __launch_bounds__(PF_T) void attn_prefill_kernel(
       ps[wave][(4 * fq + i) * VS + fr] = (bf16)p0;
       ps[wave][(4 * fq + i) * VS + 16 + fr] = (bf16)p1;
     }
+    if constexpr (!SIG) {
 #pragma unroll
-    for (int nd = 0; nd < ND; ++nd)
+      for (int nd = 0; nd < ND; ++nd)
 #pragma unroll
-      for (int i = 0; i < 4; ++i) o[nd][i] *= alpha[i];
+        for (int i = 0; i < 4; ++i) o[nd][i] *= alpha[i];
+    }
     __syncthreads();
     // O += P V : A = P[16 q][32 keys], B = V[32 keys][16 d]
     const bf16x8 pa = *(const bf16x8*)(&ps[wave][fr * VS + 8 * fq]);
@@ -633,7 +683,10 @@ __global__ __launch_bounds__(PF_T) void attn_prefill_kernel(
 #pragma unroll
     for (int nd = 0; nd < ND; ++nd) {
       const int d = 16 * nd + fr;
-      if (d < DH) out[(long)(qbeg + qr) * ldo + (long)h * DH + d] = (bf16)(o[nd][i] * inv);
+      if (d < DH) {
+        const float gf = !DENSE && E.gate ? gate_at(E, qbeg + qr, h * DH + d) : 1.f;
+        out[(long)(qbeg + qr) * ldo + (long)h * DH + d] = (bf16)(o[nd][i] * inv * gf);
+      }
     }
   }
 }
@@ -655,7 +708,8 @@ extern "C" int la_attn_decode(const void* q, const void* kc, const void* vc, con
                               void* out, void* part_o, void* part_ml, void* tickets, const void* rope_p,
                               long rope_slab, int rope_S, const void* rope_bias, const int* pos, const int* slots,
                               const float* cos_sin, float softcap, int window, int nw, const float* dist_bias,
-                              int nbias, const float* sink, void* stream) {
+                              int nbias, const float* sink, const float* sig, int chunk, const void* gate, long ldg,
+                              void* stream) {
   // nw bit 8: split even short sequences over the grid's partitions (few sequences: the
   // parallelism is worth the merge); otherwise a sequence of <= DEC_ONE_PART keys is one partition
   const int one_part = (nw & 256) ? 0 : g_dec_one_part;
@@ -668,8 +722,8 @@ extern "C" int la_attn_decode(const void* q, const void* kc, const void* vc, con
   if (rope_p && ((Dh & 31) || !pos || !slots || !cos_sin || rope_S < 0)) return -1;
   if (!rope_p && !q) return -1;
   const la::DecRope R{rope_p, rope_slab, rope_S, (const float*)rope_bias, pos, slots, cos_sin, (Hq + 2 * Hkv) * Dh};
-  if (dist_bias && nbias < 1) return -1;
-  const la::DecExtra E{dist_bias, nbias, sink};
+  if ((dist_bias && nbias < 1) || (sink && sig) || chunk < 0 || (gate && ldg < (long)Hq * Dh)) return -1;
+  const la::DecExtra E{dist_bias, nbias, sink, sig, chunk, (const bf16*)gate, ldg};
   const int G = Hq / Hkv;
   hipStream_t st = (hipStream_t)stream;
   dim3 grid(P, Hkv, B);
@@ -687,6 +741,24 @@ extern "C" int la_attn_decode(const void* q, const void* kc, const void* vc, con
   hipLaunchKernelGGL((la::attn_decode_kernel<D, GT, NW, V>), grid, dim3(NW * 64), 0, st, (const bf16*)q,        \
                      (const bf16*)kc, (const bf16*)vc, block_tables, max_blocks, seq_lens, Hkv, G, BS, sl2, PS,  \
                      (bf16*)out, po, pml, P, tk, R, cap_l2, cap_mul, window, one_part, E)
+  if (sig) {   // sigmoid weights: fewer instances (GT only sizes the cross-wave merge)
+#define DEC_SIG(D)                                             \
+  case D:                                                      \
+    if (G <= 4) {                                              \
+      if (nw == 1) DEC_LAUNCH(D, 4, 1, 4);                     \
+      else DEC_LAUNCH(D, 4, 4, 4);                             \
+    } else {                                                   \
+      if (nw == 1) DEC_LAUNCH(D, 16, 1, 4);                    \
+      else DEC_LAUNCH(D, 16, 4, 4);                            \
+    }                                                          \
+    break;
+    switch (Dh) {
+      DEC_SIG(64) DEC_SIG(80) DEC_SIG(96) DEC_SIG(128) DEC_SIG(192) DEC_SIG(256)
+      default: return -2;
+    }
+#undef DEC_SIG
+    return (int)hipGetLastError();
+  }
 #define DEC_NW(D, GT, NW)                                                  \
   do {                                                                     \
     if constexpr (D == 128 && GT == 4 && NW == 1) {                        \
@@ -752,15 +824,21 @@ extern "C" int la_attn_dense(const void* q, long ldq, const void* k, long ldk, c
 extern "C" int la_attn_prefill(const void* q, const void* kc, const void* vc, const int* tiles, int ntiles,
                                const int* cu_q, const int* ctx_lens, const int* block_tables, int max_blocks, int Hq,
                                int Hkv, int Dh, int BS, float scale, void* out, float softcap, int window,
-                               const float* dist_bias, int nbias, const float* sink, void* stream) {
-  if (Hq % Hkv || (dist_bias && nbias < 1)) return -1;
-  const la::DecExtra E{dist_bias, nbias, sink};
+                               const float* dist_bias, int nbias, const float* sink, const float* sig, int chunk,
+                               const void* gate, long ldg, void* stream) {
+  if (Hq % Hkv || (dist_bias && nbias < 1) || (sink && sig) || chunk < 0 || (gate && ldg < (long)Hq * Dh)) return -1;
+  const la::DecExtra E{dist_bias, nbias, sink, sig, chunk, (const bf16*)gate, ldg};
   hipStream_t st = (hipStream_t)stream;
   dim3 grid(ntiles, Hq);
-#define PF(D)                                                                                                     \
-  hipLaunchKernelGGL(la::attn_prefill_kernel<D>, grid, dim3(la::PF_T), 0, st, (const bf16*)q, (const bf16*)kc,    \
-                     (const bf16*)vc, tiles, cu_q, ctx_lens, block_tables, max_blocks, Hq, Hkv, BS, scale,       \
-                     (bf16*)out, softcap, window, 0L, 0L, 0L, 0L, E)
+#define PF_LAUNCH(D, SG)                                                                                          \
+  hipLaunchKernelGGL((la::attn_prefill_kernel<D, false, SG>), grid, dim3(la::PF_T), 0, st, (const bf16*)q,        \
+                     (const bf16*)kc, (const bf16*)vc, tiles, cu_q, ctx_lens, block_tables, max_blocks, Hq, Hkv,  \
+                     BS, scale, (bf16*)out, softcap, window, 0L, 0L, 0L, 0L, E)
+#define PF(D)                       \
+  do {                              \
+    if (sig) PF_LAUNCH(D, true);    \
+    else PF_LAUNCH(D, false);       \
+  } while (0)
   switch (Dh) {
     case 64: PF(64); break;
     case 80: PF(80); break;
@@ -771,5 +849,6 @@ extern "C" int la_attn_prefill(const void* q, const void* kc, const void* vc, co
     default: return -2;
   }
 #undef PF
+#undef PF_LAUNCH
   return (int)hipGetLastError();
 }

@@ -6,6 +6,11 @@
 //   visible j:   j <= i, same chunk of `chunk` positions (chunk 0: all), within `window` (0: all)
 //   o_h(i)     = gate_h(i) * sum_j softmax_j(s'_h(i, .)) v(j)              (gate null: 1)
 //
+// or, with a bias `sig` per head, without a softmax: the weight of a visible key is
+// sigmoid(s'_h(i, j) + sig_h), not normalised over the keys.  The same kernels do it with the running
+// maximum fixed at 0 and the running sum at 1 (counted by the first key split).  The gate is one
+// logit per (row, head), or one per output channel.
+//
 // The head mix couples all heads of a (query, key) pair, so one workgroup owns ONE query row with
 // every head: per tile of 64 keys it forms the H x 64 raw scores, mixes them through LDS, runs one
 // online-softmax step per head (a wave per head, a lane per key) and accumulates P.V with threads
@@ -57,8 +62,8 @@ __global__ __launch_bounds__(AM_NT) void attn_mix_rows_kernel(
     const AT* __restrict__ q, const AT* __restrict__ kc, const AT* __restrict__ vc, const int* __restrict__ row_seq,
     const int* __restrict__ pos, const int* __restrict__ bt, int maxb, int H, int G, int Dk, int Dv, int BS,
     float scale, float softcap, const float* __restrict__ slopes, const float* __restrict__ talk, int chunk,
-    int window, const AT* __restrict__ gate, int ldg, AT* __restrict__ out, const float* __restrict__ dbias, int nbias,
-    const float* __restrict__ sink) {
+    int window, const AT* __restrict__ gate, int ldg, int gch, AT* __restrict__ out, const float* __restrict__ dbias,
+    int nbias, const float* __restrict__ sink, const float* __restrict__ sig) {
   extern __shared__ float lds[];
   float* qs = lds;                       // [H][Dk]
   float* s1 = qs + H * Dk;               // [H][KT] raw scores
@@ -73,7 +78,11 @@ __global__ __launch_bounds__(AM_NT) void attn_mix_rows_kernel(
   const bool vec = (Dk * sizeof(AT)) % 16 == 0;
   for (int e = tid; e < H * Dk; e += AM_NT) qs[e] = (float)q[(long)r * H * Dk + e];
   // a sink is a logit without key or value: the running (max, sum) start at (sink, 1) instead of (-inf, 0)
-  for (int h = tid; h < H; h += AM_NT) { mrun[h] = sink ? sink[h] : -INFINITY; lrun[h] = sink ? 1.f : 0.f; }
+  for (int h = tid; h < H; h += AM_NT) {
+    mrun[h] = sink ? sink[h] : (sig ? 0.f : -INFINITY);
+    lrun[h] = sink || sig ? 1.f : 0.f;
+    if (sig) alpha[h] = 1.f;
+  }
   int lo = 0;
   if (chunk > 0) lo = (i / chunk) * chunk;
   if (window > 0) lo = max(lo, i - window + 1);
@@ -116,6 +125,10 @@ __global__ __launch_bounds__(AM_NT) void attn_mix_rows_kernel(
     for (int h = tid >> 6; h < H; h += AM_NT / 64) {
       const int lane = tid & 63;
       const float s = s2[h * AM_KT + lane];
+      if (sig) {
+        s2[h * AM_KT + lane] = 1.f / (1.f + expf(-(s + sig[h])));   // hidden keys: s = -inf, weight 0
+        continue;
+      }
       const float mo = mrun[h];
       const float mn = fmaxf(mo, wave_max(s));
       const float p = (s == -INFINITY) ? 0.f : __expf(s - mn);
@@ -158,7 +171,7 @@ __global__ __launch_bounds__(AM_NT) void attn_mix_rows_kernel(
     if (o < HV) {
       const int h = o / Dv;
       float v = acc[e] / lrun[h];
-      if (gate) v *= 1.f / (1.f + __expf(-(float)gate[(long)r * ldg + h]));
+      if (gate) v *= 1.f / (1.f + expf(-(float)gate[(long)r * ldg + (gch ? o : h)]));
       out[(long)r * HV + o] = (AT)v;
     }
   }
@@ -189,8 +202,9 @@ __global__ __launch_bounds__(NW * 64) void attn_mix_tile_kernel(
     const int* __restrict__ tiles, const int* __restrict__ cu_q, const int* __restrict__ pos,
     const int* __restrict__ bt, int maxb, int H, int G, int Dk, int Dv, int BS, float scale, float softcap,
     const float* __restrict__ slopes, const float* __restrict__ talk, int chunk, int window,
-    const bf16* __restrict__ gate, int ldg, bf16* __restrict__ out, int nsplit, float* __restrict__ part_o,
-    float* __restrict__ part_ml, const float* __restrict__ dbias, int nbias, const float* __restrict__ sink) {
+    const bf16* __restrict__ gate, int ldg, int gch, bf16* __restrict__ out, int nsplit, float* __restrict__ part_o,
+    float* __restrict__ part_ml, const float* __restrict__ dbias, int nbias, const float* __restrict__ sink,
+    const float* __restrict__ sig) {
   extern __shared__ float lds[];
   float* s1 = lds;                           // [H][16][AT_SS]
   float* mrun = s1 + H * 16 * AT_SS;         // [H * 16]
@@ -208,7 +222,11 @@ __global__ __launch_bounds__(NW * 64) void attn_mix_tile_kernel(
   const int rep = H / G, KC = Dk / 32;
   // sink: a logit without key or value, counted once per (head, query) -- by the first key split
   const bool sunk = sink != nullptr && blockIdx.y == 0;
-  for (int e = tid; e < H * 16; e += NW * 64) { mrun[e] = sunk ? sink[e >> 4] : -INFINITY; lrun[e] = sunk ? 1.f : 0.f; }
+  for (int e = tid; e < H * 16; e += NW * 64) {
+    mrun[e] = sunk ? sink[e >> 4] : (sig ? 0.f : -INFINITY);
+    lrun[e] = sunk || (sig && blockIdx.y == 0) ? 1.f : 0.f;
+    if (sig) alpha[e] = 1.f;
+  }
   f32x4 o[HPW][NDV];
 #pragma unroll
   for (int a = 0; a < HPW; ++a)
@@ -379,6 +397,13 @@ __global__ __launch_bounds__(NW * 64) void attn_mix_tile_kernel(
     for (int r = tid; r < H * 16; r += NW * 64) {
       if ((r & 15) >= nrow) continue;            // rows past the portion's end (decode: 15 of 16)
       const float* sr = s1 + r * AT_SS;
+      if (sig) {                                 // weights of their own, no softmax; hidden keys: -inf, weight 0
+        const float sb = sig[r >> 4];
+        bf16* pr = pb + r * AT_PS;
+#pragma unroll 8
+        for (int k = 0; k < AT_KT; ++k) pr[k] = (bf16)(1.f / (1.f + __expf(-(sr[k] + sb))));
+        continue;
+      }
       float mx = -INFINITY;
 #pragma unroll 8
       for (int k = 0; k < AT_KT; ++k) mx = fmaxf(mx, sr[k]);
@@ -466,11 +491,16 @@ __global__ __launch_bounds__(NW * 64) void attn_mix_tile_kernel(
       }
       const float l = lrun[h * 16 + qr];
       float f = l > 0.f ? 1.f / l : 0.f;
-      if (gate) f *= 1.f / (1.f + __expf(-(float)gate[(long)(row0 + qr) * ldg + h]));
+      const bf16* gr = gate ? gate + (long)(row0 + qr) * ldg : nullptr;
+      if (gr && !gch) f *= 1.f / (1.f + __expf(-(float)gr[h]));
 #pragma unroll
       for (int nd = 0; nd < NDV; ++nd) {
         const int d = 16 * nd + fr;
-        if (d < Dv) out[((long)(row0 + qr) * H + h) * Dv + d] = (bf16)(o[hi][nd][i] * f);
+        if (d < Dv) {
+          float v = o[hi][nd][i] * f;
+          if (gr && gch) v *= 1.f / (1.f + __expf(-(float)gr[h * Dv + d]));
+          out[((long)(row0 + qr) * H + h) * Dv + d] = (bf16)v;
+        }
       }
     }
   }
@@ -479,7 +509,7 @@ __global__ __launch_bounds__(NW * 64) void attn_mix_tile_kernel(
 // out[row][h][d] = gate * sum_s o_s e^(m_s - M) / sum_s l_s e^(m_s - M) over the key splits
 __global__ __launch_bounds__(128) void attn_mix_merge_kernel(const float* __restrict__ part_o,
                                                              const float* __restrict__ part_ml, int nsplit, int H, int Dv,
-                                                             const bf16* __restrict__ gate, int ldg,
+                                                             const bf16* __restrict__ gate, int ldg, int gch,
                                                              bf16* __restrict__ out) {
   const int row = blockIdx.x, h = blockIdx.y;
   const long base = ((long)row * H + h) * nsplit;
@@ -491,14 +521,16 @@ __global__ __launch_bounds__(128) void attn_mix_merge_kernel(const float* __rest
     if (m != -INFINITY) L = fmaf(part_ml[2 * (base + s) + 1], __expf(m - M), L);
   }
   float f = L > 0.f ? 1.f / L : 0.f;
-  if (gate) f *= 1.f / (1.f + __expf(-(float)gate[(long)row * ldg + h]));
+  if (gate && !gch) f *= 1.f / (1.f + __expf(-(float)gate[(long)row * ldg + h]));
   for (int d = threadIdx.x; d < Dv; d += 128) {
     float acc = 0.f;
     for (int s = 0; s < nsplit; ++s) {
       const float m = part_ml[2 * (base + s)];
       if (m != -INFINITY) acc = fmaf(part_o[(base + s) * Dv + d], __expf(m - M), acc);
     }
-    out[((long)row * H + h) * Dv + d] = (bf16)(acc * f);
+    acc *= f;
+    if (gate && gch) acc *= 1.f / (1.f + __expf(-(float)gate[(long)row * ldg + h * Dv + d]));
+    out[((long)row * H + h) * Dv + d] = (bf16)acc;
   }
 }
 
@@ -506,14 +538,15 @@ template <int NW, int HPW, int NDV>
 static int launch_tile(int nsplit, void* part_o, void* part_ml, int ntiles, size_t shm, hipStream_t s, const void* q, const void* kc, const void* vc,
                        const void* tiles, const void* cu_q, const void* pos, const void* bt, int maxb, int H, int G,
                        int Dk, int Dv, int BS, float scale, float softcap, const void* slopes, const void* talk,
-                       int chunk, int window, const void* gate, int ldg, void* out, const void* dbias, int nbias,
-                       const void* sink) {
+                       int chunk, int window, const void* gate, int ldg, int gch, void* out, const void* dbias, int nbias,
+                       const void* sink, const void* sig) {
   auto k = attn_mix_tile_kernel<NW, HPW, NDV>;
   if (shm > 48 * 1024) (void)hipFuncSetAttribute((const void*)k, hipFuncAttributeMaxDynamicSharedMemorySize, (int)shm);
   hipLaunchKernelGGL(k, dim3(ntiles, nsplit), dim3(NW * 64), shm, s, (const bf16*)q, (const bf16*)kc, (const bf16*)vc,
                      (const int*)tiles, (const int*)cu_q, (const int*)pos, (const int*)bt, maxb, H, G, Dk, Dv, BS, scale,
-                     softcap, (const float*)slopes, (const float*)talk, chunk, window, (const bf16*)gate, ldg,
-                     (bf16*)out, nsplit, (float*)part_o, (float*)part_ml, (const float*)dbias, nbias, (const float*)sink);
+                     softcap, (const float*)slopes, (const float*)talk, chunk, window, (const bf16*)gate, ldg, gch,
+                     (bf16*)out, nsplit, (float*)part_o, (float*)part_ml, (const float*)dbias, nbias, (const float*)sink,
+                     (const float*)sig);
   return (int)hipGetLastError();
 }
 
@@ -522,10 +555,10 @@ static int launch_tile(int nsplit, void* part_o, void* part_ml, int ntiles, size
 extern "C" int la_attn_mix_rows(int f32, const void* q, const void* kc, const void* vc, const void* row_seq,
                                 const void* pos, const void* bt, int maxb, int T, int H, int G, int Dk, int Dv, int BS,
                                 float scale, float softcap, const void* slopes, const void* talk, int chunk, int window,
-                                const void* gate, int ldg, void* out, const void* dbias, int nbias, const void* sink,
-                                void* stream) {
+                                const void* gate, int ldg, int gch, void* out, const void* dbias, int nbias,
+                                const void* sink, const void* sig, void* stream) {
   using namespace la;
-  if (T <= 0 || H <= 0 || G <= 0 || H % G || H * Dv > AM_NT * AM_MAXO || (dbias && nbias < 1)) return -1;
+  if (T <= 0 || H <= 0 || G <= 0 || H % G || H * Dv > AM_NT * AM_MAXO || (dbias && nbias < 1) || (sink && sig)) return -1;
   const size_t shm = sizeof(float) * ((size_t)H * Dk + 2 * (size_t)H * AM_KT + 3 * (size_t)H);
   if (shm > 160 * 1024) return -2;
   hipStream_t s = (hipStream_t)stream;
@@ -534,15 +567,15 @@ extern "C" int la_attn_mix_rows(int f32, const void* q, const void* kc, const vo
       (void)hipFuncSetAttribute((const void*)attn_mix_rows_kernel<float>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)shm);
     hipLaunchKernelGGL((attn_mix_rows_kernel<float>), dim3(T), dim3(AM_NT), shm, s, (const float*)q, (const float*)kc,
                        (const float*)vc, (const int*)row_seq, (const int*)pos, (const int*)bt, maxb, H, G, Dk, Dv, BS,
-                       scale, softcap, (const float*)slopes, (const float*)talk, chunk, window, (const float*)gate, ldg,
-                       (float*)out, (const float*)dbias, nbias, (const float*)sink);
+                       scale, softcap, (const float*)slopes, (const float*)talk, chunk, window, (const float*)gate, ldg, gch,
+                       (float*)out, (const float*)dbias, nbias, (const float*)sink, (const float*)sig);
   } else {
     if (shm > 48 * 1024)
       (void)hipFuncSetAttribute((const void*)attn_mix_rows_kernel<bf16>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)shm);
     hipLaunchKernelGGL((attn_mix_rows_kernel<bf16>), dim3(T), dim3(AM_NT), shm, s, (const bf16*)q, (const bf16*)kc,
                        (const bf16*)vc, (const int*)row_seq, (const int*)pos, (const int*)bt, maxb, H, G, Dk, Dv, BS,
-                       scale, softcap, (const float*)slopes, (const float*)talk, chunk, window, (const bf16*)gate, ldg,
-                       (bf16*)out, (const float*)dbias, nbias, (const float*)sink);
+                       scale, softcap, (const float*)slopes, (const float*)talk, chunk, window, (const bf16*)gate, ldg, gch,
+                       (bf16*)out, (const float*)dbias, nbias, (const float*)sink, (const float*)sig);
   }
   return (int)hipGetLastError();
 }
@@ -556,11 +589,12 @@ extern "C" int la_attn_mix_rows(int f32, const void* q, const void* kc, const vo
 extern "C" int la_attn_mix_tiles(const void* q, const void* kc, const void* vc, const void* tiles, int ntiles,
                                  const void* cu_q, const void* pos, const void* bt, int maxb, int H, int G, int Dk,
                                  int Dv, int BS, float scale, float softcap, const void* slopes, const void* talk,
-                                 int chunk, int window, const void* gate, int ldg, void* out, int nsplit, void* part_o,
-                                 void* part_ml, int rows, const void* dbias, int nbias, const void* sink, void* stream) {
+                                 int chunk, int window, const void* gate, int ldg, int gch, void* out, int nsplit,
+                                 void* part_o, void* part_ml, int rows, const void* dbias, int nbias, const void* sink,
+                                 const void* sig, void* stream) {
   using namespace la;
   if (ntiles <= 0 || H <= 0 || G <= 0 || H % G || nsplit < 1 || nsplit > 64 || (nsplit > 1 && (!part_o || !part_ml)) ||
-      (dbias && nbias < 1))
+      (dbias && nbias < 1) || (sink && sig))
     return -1;
   if ((Dk % 32) || (Dv % 16) || Dv > 128 || H > 32 || (BS & 7)) return 1;
   const size_t shm = (size_t)H * 16 * (AT_SS * 4 + 3 * 4 + AT_PS * 2);
@@ -572,14 +606,14 @@ extern "C" int la_attn_mix_tiles(const void* q, const void* kc, const void* vc, 
 #define LA_TILE(NW, HPW, NDV)                                                                                      \
   if (rc == 1 && nw == NW && hpw <= HPW && ndv == NDV)                                                             \
     rc = launch_tile<NW, HPW, NDV>(nsplit, part_o, part_ml, ntiles, shm, s, q, kc, vc, tiles, cu_q, pos, bt, maxb, H, \
-                                   G, Dk, Dv, BS, scale, softcap, slopes, talk, chunk, window, gate, ldg, out, dbias,    \
-                                   nbias, sink);
+                                   G, Dk, Dv, BS, scale, softcap, slopes, talk, chunk, window, gate, ldg, gch, out,       \
+                                   dbias, nbias, sink, sig);
   LA_TILE(4, 1, 2) LA_TILE(4, 1, 4) LA_TILE(4, 1, 8) LA_TILE(4, 2, 2) LA_TILE(4, 2, 4) LA_TILE(4, 2, 8)
   LA_TILE(8, 2, 2) LA_TILE(8, 2, 4) LA_TILE(8, 2, 8) LA_TILE(8, 4, 2) LA_TILE(8, 4, 4) LA_TILE(8, 4, 8)
 #undef LA_TILE
   if (rc == 0 && nsplit > 1) {
     hipLaunchKernelGGL(attn_mix_merge_kernel, dim3(rows, H), dim3(128), 0, s, (const float*)part_o, (const float*)part_ml,
-                       nsplit, H, Dv, (const bf16*)gate, ldg, (bf16*)out);
+                       nsplit, H, Dv, (const bf16*)gate, ldg, gch, (bf16*)out);
     rc = (int)hipGetLastError();
   }
   return rc;

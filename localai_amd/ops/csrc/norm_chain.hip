@@ -4,7 +4,7 @@
 //   norm_chain:  res <- (replace ? 0 : res) + post(branch) + add_vec;  out = pre(res)
 //       post:  none | dyt: tanh(alpha y) * w + b | rms: y / sqrt(mean(y^2) + eps) * w
 //              | ln: (y - mean) / sqrt(mean((y - mean)^2) + eps) * w  (layer norm, no bias)
-//       pre:   none | dyt | cast (the stream itself in the output type) | ln (eps in the alpha slot)
+//       pre:   none | dyt | cast (the stream itself in the output type) | ln, rms (eps in the alpha slot)
 //     one launch where a pre-normed stream has "add + norm": the branch's own norm, the residual
 //     add and the next sublayer's input norm.  A workgroup per row; the rms variant reads the
 //     branch row twice (second time from cache) instead of holding it in registers, so any width runs.
@@ -12,6 +12,10 @@
 //     the boundary of a pre-normed fp32 stream whose norm works on groups
 //   poly_norm_act:   y = a z / rms(z) + b z^2 / rms(z^2) + c z^3 / rms(z^3) + e over a row
 //   sigmoid_mul:     x * sigmoid(gate), the gate being columns of a wider row
+//   stream_conv: res <- res + post(branch) (post: none or rms), h_t = res_t + sum_j w[j] res_(t - taps + 1 + j): a
+//     depthwise causal convolution on the stream itself, its tail of taps - 1 fp32 rows per sequence in a
+//     state slot, the sum handed to the next sublayer in its type
+//   glu_act:     act(gate) * up, act = silu or the tanh form of gelu; any width, bf16 or fp32
 //   glu_clamp:   g = min(gate, limit), u = clamp(up, -limit, limit), y = g sigmoid(slope g) (u + 1)
 //   side_gate:   gelu_tanh(z[t][c]) * table[tok[t]][col0 + c]
 //
@@ -84,10 +88,13 @@ __global__ __launch_bounds__(NC_NT) void norm_chain_kernel(float* __restrict__ r
     if (pre == NC_DYT) put(out, out_f32, base + c, fmaf(tanhf(qa * x), qw[c], qb[c]));
     else if (pre == NC_CAST) put(out, out_f32, base + c, x);
   }
-  if (pre == NC_LN) {   // layer norm of the updated row: every thread re-reads the columns it wrote
-    float sm = 0.f;
-    for (int c = tid; c < D; c += NC_NT) sm += res[base + c];
-    const float m2 = block_sum<NC_NT>(sm, red) / (float)D;
+  if (pre == NC_LN || pre == NC_RMS) {   // norm of the updated row: every thread re-reads the columns it wrote
+    float m2 = 0.f;
+    if (pre == NC_LN) {
+      float sm = 0.f;
+      for (int c = tid; c < D; c += NC_NT) sm += res[base + c];
+      m2 = block_sum<NC_NT>(sm, red) / (float)D;
+    }
     float ss = 0.f;
     for (int c = tid; c < D; c += NC_NT) {
       const float d = res[base + c] - m2;
@@ -166,13 +173,16 @@ __global__ __launch_bounds__(NC_NT) void norm_chain4_kernel(float* __restrict__ 
       }
     }
   }
-  if (pre == NC_LN) {   // layer norm of the updated row: every thread re-reads the columns it wrote
-    float sm = 0.f;
-    for (int c = tid * 4; c < D; c += NC_NT * 4) {
-      const float4 v = *(const float4*)(res + base + c);
-      sm += (v.x + v.y) + (v.z + v.w);
+  if (pre == NC_LN || pre == NC_RMS) {   // norm of the updated row: every thread re-reads the columns it wrote
+    float m2 = 0.f;
+    if (pre == NC_LN) {
+      float sm = 0.f;
+      for (int c = tid * 4; c < D; c += NC_NT * 4) {
+        const float4 v = *(const float4*)(res + base + c);
+        sm += (v.x + v.y) + (v.z + v.w);
+      }
+      m2 = block_sum<NC_NT>(sm, red) / (float)D;
     }
-    const float m2 = block_sum<NC_NT>(sm, red) / (float)D;
     float ss = 0.f;
     for (int c = tid * 4; c < D; c += NC_NT * 4) {
       const float4 v = *(const float4*)(res + base + c);
@@ -190,6 +200,103 @@ __global__ __launch_bounds__(NC_NT) void norm_chain4_kernel(float* __restrict__ 
       }
     }
   }
+}
+
+// Convolution of the stream, a workgroup per row, V columns a thread.  wt: weights tap-major [taps][D].  Row t of
+// sequence seq sits m rows after its portion's start at position p: the stream d tokens back is row t - d of
+// the batch, or the tail's row taps - 1 - (d - m) ([taps - 1][D] of the sequence's slot: the rows before the
+// portion), or nothing before position 0.  SINGLE: every sequence brings one row; the branch's norm and the
+// residual add come first and the tail advances, all in one launch (each thread is the only reader and
+// writer of its columns of the row and of the slot).
+template <int V, bool SINGLE>
+__global__ __launch_bounds__(NC_NT) void stream_conv_kernel(float* __restrict__ res, int D, RowSrc src, int has_src, int post,
+                                                            const float* __restrict__ pw, float eps,
+                                                            const float* __restrict__ wt, int taps,
+                                                            const int* __restrict__ row_seq, const int* __restrict__ cu_q,
+                                                            const int* __restrict__ pos, const int* __restrict__ sslot,
+                                                            float* __restrict__ tail, void* __restrict__ out, int out_f32) {
+  typedef float fvec __attribute__((ext_vector_type(V)));
+  typedef bf16 bvec __attribute__((ext_vector_type(V)));
+  __shared__ float red[NC_NT / 64];
+  const int t = blockIdx.x, tid = threadIdx.x;
+  const long base = (long)t * D;
+  const int seq = SINGLE ? t : row_seq[t], m = SINGLE ? 0 : t - cu_q[seq], p = pos[t], ss = sslot[seq];
+  float* st = tail + (long)ss * (taps - 1) * D;
+  auto load = [&](int c) -> fvec {
+    fvec y;
+    if (V == 4 && src.S <= 1) {
+      if (src.f32) y = *(const fvec*)((const float*)src.p + base + c);
+      else {
+        const bvec b = *(const bvec*)((const bf16*)src.p + base + c);
+#pragma unroll
+        for (int j = 0; j < V; ++j) y[j] = (float)b[j];
+      }
+    } else {
+#pragma unroll
+      for (int j = 0; j < V; ++j) y[j] = src_at(src, base + c + j);
+    }
+    return y;
+  };
+  float inv = 1.f;
+  if (SINGLE && has_src && post == NC_RMS) {
+    float s2 = 0.f;
+    for (int c = tid * V; c < D; c += NC_NT * V) {
+      const fvec y = load(c);
+#pragma unroll
+      for (int j = 0; j < V; ++j) s2 = fmaf(y[j], y[j], s2);
+    }
+    inv = 1.f / sqrtf(block_sum<NC_NT>(s2, red) / (float)D + eps);
+  }
+  for (int c = tid * V; c < D; c += NC_NT * V) {
+    fvec x = *(const fvec*)(res + base + c);
+    if (SINGLE && has_src) {
+      const fvec y = load(c);
+#pragma unroll
+      for (int j = 0; j < V; ++j) x[j] += post == NC_RMS ? y[j] * inv * pw[c + j] : y[j];
+      *(fvec*)(res + base + c) = x;
+    }
+    fvec acc = {};
+    for (int i = 0; i + 1 < taps; ++i) {
+      const int d = taps - 1 - i;        // tokens back
+      fvec h = {};
+      if (d <= p) {
+        if (d <= m) h = *(const fvec*)(res + base - (long)d * D + c);
+        else if (ss >= 0) h = *(const fvec*)(st + (long)(taps - 1 - (d - m)) * D + c);
+      }
+      if (SINGLE && ss >= 0 && i > 0) *(fvec*)(st + (long)(i - 1) * D + c) = h;
+      const fvec w = *(const fvec*)(wt + (long)i * D + c);
+#pragma unroll
+      for (int j = 0; j < V; ++j) acc[j] = fmaf(w[j], h[j], acc[j]);
+    }
+    if (SINGLE && ss >= 0 && taps > 1) *(fvec*)(st + (long)(taps - 2) * D + c) = x;
+    const fvec w = *(const fvec*)(wt + (long)(taps - 1) * D + c);
+#pragma unroll
+    for (int j = 0; j < V; ++j) acc[j] = x[j] + fmaf(w[j], x[j], acc[j]);
+    if (out_f32) *(fvec*)((float*)out + base + c) = acc;
+    else {
+      bvec o;
+#pragma unroll
+      for (int j = 0; j < V; ++j) o[j] = (bf16)acc[j];
+      *(bvec*)((bf16*)out + base + c) = o;
+    }
+  }
+}
+
+int conv_tail_f32(const float* u, int ldp, int taps, int C, int nseq, const int* cu_q, const int* sslot, float* state,
+                  hipStream_t st);      // shortconv.hip
+
+// act(gate) * up of rows [gate | up]
+enum { GLU_SILU = 0, GLU_GELU_TANH = 1 };
+__global__ __launch_bounds__(256) void glu_act_kernel(RowSrc src, int F, long total, int mode, void* __restrict__ out,
+                                                      int out_f32) {
+  const long e = (long)blockIdx.x * 256 + threadIdx.x;
+  if (e >= total) return;
+  const long t = e / F;
+  const int c = (int)(e - t * F);
+  const float g = src_at(src, t * 2 * F + c), u = src_at(src, t * 2 * F + F + c);
+  const float a = mode == GLU_SILU ? g / (1.f + expf(-g))
+                                   : 0.5f * g * (1.f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g)));
+  put(out, out_f32, e, a * u);
 }
 
 __global__ __launch_bounds__(256) void glu_clamp_kernel(RowSrc src, int F, long total, float limit, float slope,
@@ -381,6 +488,43 @@ __global__ __launch_bounds__(256) void sigmoid_mul8_kernel(const bf16* __restric
 
 }  // namespace la
 
+// single: every sequence brings one row (cu_q and row_seq unused) -- the branch (sp, may be null) is added in
+// the same launch; otherwise sp must be null (la_norm_chain adds it) and a second launch advances the tails.
+extern "C" int la_stream_conv(void* res, int T, int D, const void* sp, int src_f32, long slab, int S, int post,
+                              const void* pw, float eps, const void* wt, int taps, int nseq, const void* row_seq,
+                              const void* cu_q, const void* pos, const void* sslot, void* tail, int single, void* out,
+                              int out_f32, void* stream) {
+  using namespace la;
+  if (T <= 0 || D <= 0 || taps < 1 || nseq <= 0 || !res || !wt || !pos || !sslot || !out || (taps > 1 && !tail)) return -1;
+  if (single ? nseq != T : (!row_seq || !cu_q || sp != nullptr)) return -2;
+  if (sp && ((post != NC_NONE && post != NC_RMS) || (post == NC_RMS && !pw) || (src_f32 && S < 1))) return -3;
+  RowSrc s{sp, src_f32, slab, S};
+  hipStream_t st = (hipStream_t)stream;
+#define LA_SCV(V, SG)                                                                                                  \
+  hipLaunchKernelGGL((stream_conv_kernel<V, SG>), dim3(T), dim3(NC_NT), 0, st, (float*)res, D, s, sp != nullptr, post, \
+                     (const float*)pw, eps, (const float*)wt, taps, (const int*)row_seq, (const int*)cu_q,             \
+                     (const int*)pos, (const int*)sslot, (float*)tail, out, out_f32)
+  if (single) {
+    if (!(D & 3)) LA_SCV(4, true); else LA_SCV(1, true);
+    return (int)hipGetLastError();
+  }
+  if (!(D & 3)) LA_SCV(4, false); else LA_SCV(1, false);
+#undef LA_SCV
+  if (taps > 1) return conv_tail_f32((const float*)res, D, taps, D, nseq, (const int*)cu_q, (const int*)sslot, (float*)tail, st);
+  return (int)hipGetLastError();
+}
+
+extern "C" int la_glu_act(const void* sp, int src_f32, long slab, int S, int T, int F, int mode, void* out, int out_f32,
+                          void* stream) {
+  using namespace la;
+  if (T <= 0 || F <= 0 || !sp || !out || (src_f32 && S < 1) || (mode != GLU_SILU && mode != GLU_GELU_TANH)) return -1;
+  RowSrc s{sp, src_f32, slab, S};
+  const long total = (long)T * F;
+  hipLaunchKernelGGL(glu_act_kernel, dim3((unsigned)((total + 255) / 256)), dim3(256), 0, (hipStream_t)stream, s, F, total,
+                     mode, out, out_f32);
+  return (int)hipGetLastError();
+}
+
 extern "C" int la_add_group_norm(void* res, int T, int D, const void* sp, int src_f32, long slab, int S, const void* w,
                                  float eps, int groups, void* out, int out_f32, void* stream) {
   using namespace la;
@@ -436,7 +580,7 @@ extern "C" int la_norm_chain(void* res, int T, int D, const void* sp, int src_f3
   if (post == NC_DYT && (!pw || !pb)) return -2;
   if ((post == NC_RMS || post == NC_LN) && !pw) return -2;
   if (pre == NC_DYT && (!qw || !qb)) return -2;
-  if (pre == NC_LN && !qw) return -2;
+  if ((pre == NC_LN || pre == NC_RMS) && !qw) return -2;
   if (pre != NC_NONE && !out) return -3;
   const int has = sp != nullptr;
   if (has && src_f32 && S < 1) return -4;

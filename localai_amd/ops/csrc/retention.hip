@@ -22,6 +22,10 @@
 // whose q / k rows are shared by groups of heads (state-space mixers, mamba2.hip):
 //   S_t = a_(t,h) S_(t-1) + k_(t,g) (s_(t,h) v_(t,h))^T,   o_t = S_t^T q_(t,g)
 // with a (tok_dec) and s (tok_vs) fp32 per (token, head) and Gqk groups; la::decay_scan_f32 is that entry.
+//
+// Lightning attention (la_lightning) is the scan with a fixed decay per head over q | k | v projection
+// rows without rotation or key scale, each passed through silu as the scan stages it (no prepared q | k
+// rows: qk null); lightning_out_kernel then norms the row of all heads together and applies the gate.
 #include "common.h"
 
 namespace la {
@@ -31,6 +35,9 @@ constexpr int RT_TC = 16;     // tokens staged per chunk
 constexpr int RT_SEG = 128;   // rows per segment of a segmented portion
 constexpr int RT_JOIN_MAXSEG = 1024;   // segments of one portion the join holds decay products for
 enum { RT_WHOLE = 0, RT_LOCAL = 1, RT_FINAL = 2 };
+
+template <typename T>
+LA_DEV float silu_f(T x) { return (float)x / (1.f + expf(-(float)x)); }
 
 // qk[t][0][h][d] = rotated q, qk[t][1][h][d] = rotated k * kscale (fp32): a thread per (row, head, pair or plain dim)
 template <typename AT>
@@ -122,7 +129,11 @@ __global__ __launch_bounds__(RT_NT) void retention_scan_kernel(
     for (int e = tid; e < n * DkP; e += RT_NT) {
       const int tt = e / DkP, d = e - tt * DkP;
       float qv = 0.f, kv = 0.f;
-      if (d < Dk) {
+      if (d < Dk && !qk) {                 // projection rows [q (Gqk x Dk) | k | v | ...], silu on each
+        const AT* row = src + (long)(t0 + tt) * ld + (long)g * Dk + d;
+        if (EMIT) qv = silu_f(row[0]);
+        kv = silu_f(row[(long)Gqk * Dk]);
+      } else if (d < Dk) {
         const float* row = qk + ((long)(t0 + tt) * 2 * Gqk + g) * Dk + d;
         if (EMIT) qv = row[0];
         kv = row[(long)Gqk * Dk];
@@ -133,6 +144,7 @@ __global__ __launch_bounds__(RT_NT) void retention_scan_kernel(
     for (int e = tid; e < n * cpw; e += RT_NT) {
       const int tt = e / cpw, cc = e - tt * cpw;
       float v = (c0 + cc < Dv) ? (float)src[(long)(t0 + tt) * ld + vcol + c0 + cc] : 0.f;
+      if (!qk) v = silu_f(v);
       if (tok_vs) v *= tok_vs[(long)(t0 + tt) * ldtok + h];
       vs[e] = v;
     }
@@ -247,8 +259,54 @@ __global__ __launch_bounds__(256) void retention_out_kernel(const float* __restr
   }
 }
 
+// out[t] = o[t] / sqrt(mean over all N = H Dv columns + eps) * w * sigmoid(gate[t]): a workgroup per token.
+// Rows of up to 8 KEEP values a thread stay in registers between the two passes; 4-wide where N and the rows allow
+template <typename AT, int V>
+__global__ __launch_bounds__(RT_NT) void lightning_out_kernel(const float* __restrict__ o, const AT* __restrict__ src,
+                                                              long ld, long gcol, int N, const float* __restrict__ w,
+                                                              float eps, AT* __restrict__ out) {
+  typedef float fvec __attribute__((ext_vector_type(V)));
+  typedef AT avec __attribute__((ext_vector_type(V)));
+  __shared__ float red[RT_NT / 64];
+  constexpr int KEEP = 4;
+  const int t = blockIdx.x, tid = threadIdx.x;
+  const float* orow = o + (long)t * N;
+  const AT* grow = src + t * ld + gcol;
+  fvec held[KEEP];
+  float ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < KEEP; ++k) {
+    const int c = (tid + k * RT_NT) * V;
+    if (c < N) {
+      held[k] = *(const fvec*)(orow + c);
+#pragma unroll
+      for (int j = 0; j < V; ++j) ss = fmaf(held[k][j], held[k][j], ss);
+    }
+  }
+  for (int c = (tid + KEEP * RT_NT) * V; c < N; c += RT_NT * V) {
+    const fvec x = *(const fvec*)(orow + c);
+#pragma unroll
+    for (int j = 0; j < V; ++j) ss = fmaf(x[j], x[j], ss);
+  }
+  const float inv = 1.f / sqrtf(block_sum<RT_NT>(ss, red) / (float)N + eps);
+  auto emit = [&](int c, const fvec& x) {
+    const avec g = *(const avec*)(grow + c);
+    const fvec wv = *(const fvec*)(w + c);
+    avec y;
+#pragma unroll
+    for (int j = 0; j < V; ++j) y[j] = (AT)(x[j] * inv * wv[j] / (1.f + expf(-(float)g[j])));
+    *(avec*)(out + (long)t * N + c) = y;
+  };
+#pragma unroll
+  for (int k = 0; k < KEEP; ++k) {
+    const int c = (tid + k * RT_NT) * V;
+    if (c < N) emit(c, held[k]);
+  }
+  for (int c = (tid + KEEP * RT_NT) * V; c < N; c += RT_NT * V) emit(c, *(const fvec*)(orow + c));
+}
+
 // The scan over prepared rows: v from src (row stride ld, head h at column vcol0 + h Dv), q | k rows
-// fp32 [T][2][Gqk][Dk], a fixed decay per head or tok_dec / tok_vs per (token, head) (row stride ldtok).
+// fp32 [T][2][Gqk][Dk] (null: the leading columns of src, through silu), a fixed decay per head or tok_dec / tok_vs per (token, head) (row stride ldtok).
 template <typename AT>
 static int scan_core(const AT* src, int ld, long vcol0, int T, int nseq, int H, int Gqk, int Dk, int Dv, const int* pos,
                      const int* cu_q, const int* sslots, float* state, const float* decay, const float* tok_dec,
@@ -334,7 +392,44 @@ int decay_scan_f32(const float* v, int ldv, const float* qk, int T, int nseq, in
                           qk, o, seg, max_rows > 0 ? max_rows : T, st);
 }
 
+template <typename AT>
+static int launch_lightning(const AT* src, int ld, int T, int nseq, int H, int Dk, int Dv, const int* pos, const int* cu_q,
+                            const int* sslots, float* state, const float* decay, const float* w, float eps, float* o,
+                            AT* out, float* seg, int max_rows, hipStream_t st) {
+  const int rc = scan_core<AT>(src, ld, 2L * H * Dk, T, nseq, H, H, Dk, Dv, pos, cu_q, sslots, state, decay, nullptr,
+                               nullptr, 0, nullptr, o, seg, max_rows, st);
+  if (rc) return rc;
+  const int N = H * Dv;
+  const long gcol = 2L * H * Dk + N;
+  if (!(N & 3) && !(ld & 3) && !(gcol & 3) && !(((uintptr_t)src | (uintptr_t)out) & 15))
+    hipLaunchKernelGGL((lightning_out_kernel<AT, 4>), dim3(T), dim3(RT_NT), 0, st, (const float*)o, src, (long)ld, gcol, N,
+                       w, eps, out);
+  else
+    hipLaunchKernelGGL((lightning_out_kernel<AT, 1>), dim3(T), dim3(RT_NT), 0, st, (const float*)o, src, (long)ld, gcol, N,
+                       w, eps, out);
+  return (int)hipGetLastError();
+}
+
 }  // namespace la
+
+// src rows [q (H Dk) | k (H Dk) | v (H Dv) | gate (H Dv)], row stride ld; o [T][H Dv] fp32 scratch; w [H Dv];
+// seg as in la_retention
+extern "C" int la_lightning(int f32, const void* src, int ld, int T, int nseq, int H, int Dk, int Dv, const void* pos,
+                            const void* cu_q, const void* sslots, void* state, int nslots, const void* decay, const void* w,
+                            float eps, void* o, void* out, void* seg, int max_rows, void* stream) {
+  using namespace la;
+  if (T <= 0 || nseq <= 0 || H <= 0 || Dk <= 0 || Dv <= 0 || nslots <= 0 || ld < 2 * H * (Dk + Dv)) return -1;
+  if (!src || !pos || !cu_q || !sslots || !state || !decay || !w || !o || !out) return -2;
+  if (max_rows <= 0) max_rows = T;
+  hipStream_t st = (hipStream_t)stream;
+  if (f32)
+    return launch_lightning<float>((const float*)src, ld, T, nseq, H, Dk, Dv, (const int*)pos, (const int*)cu_q,
+                                   (const int*)sslots, (float*)state, (const float*)decay, (const float*)w, eps, (float*)o,
+                                   (float*)out, (float*)seg, max_rows, st);
+  return launch_lightning<bf16>((const bf16*)src, ld, T, nseq, H, Dk, Dv, (const int*)pos, (const int*)cu_q,
+                                (const int*)sslots, (float*)state, (const float*)decay, (const float*)w, eps, (float*)o,
+                                (bf16*)out, (float*)seg, max_rows, st);
+}
 
 extern "C" int la_retention(int f32, const void* src, int T, int nseq, int H, int Dk, int Dv, const void* pos,
                             const void* cu_q, const void* sslots, void* state, int nslots, const void* decay,

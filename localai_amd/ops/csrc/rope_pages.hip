@@ -13,6 +13,9 @@
 //   qk_norm_pages: no rotation: every query and key head divided by its root mean square (fp32,
 //                no weight), queries times a temperature 1 + coef ln(floor((pos + 1) / every) + 1);
 //                K / V appended as above.  A wave per head.
+//   qk_row_norm_rope_pages: q and k normed over the WHOLE projection (all heads together) with a
+//                weight per channel, rotated like rope_pages' half layout, q times a number per head; the
+//                values are the raw keys (before norm and rotation).
 //   sinusoid_add: additive positions on the fp32 stream, column 2i += sin(pos f_i), 2i + 1 += cos.
 //
 // A workgroup per token; the token's cos / sin are computed once into LDS.
@@ -231,6 +234,88 @@ __global__ __launch_bounds__(RP_NT) void qk_norm_rope_pages_kernel(
   }
 }
 
+// row [q (H x D) | k (G x D)] with row stride ld.  All H D query columns share one root mean square, all G D
+// key columns another; then the weights, the rotation and the head's number (queries).  K pages get the
+// result, V pages the raw key.  A unit is V neighbouring dims, or V pairs of the rotated span.
+template <typename AT, int V>
+__global__ __launch_bounds__(RP_NT) void qk_row_norm_rope_pages_kernel(
+    const AT* __restrict__ src, long ld, int H, int D, int G, const int* __restrict__ pos, const int* __restrict__ slots,
+    const float* __restrict__ qw, const float* __restrict__ kw, const float* __restrict__ hscale, float eps,
+    const float* __restrict__ freqs, int rot, AT* __restrict__ q_out, AT* __restrict__ kc, AT* __restrict__ vc, int BS) {
+  typedef AT avec __attribute__((ext_vector_type(V)));
+  extern __shared__ float cs[];          // [rot / 2][2]
+  __shared__ float red[2][RP_NT / 64];
+  const int t = blockIdx.x, tid = threadIdx.x;
+  const int Cq = H * D, Ck = G * D, half = rot >> 1;
+  const AT* row = src + (long)t * ld;
+  const int p = pos[t];
+  for (int i = tid; i < half; i += RP_NT) sincosf((float)p * freqs[i], &cs[2 * i + 1], &cs[2 * i]);
+  float sq = 0.f, sk = 0.f;
+  for (int c = tid * V; c < Cq + Ck; c += RP_NT * V) {   // V divides D: a unit never spans q and k
+    const avec x = *(const avec*)(row + c);
+    float a = 0.f;
+#pragma unroll
+    for (int j = 0; j < V; ++j) a = fmaf((float)x[j], (float)x[j], a);
+    if (c < Cq) sq += a; else sk += a;
+  }
+  sq = wave_sum(sq);
+  sk = wave_sum(sk);
+  if ((tid & 63) == 0) {
+    red[0][tid >> 6] = sq;
+    red[1][tid >> 6] = sk;
+  }
+  __syncthreads();
+  sq = sk = 0.f;
+#pragma unroll
+  for (int w = 0; w < RP_NT / 64; ++w) {
+    sq += red[0][w];
+    sk += red[1][w];
+  }
+  const float iq = 1.f / sqrtf(sq / (float)Cq + eps), ik = 1.f / sqrtf(sk / (float)Ck + eps);
+  const int slot = slots[t];
+  const int blk = slot >= 0 ? slot / BS : 0, off = slot >= 0 ? slot - blk * BS : 0;
+  const int pairs = half / V, per = pairs + (D - rot) / V;    // units per head
+  for (int e = tid; e < (H + G) * per; e += RP_NT) {
+    const int u = e / per, k = e - u * per;
+    const bool isq = u < H;
+    if (!isq && slot < 0) continue;
+    const int g = isq ? u : u - H;
+    const AT* x = isq ? row + (long)g * D : row + Cq + (long)g * D;
+    const float* w = (isq ? qw : kw) + (long)g * D;
+    const float f = isq ? iq * (hscale ? hscale[g] : 1.f) : ik;
+    AT* dst = isq ? q_out + (long)t * Cq + (long)g * D : kc + (((long)blk * G + g) * BS + off) * D;
+    AT* vd = isq ? nullptr : vc + (((long)blk * G + g) * (BS >> 3) + (off >> 3)) * D * 8 + (off & 7);
+    if (k < pairs) {
+      const int d = k * V;
+      const avec a = *(const avec*)(x + d), b = *(const avec*)(x + d + half);
+      avec ya, yb;
+#pragma unroll
+      for (int j = 0; j < V; ++j) {
+        const float c = cs[2 * (d + j)], sn = cs[2 * (d + j) + 1];
+        const float av = (float)a[j] * f * w[d + j], bv = (float)b[j] * f * w[d + half + j];
+        ya[j] = (AT)(av * c - bv * sn);
+        yb[j] = (AT)(bv * c + av * sn);
+        if (vd) {
+          vd[(d + j) * 8] = a[j];
+          vd[(d + half + j) * 8] = b[j];
+        }
+      }
+      *(avec*)(dst + d) = ya;
+      *(avec*)(dst + d + half) = yb;
+    } else {
+      const int d = rot + (k - pairs) * V;
+      const avec a = *(const avec*)(x + d);
+      avec ya;
+#pragma unroll
+      for (int j = 0; j < V; ++j) {
+        ya[j] = (AT)((float)a[j] * f * w[d + j]);
+        if (vd) vd[(d + j) * 8] = a[j];
+      }
+      *(avec*)(dst + d) = ya;
+    }
+  }
+}
+
 // every head of a row turned over its whole width, dims m and m + Dv / 2 by sign * pos * freqs[m], times scale
 template <typename AT>
 __global__ __launch_bounds__(RP_NT) void rotate_heads_kernel(const AT* __restrict__ x, int H, int Dv,
@@ -273,6 +358,27 @@ extern "C" int la_qk_norm_rope_pages(int f32, const void* src, long ld, int T, i
     hipLaunchKernelGGL(qk_norm_rope_pages_kernel<bf16>, dim3(T), dim3(RP_NT), shm, (hipStream_t)stream, (const bf16*)src, ld,
                        H, D, G, Dv, (const int*)pos, (const int*)slots, (const float*)qw, (const float*)kw, eps,
                        (const float*)freqs, mag, rot, (const float*)vfreqs, (bf16*)q_out, (bf16*)kc, (bf16*)vc, BS);
+  return (int)hipGetLastError();
+}
+
+extern "C" int la_qk_row_norm_rope_pages(int f32, const void* src, long ld, int T, int H, int D, int G, const void* pos,
+                                         const void* slots, const void* qw, const void* kw, const void* hscale, float eps,
+                                         const void* freqs, int rot, void* q_out, void* kc, void* vc, int BS,
+                                         void* stream) {
+  using namespace la;
+  if (T <= 0 || H <= 0 || D <= 0 || G <= 0 || (rot & 1) || rot < 0 || rot > D) return -1;
+  if (ld < (long)(H + G) * D || BS <= 0 || (BS & 7)) return -2;
+  if (!src || !pos || !slots || !qw || !kw || (rot > 0 && !freqs) || !q_out || !kc || !vc) return -3;
+  const size_t shm = (size_t)(rot + 2) * sizeof(float);
+#define LA_QKR(AT, V)                                                                                                   \
+  hipLaunchKernelGGL((qk_row_norm_rope_pages_kernel<AT, V>), dim3(T), dim3(RP_NT), shm, (hipStream_t)stream,            \
+                     (const AT*)src, ld, H, D, G, (const int*)pos, (const int*)slots, (const float*)qw, (const float*)kw, \
+                     (const float*)hscale, eps, (const float*)freqs, rot, (AT*)q_out, (AT*)kc, (AT*)vc, BS)
+  const bool aligned = (((uintptr_t)src | (uintptr_t)q_out | (uintptr_t)kc) & 15) == 0;
+  if (f32) LA_QKR(float, 1);
+  else if (aligned && !(D & 7) && !(rot & 15) && !(ld & 7)) LA_QKR(bf16, 8);
+  else LA_QKR(bf16, 1);
+#undef LA_QKR
   return (int)hipGetLastError();
 }
 

@@ -177,6 +177,14 @@ __global__ __launch_bounds__(256) void shortconv_state_kernel(const AT* __restri
   }
 }
 
+// the same for an fp32 stream of width C convolved elsewhere (norm_chain.hip stream_conv)
+int conv_tail_f32(const float* u, int ldp, int taps, int C, int nseq, const int* cu_q, const int* sslot, float* state,
+                  hipStream_t st) {
+  hipLaunchKernelGGL((shortconv_state_kernel<float>), dim3((C + 255) / 256, nseq), dim3(256), 0, st, u, ldp, taps, C, cu_q,
+                     sslot, state);
+  return (int)hipGetLastError();
+}
+
 }  // namespace la
 
 // f32: 1 = fp32 activations / cache / state, 0 = bf16.  single: every sequence brings exactly one
