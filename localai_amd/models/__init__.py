@@ -10,7 +10,8 @@ import importlib
 MODEL_CLASSES = {"suganex": ("localai_amd.models.suganex", "SuganexModel"),
                  "dadizen": ("localai_amd.models.dadizen", "DadizenModel"),
                  "vinozen": ("localai_amd.models.vinozen", "VinozenModel"),
-                 "gosuvik": ("localai_amd.models.gosuvik", "GosuvikModel")}
+                 "gosuvik": ("localai_amd.models.gosuvik", "GosuvikModel"),
+                 "dobelix": ("localai_amd.models.dobelix", "DobelixModel")}
 
 
 def model_class(arch: str):
