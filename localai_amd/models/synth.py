@@ -1593,3 +1593,57 @@ def write_gosuvik(out_dir: str, width: int = 256, kinds=("channel_delta", "laten
         json.dump(cfg, f_)
     save_file(W, os.path.join(out_dir, "model.safetensors"))
     return out_dir
+
+
+def write_dobelix(out_dir: str, width: int = 256, kinds=("lightning", "attention"), heads: int = 4, kv_heads: int = 2,
+                  dim: int = 64, l_heads: int = 4, l_dim: int = 64, l_vdim: int = 64, taps: int = 4, chunk: int = 256,
+                  ff: int = 1024, vocab: int = 32000, seed: int = 0) -> str:
+    """Random-init Dobelix checkpoint directory (config.json + model.safetensors, bf16): one layer per entry of
+    `kinds`: lightning attention with l_heads heads of l_dim x l_vdim and decays between 0.6 and 0.999, or
+    chunked sigmoid attention with `heads` query heads over kv_heads key heads of width dim; dense
+    feed-forwards of width ff.  Benchmarks and smoke runs; the weights mean nothing."""
+    import json
+
+    import torch
+    from safetensors.torch import save_file
+    os.makedirs(out_dir, exist_ok=True)
+    g = torch.Generator().manual_seed(seed)
+    D = width
+
+    def rnd(*shape, s):
+        return (torch.randn(*shape, generator=g, dtype=torch.float32) * s).to(torch.bfloat16)
+
+    def lin(a, b):
+        return rnd(a, b, s=b ** -0.5)
+
+    def norm(k):
+        return (1.0 + rnd(k, s=0.05).float()).to(torch.bfloat16)
+
+    W = {"embed": rnd(vocab, D, s=0.5), "final.norm": norm(D), "head": lin(vocab, D)}
+    layers = []
+    for i, kind in enumerate(kinds):
+        p = f"l{i}.mix."
+        W[f"l{i}.norm1"], W[f"l{i}.norm2"], W[f"l{i}.canon1"] = norm(D), norm(D), rnd(D, taps, s=0.3)
+        if kind == "lightning":
+            steps = [0.5 * (0.001 / 0.5) ** (k / max(1, l_heads - 1)) for k in range(l_heads)]
+            m = {"heads": l_heads, "dim": l_dim, "vdim": l_vdim, "decay": [2.718281828459045 ** -x for x in steps]}
+            W[p + "q"], W[p + "k"], W[p + "v"] = lin(l_heads * l_dim, D), lin(l_heads * l_dim, D), lin(l_heads * l_vdim, D)
+            W[p + "g"], W[p + "o"], W[p + "norm"] = lin(l_heads * l_vdim, D), lin(D, l_heads * l_vdim), norm(l_heads * l_vdim)
+        elif kind == "attention":
+            m = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "mask": {"size": chunk},
+                 "rot": {"dims": dim, "base": 10000.0}}
+            W[p + "q"], W[p + "k"], W[p + "g"], W[p + "o"] = (lin(heads * dim, D), lin(kv_heads * dim, D), lin(heads * dim, D),
+                                                              lin(D, heads * dim))
+            W[p + "q.norm"], W[p + "k.norm"] = norm(heads * dim), norm(kv_heads * dim)
+            W[p + "temp"], W[p + "pb"] = norm(heads), (rnd(heads, s=0.2).float() - 4.0).to(torch.bfloat16)
+        else:
+            raise ValueError(f"unknown mixer kind {kind!r}")
+        p = f"l{i}.mlp."
+        W[p + "gate"], W[p + "up"], W[p + "down"] = lin(ff, D), lin(ff, D), lin(D, ff)
+        layers.append({"type": kind, "mixer": m, "mlp": {"kind": "dense", "ff": ff}})
+    cfg = {"architecture": "Dobelix", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "canon": {"taps": taps},
+           "embedding": {"scale": 1.5}, "logit_scale": 0.5, "layers": layers}
+    with open(os.path.join(out_dir, "config.json"), "w") as f_:
+        json.dump(cfg, f_)
+    save_file(W, os.path.join(out_dir, "model.safetensors"))
+    return out_dir

@@ -1509,16 +1509,31 @@ def _dec_split_short(B: int, Hkv: int) -> bool:
     return B * Hkv <= DEC_SPLIT_SHORT
 
 
+def _decode_parts_max(B: int, Hkv: int, max_len: int, block_size: int) -> Tuple[int, int]:
+    """(partitions before rounding, key granularity) of attn_decode; the partitions grow with max_len."""
+    max_len = max(1, max_len)
+    nw = decode_waves(B, Hkv)
+    gran = max(32, block_size) if _dec_split_short(B, Hkv) else 128
+    P = max(1, min(-(-DEC_TARGET_WAVES // (B * Hkv * nw)), -(-max_len // gran), 64))
+    return max(P, -(-max_len // (2048 * block_size))), gran
+
+
+def decode_span(max_len: int, window: int, chunk: int, block_size: int) -> int:
+    """The most keys attn_decode walks for sequences of up to max_len tokens: its partitions start at the
+    page of the first key inside the window / the chunk."""
+    for n in (window, chunk):
+        if n > 0:
+            max_len = min(max_len, n + block_size)
+    return max_len
+
+
 def decode_partitions(B: int, Hkv: int, max_len: int, block_size: int = 32) -> Tuple[int, int]:
     """Split-KV partitioning for attn_decode: (P, PS).  Enough partitions to put ~16 waves on
     every CU; each workgroup (decode_waves waves) covers PS keys (multiple of 128 -- of 32 for
     the few-sequence split -- at most 2048 pages so the partition's block-table slice fits the
     kernel's LDS stage)."""
     max_len = max(1, max_len)
-    nw = decode_waves(B, Hkv)
-    gran = max(32, block_size) if _dec_split_short(B, Hkv) else 128
-    P = max(1, min(-(-DEC_TARGET_WAVES // (B * Hkv * nw)), -(-max_len // gran), 64))
-    P = max(P, -(-max_len // (2048 * block_size)))
+    P, gran = _decode_parts_max(B, Hkv, max_len, block_size)
     PS = -(-(-(-max_len // P)) // gran) * gran
     P = -(-max_len // PS)
     return P, PS
@@ -1529,8 +1544,9 @@ def _dec_nw(B: int, Hkv: int) -> int:
 
 
 def decode_workspace(B: int, Hq: int, Hkv: int, Dh: int, max_len: int, device, block_size: int = 32):
-    """Persistent buffers for attn_decode (split-KV partials + self-resetting merge tickets)."""
-    P, _ = decode_partitions(B, Hkv, max_len, block_size)
+    """Persistent buffers for attn_decode (split-KV partials + self-resetting merge tickets): large enough for
+    every span of keys up to max_len (a window or a chunk shortens it)."""
+    P, _ = _decode_parts_max(B, Hkv, max_len, block_size)
     return (torch.empty(max(1, B * Hq * P * Dh), dtype=torch.float32, device=device),
             torch.empty(max(1, B * Hq * P * 2), dtype=torch.float32, device=device),
             torch.zeros(max(1, B * Hkv), dtype=torch.int32, device=device))
@@ -1570,7 +1586,7 @@ def attn_decode(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, b
             raise ValueError("attn_decode: score extras, chunks and gates have no CPU path here (attn_mix has)")
         return _attn_ref_decode(q, k_cache, v_cache, block_tables, seq_lens, scale, softcap, window)
     ldg = _attn_extras("attn_decode", B, Hq, Dh, dist_bias, sink, sigmoid_bias, gate)
-    P, PS = decode_partitions(B, Hkv, max_seq_len, BS)
+    P, PS = decode_partitions(B, Hkv, decode_span(max_seq_len, window, chunk, BS), BS)
     if out is None:
         out = torch.empty(B, Hq, Dh, dtype=torch.bfloat16, device=q.device)
     if (workspace is None or len(workspace) < 3 or workspace[0].numel() < B * Hq * P * Dh
@@ -1615,7 +1631,7 @@ def attn_decode_rope(qkv: Partial, pos: torch.Tensor, slots: torch.Tensor, cos_s
                            workspace=workspace, softcap=softcap, window=window)
     if Hq % Hkv or tuple(v_cache.shape) != (nblk, Hkv, BS // 8, Dh, 8) or k_cache.shape[3] != Dh:
         raise ValueError("attn_decode_rope: head/cache shape mismatch")
-    P, PS = decode_partitions(T, Hkv, max_seq_len, BS)
+    P, PS = decode_partitions(T, Hkv, decode_span(max_seq_len, window, 0, BS), BS)
     if out is None:
         out = torch.empty(T, Hq, Dh, dtype=torch.bfloat16, device=qkv.t.device)
     if (workspace is None or len(workspace) < 3 or workspace[0].numel() < T * Hq * P * Dh

@@ -156,11 +156,12 @@ __global__ __launch_bounds__(NW * 64) __attribute__((amdgpu_waves_per_eu(2))) vo
   // a short sequence takes ONE partition of DEC_ONE_PART keys instead, so it skips the split-KV
   // merge round trip (partials + ticket + last-arriver reduction) -- worth more than the
   // parallelism at a few hundred keys.  Decided per sequence, uniformly for its workgroups.
-  const int PS = (L <= one_part && PS_grid < one_part) ? one_part : PS_grid;
-  const int t0 = p * PS;
-  if (t0 >= L) return;  // empty partition: the combiner only waits for ceil(L / PS) of them
   int wlo = window > 0 ? L - window : 0;  // first key inside the sliding window / the chunk
   if (E.chunk > 0) wlo = max(wlo, (L - 1) / E.chunk * E.chunk);
+  const int base = wlo > 0 ? wlo / BS * BS : 0;  // partitions start at the page of the first visible key
+  const int PS = (L - base <= one_part && PS_grid < one_part) ? one_part : PS_grid;
+  const int t0 = base + p * PS;
+  if (t0 >= L) return;  // empty partition: the combiner only waits for ceil((L - base) / PS) of them
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int r = lane & 15, g = lane >> 4;
   const int kend = min(L, t0 + PS);
@@ -371,7 +372,7 @@ __global__ __launch_bounds__(NW * 64) __attribute__((amdgpu_waves_per_eu(2))) vo
   // wave totals: lsum over the 4 lane groups (same head r)
   lsum += __shfl_xor(lsum, 16, 64);
   lsum += __shfl_xor(lsum, 32, 64);
-  const int np = (L + PS - 1) / PS;  // partitions holding keys of this sequence
+  const int np = (L - base + PS - 1) / PS;  // partitions holding keys of this sequence
   if constexpr (NW == 1) {
     // one wave per workgroup: its accumulators ARE the partition's result (no LDS merge).
     // o[nd][i] is head 4g+i at d = 16nd + r; that head's (m, l) live in lane 4g+i.

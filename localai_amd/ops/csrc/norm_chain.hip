@@ -42,6 +42,34 @@ LA_DEV float src_at(const RowSrc& s, long idx) {
   return (float)((const bf16*)s.p)[idx];
 }
 
+// four neighbouring columns; slabs are requested four at a time (clamped index, masked: no branch between loads)
+LA_DEV f32x4 src4_at(const RowSrc& s, long idx) {
+  if (!s.f32) {
+    const bf16x4 b = *(const bf16x4*)((const bf16*)s.p + idx);
+    return f32x4{(float)b[0], (float)b[1], (float)b[2], (float)b[3]};
+  }
+  const float* f = (const float*)s.p + idx;
+  if (s.S <= 1) return *(const f32x4*)f;
+  f32x4 a = {0.f, 0.f, 0.f, 0.f};
+  for (int k0 = 0; k0 < s.S; k0 += 4) {
+    f32x4 t[4];
+#pragma unroll
+    for (int k = 0; k < 4; ++k) t[k] = *(const f32x4*)(f + (long)min(k0 + k, s.S - 1) * s.slab);
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      const float m = k0 + k < s.S ? 1.f : 0.f;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) a[j] = fmaf(m, t[k][j], a[j]);
+    }
+  }
+  return a;
+}
+
+LA_DEV void put4(void* out, int out_f32, long idx, const f32x4& v) {
+  if (out_f32) *(f32x4*)((float*)out + idx) = v;
+  else *(bf16x4*)((bf16*)out + idx) = bf16x4{(bf16)v[0], (bf16)v[1], (bf16)v[2], (bf16)v[3]};
+}
+
 LA_DEV void put(void* out, int out_f32, long idx, float v) {
   if (out_f32) ((float*)out)[idx] = v;
   else ((bf16*)out)[idx] = (bf16)v;
@@ -49,6 +77,7 @@ LA_DEV void put(void* out, int out_f32, long idx, float v) {
 
 enum { NC_NONE = 0, NC_DYT = 1, NC_RMS = 2, NC_CAST = 3, NC_LN = 4 };
 constexpr int NC_NT = 256;
+constexpr int NC_FEW_ROWS = 512;   // up to here a row gets a workgroup of 1024 threads (wide rows)
 
 __global__ __launch_bounds__(NC_NT) void norm_chain_kernel(float* __restrict__ res, int D, RowSrc src, int has_src,
                                                            int post, float pa, const float* __restrict__ pw,
@@ -105,54 +134,56 @@ __global__ __launch_bounds__(NC_NT) void norm_chain_kernel(float* __restrict__ r
   }
 }
 
-// widths that are a multiple of 4 with one-matrix sources: 4 columns per thread, 16-byte accesses to the stream
-__global__ __launch_bounds__(NC_NT) void norm_chain4_kernel(float* __restrict__ res, int D, const void* __restrict__ sp,
-                                                            int src_f32, int has_src, int post, float pa,
-                                                            const float* __restrict__ pw, const float* __restrict__ pb,
-                                                            float eps, const float* __restrict__ addv, int replace,
-                                                            int pre, float qa, const float* __restrict__ qw,
-                                                            const float* __restrict__ qb, void* __restrict__ out,
-                                                            int out_f32) {
-  __shared__ float red[NC_NT / 64];
+// Widths that are a multiple of 4: 4 columns per thread, 16-byte accesses; the branch row (slabs summed)
+// stays in registers between the statistics and the update for the first KEEP * 4 NT columns.  NT = 1024
+// for batches of few rows (decoding), where a row's chain of load latencies is what a launch costs.
+template <int NT>
+__global__ __launch_bounds__(NT) void norm_chain4_kernel(float* __restrict__ res, int D, RowSrc src, int has_src, int post,
+                                                         float pa, const float* __restrict__ pw,
+                                                         const float* __restrict__ pb, float eps,
+                                                         const float* __restrict__ addv, int replace, int pre, float qa,
+                                                         const float* __restrict__ qw, const float* __restrict__ qb,
+                                                         void* __restrict__ out, int out_f32) {
+  constexpr int KEEP = NT >= 1024 ? 1 : 4;
+  __shared__ float red[NT / 64];
   const int t = blockIdx.x, tid = threadIdx.x;
   const long base = (long)t * D;
-  auto load = [&](int c, float* y) {
-    if (src_f32) {
-      const float4 v = *(const float4*)((const float*)sp + base + c);
-      y[0] = v.x; y[1] = v.y; y[2] = v.z; y[3] = v.w;
-    } else {
-      const bf16x4 v = *(const bf16x4*)((const bf16*)sp + base + c);
-#pragma unroll
-      for (int j = 0; j < 4; ++j) y[j] = (float)v[j];
-    }
-  };
+  f32x4 held[KEEP];
   float inv = 1.f, mean = 0.f;
+  if (has_src) {
+#pragma unroll
+    for (int k = 0; k < KEEP; ++k) {
+      const int c = (tid + k * NT) * 4;
+      if (c < D) held[k] = src4_at(src, base + c);
+    }
+  }
   if (has_src && (post == NC_RMS || post == NC_LN)) {
     if (post == NC_LN) {
       float sm = 0.f;
-      for (int c = tid * 4; c < D; c += NC_NT * 4) {
-        float y[4];
-        load(c, y);
+#pragma unroll
+      for (int k = 0; k < KEEP; ++k)
+        if ((tid + k * NT) * 4 < D) sm += (held[k][0] + held[k][1]) + (held[k][2] + held[k][3]);
+      for (int c = (tid + KEEP * NT) * 4; c < D; c += NT * 4) {
+        const f32x4 y = src4_at(src, base + c);
         sm += (y[0] + y[1]) + (y[2] + y[3]);
       }
-      mean = block_sum<NC_NT>(sm, red) / (float)D;
+      mean = block_sum<NT>(sm, red) / (float)D;
     }
     float ss = 0.f;
-    for (int c = tid * 4; c < D; c += NC_NT * 4) {
-      float y[4];
-      load(c, y);
+    auto sq = [&](const f32x4& y) {
 #pragma unroll
       for (int j = 0; j < 4; ++j) ss = fmaf(y[j] - mean, y[j] - mean, ss);
-    }
-    ss = block_sum<NC_NT>(ss, red);
+    };
+#pragma unroll
+    for (int k = 0; k < KEEP; ++k)
+      if ((tid + k * NT) * 4 < D) sq(held[k]);
+    for (int c = (tid + KEEP * NT) * 4; c < D; c += NT * 4) sq(src4_at(src, base + c));
+    ss = block_sum<NT>(ss, red);
     inv = 1.f / sqrtf(ss / (float)D + eps);
   }
-  for (int c = tid * 4; c < D; c += NC_NT * 4) {
-    const float4 xv = *(const float4*)(res + base + c);
-    float x[4] = {xv.x, xv.y, xv.z, xv.w};
+  auto update = [&](int c, f32x4 y) {
+    f32x4 x = *(const f32x4*)(res + base + c);
     if (has_src) {
-      float y[4];
-      load(c, y);
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
         if (post == NC_DYT) y[j] = fmaf(tanhf(pa * y[j]), pw[c + j], pb[c + j]);
@@ -160,44 +191,43 @@ __global__ __launch_bounds__(NC_NT) void norm_chain4_kernel(float* __restrict__ 
         if (addv) y[j] += addv[c + j];
         x[j] = replace ? y[j] : x[j] + y[j];
       }
-      *(float4*)(res + base + c) = make_float4(x[0], x[1], x[2], x[3]);
+      *(f32x4*)(res + base + c) = x;
     }
     if (pre == NC_DYT || pre == NC_CAST) {
-      float o[4];
+      f32x4 o = x;
+      if (pre == NC_DYT) {
 #pragma unroll
-      for (int j = 0; j < 4; ++j) o[j] = pre == NC_DYT ? fmaf(tanhf(qa * x[j]), qw[c + j], qb[c + j]) : x[j];
-      if (out_f32) *(float4*)((float*)out + base + c) = make_float4(o[0], o[1], o[2], o[3]);
-      else {
-        bf16x4 ob = {(bf16)o[0], (bf16)o[1], (bf16)o[2], (bf16)o[3]};
-        *(bf16x4*)((bf16*)out + base + c) = ob;
+        for (int j = 0; j < 4; ++j) o[j] = fmaf(tanhf(qa * x[j]), qw[c + j], qb[c + j]);
       }
+      put4(out, out_f32, base + c, o);
     }
+  };
+#pragma unroll
+  for (int k = 0; k < KEEP; ++k) {
+    const int c = (tid + k * NT) * 4;
+    if (c < D) update(c, held[k]);
   }
+  for (int c = (tid + KEEP * NT) * 4; c < D; c += NT * 4) update(c, has_src ? src4_at(src, base + c) : f32x4{0.f, 0.f, 0.f, 0.f});
   if (pre == NC_LN || pre == NC_RMS) {   // norm of the updated row: every thread re-reads the columns it wrote
     float m2 = 0.f;
     if (pre == NC_LN) {
       float sm = 0.f;
-      for (int c = tid * 4; c < D; c += NC_NT * 4) {
+      for (int c = tid * 4; c < D; c += NT * 4) {
         const float4 v = *(const float4*)(res + base + c);
         sm += (v.x + v.y) + (v.z + v.w);
       }
-      m2 = block_sum<NC_NT>(sm, red) / (float)D;
+      m2 = block_sum<NT>(sm, red) / (float)D;
     }
     float ss = 0.f;
-    for (int c = tid * 4; c < D; c += NC_NT * 4) {
+    for (int c = tid * 4; c < D; c += NT * 4) {
       const float4 v = *(const float4*)(res + base + c);
       ss = fmaf(v.x - m2, v.x - m2, fmaf(v.y - m2, v.y - m2, fmaf(v.z - m2, v.z - m2, fmaf(v.w - m2, v.w - m2, ss))));
     }
-    const float inv2 = 1.f / sqrtf(block_sum<NC_NT>(ss, red) / (float)D + qa);
-    for (int c = tid * 4; c < D; c += NC_NT * 4) {
+    const float inv2 = 1.f / sqrtf(block_sum<NT>(ss, red) / (float)D + qa);
+    for (int c = tid * 4; c < D; c += NT * 4) {
       const float4 v = *(const float4*)(res + base + c);
-      const float o[4] = {(v.x - m2) * inv2 * qw[c], (v.y - m2) * inv2 * qw[c + 1], (v.z - m2) * inv2 * qw[c + 2],
-                          (v.w - m2) * inv2 * qw[c + 3]};
-      if (out_f32) *(float4*)((float*)out + base + c) = make_float4(o[0], o[1], o[2], o[3]);
-      else {
-        bf16x4 ob = {(bf16)o[0], (bf16)o[1], (bf16)o[2], (bf16)o[3]};
-        *(bf16x4*)((bf16*)out + base + c) = ob;
-      }
+      put4(out, out_f32, base + c, f32x4{(v.x - m2) * inv2 * qw[c], (v.y - m2) * inv2 * qw[c + 1],
+                                         (v.z - m2) * inv2 * qw[c + 2], (v.w - m2) * inv2 * qw[c + 3]});
     }
   }
 }
@@ -208,49 +238,48 @@ __global__ __launch_bounds__(NC_NT) void norm_chain4_kernel(float* __restrict__ 
 // portion), or nothing before position 0.  SINGLE: every sequence brings one row; the branch's norm and the
 // residual add come first and the tail advances, all in one launch (each thread is the only reader and
 // writer of its columns of the row and of the slot).
-template <int V, bool SINGLE>
-__global__ __launch_bounds__(NC_NT) void stream_conv_kernel(float* __restrict__ res, int D, RowSrc src, int has_src, int post,
-                                                            const float* __restrict__ pw, float eps,
-                                                            const float* __restrict__ wt, int taps,
-                                                            const int* __restrict__ row_seq, const int* __restrict__ cu_q,
-                                                            const int* __restrict__ pos, const int* __restrict__ sslot,
-                                                            float* __restrict__ tail, void* __restrict__ out, int out_f32) {
+template <int V, bool SINGLE, int NT>
+__global__ __launch_bounds__(NT) void stream_conv_kernel(float* __restrict__ res, int D, RowSrc src, int has_src, int post,
+                                                         const float* __restrict__ pw, float eps,
+                                                         const float* __restrict__ wt, int taps,
+                                                         const int* __restrict__ row_seq, const int* __restrict__ cu_q,
+                                                         const int* __restrict__ pos, const int* __restrict__ sslot,
+                                                         float* __restrict__ tail, void* __restrict__ out, int out_f32) {
   typedef float fvec __attribute__((ext_vector_type(V)));
-  typedef bf16 bvec __attribute__((ext_vector_type(V)));
-  __shared__ float red[NC_NT / 64];
+  constexpr int KEEP = NT >= 1024 ? 1 : 4;
+  __shared__ float red[NT / 64];
   const int t = blockIdx.x, tid = threadIdx.x;
   const long base = (long)t * D;
   const int seq = SINGLE ? t : row_seq[t], m = SINGLE ? 0 : t - cu_q[seq], p = pos[t], ss = sslot[seq];
   float* st = tail + (long)ss * (taps - 1) * D;
   auto load = [&](int c) -> fvec {
-    fvec y;
-    if (V == 4 && src.S <= 1) {
-      if (src.f32) y = *(const fvec*)((const float*)src.p + base + c);
-      else {
-        const bvec b = *(const bvec*)((const bf16*)src.p + base + c);
-#pragma unroll
-        for (int j = 0; j < V; ++j) y[j] = (float)b[j];
-      }
-    } else {
-#pragma unroll
-      for (int j = 0; j < V; ++j) y[j] = src_at(src, base + c + j);
-    }
-    return y;
+    if constexpr (V == 4) return src4_at(src, base + c);
+    else return fvec(src_at(src, base + c));
   };
+  fvec held[KEEP];
   float inv = 1.f;
-  if (SINGLE && has_src && post == NC_RMS) {
-    float s2 = 0.f;
-    for (int c = tid * V; c < D; c += NC_NT * V) {
-      const fvec y = load(c);
+  if (SINGLE && has_src) {
 #pragma unroll
-      for (int j = 0; j < V; ++j) s2 = fmaf(y[j], y[j], s2);
+    for (int k = 0; k < KEEP; ++k) {
+      const int c = (tid + k * NT) * V;
+      if (c < D) held[k] = load(c);
     }
-    inv = 1.f / sqrtf(block_sum<NC_NT>(s2, red) / (float)D + eps);
+    if (post == NC_RMS) {
+      float s2 = 0.f;
+      auto sq = [&](const fvec& y) {
+#pragma unroll
+        for (int j = 0; j < V; ++j) s2 = fmaf(y[j], y[j], s2);
+      };
+#pragma unroll
+      for (int k = 0; k < KEEP; ++k)
+        if ((tid + k * NT) * V < D) sq(held[k]);
+      for (int c = (tid + KEEP * NT) * V; c < D; c += NT * V) sq(load(c));
+      inv = 1.f / sqrtf(block_sum<NT>(s2, red) / (float)D + eps);
+    }
   }
-  for (int c = tid * V; c < D; c += NC_NT * V) {
+  auto column = [&](int c, const fvec& y) {
     fvec x = *(const fvec*)(res + base + c);
     if (SINGLE && has_src) {
-      const fvec y = load(c);
 #pragma unroll
       for (int j = 0; j < V; ++j) x[j] += post == NC_RMS ? y[j] * inv * pw[c + j] : y[j];
       *(fvec*)(res + base + c) = x;
@@ -272,14 +301,15 @@ __global__ __launch_bounds__(NC_NT) void stream_conv_kernel(float* __restrict__ 
     const fvec w = *(const fvec*)(wt + (long)(taps - 1) * D + c);
 #pragma unroll
     for (int j = 0; j < V; ++j) acc[j] = x[j] + fmaf(w[j], x[j], acc[j]);
-    if (out_f32) *(fvec*)((float*)out + base + c) = acc;
-    else {
-      bvec o;
+    if constexpr (V == 4) put4(out, out_f32, base + c, acc);
+    else put(out, out_f32, base + c, acc[0]);
+  };
 #pragma unroll
-      for (int j = 0; j < V; ++j) o[j] = (bf16)acc[j];
-      *(bvec*)((bf16*)out + base + c) = o;
-    }
+  for (int k = 0; k < KEEP; ++k) {
+    const int c = (tid + k * NT) * V;
+    if (c < D) column(c, held[k]);
   }
+  for (int c = (tid + KEEP * NT) * V; c < D; c += NT * V) column(c, SINGLE && has_src ? load(c) : fvec{});
 }
 
 int conv_tail_f32(const float* u, int ldp, int taps, int C, int nseq, const int* cu_q, const int* sslot, float* state,
@@ -500,15 +530,17 @@ extern "C" int la_stream_conv(void* res, int T, int D, const void* sp, int src_f
   if (sp && ((post != NC_NONE && post != NC_RMS) || (post == NC_RMS && !pw) || (src_f32 && S < 1))) return -3;
   RowSrc s{sp, src_f32, slab, S};
   hipStream_t st = (hipStream_t)stream;
-#define LA_SCV(V, SG)                                                                                                  \
-  hipLaunchKernelGGL((stream_conv_kernel<V, SG>), dim3(T), dim3(NC_NT), 0, st, (float*)res, D, s, sp != nullptr, post, \
-                     (const float*)pw, eps, (const float*)wt, taps, (const int*)row_seq, (const int*)cu_q,             \
+#define LA_SCV(V, SG, NT)                                                                                                 \
+  hipLaunchKernelGGL((stream_conv_kernel<V, SG, NT>), dim3(T), dim3(NT), 0, st, (float*)res, D, s, sp != nullptr, post,   \
+                     (const float*)pw, eps, (const float*)wt, taps, (const int*)row_seq, (const int*)cu_q,                \
                      (const int*)pos, (const int*)sslot, (float*)tail, out, out_f32)
   if (single) {
-    if (!(D & 3)) LA_SCV(4, true); else LA_SCV(1, true);
+    if (D & 3) LA_SCV(1, true, 256);
+    else if (T <= NC_FEW_ROWS && D > 1024) LA_SCV(4, true, 1024);
+    else LA_SCV(4, true, 256);
     return (int)hipGetLastError();
   }
-  if (!(D & 3)) LA_SCV(4, false); else LA_SCV(1, false);
+  if (D & 3) LA_SCV(1, false, 256); else LA_SCV(4, false, 256);
 #undef LA_SCV
   if (taps > 1) return conv_tail_f32((const float*)res, D, taps, D, nseq, (const int*)cu_q, (const int*)sslot, (float*)tail, st);
   return (int)hipGetLastError();
@@ -584,13 +616,17 @@ extern "C" int la_norm_chain(void* res, int T, int D, const void* sp, int src_f3
   if (pre != NC_NONE && !out) return -3;
   const int has = sp != nullptr;
   if (has && src_f32 && S < 1) return -4;
-  if ((D & 3) == 0 && (!has || S <= 1)) {
-    hipLaunchKernelGGL(norm_chain4_kernel, dim3(T), dim3(NC_NT), 0, (hipStream_t)stream, (float*)res, D, sp, src_f32, has,
-                       post, pa, (const float*)pw, (const float*)pb, eps, (const float*)addv, replace, pre, qa,
-                       (const float*)qw, (const float*)qb, out, out_f32);
+  RowSrc s{sp, src_f32, slab, S};
+  if ((D & 3) == 0) {
+#define LA_NC4(NT)                                                                                                        \
+  hipLaunchKernelGGL(norm_chain4_kernel<NT>, dim3(T), dim3(NT), 0, (hipStream_t)stream, (float*)res, D, s, has, post, pa, \
+                     (const float*)pw, (const float*)pb, eps, (const float*)addv, replace, pre, qa, (const float*)qw,     \
+                     (const float*)qb, out, out_f32)
+    if (T <= NC_FEW_ROWS && D > 1024) LA_NC4(1024);
+    else LA_NC4(256);
+#undef LA_NC4
     return (int)hipGetLastError();
   }
-  RowSrc s{sp, src_f32, slab, S};
   hipLaunchKernelGGL(norm_chain_kernel, dim3(T), dim3(NC_NT), 0, (hipStream_t)stream, (float*)res, D, s, has, post, pa,
                      (const float*)pw, (const float*)pb, eps, (const float*)addv, replace, pre, qa, (const float*)qw,
                      (const float*)qb, out, out_f32);

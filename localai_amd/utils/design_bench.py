@@ -6,7 +6,8 @@ checkpoint) and routed experts (beside a Mixtral-style checkpoint); Dadizen: one
 kind (windowed attention, latent attention, retention) beside the llama checkpoint; Vinozen:
 attention with a dense feed-forward, attention with routed experts, the state-space mixer, beside
 the llama and Mixtral-style checkpoints; Gosuvik: the delta rule, latent attention with routed experts,
-the parallel mixer, beside the same two -- all stored as
+the parallel mixer, beside the same two; Dobelix: one model per mixer kind (lightning attention, chunked
+sigmoid attention) beside the llama checkpoint and Dadizen's retention -- all stored as
 dense bf16 weights so every GEMM takes the same library path, and each is timed through its engine's own
 batch construction (native scheduler, paged KV pool, state slots) and `model.forward`:
   prefill: `n_seq` prompts of `prompt` tokens in one batch, tokens/s;
@@ -116,6 +117,25 @@ def _gosuvik_models(size: str, cache: str) -> Dict[str, str]:
     return out
 
 
+def _dobelix_models(size: str, cache: str) -> Dict[str, str]:
+    """Two equal layers of one mixer kind each: chunked sigmoid attention with the size's heads (chunk of the
+    size), lightning attention with half the heads at twice the value width (the proportions of the
+    retention layers it is compared with); beside the llama checkpoint and Dadizen's retention model."""
+    from ..models import synth
+    s = SIZES[size]
+    out = {}
+    for kind in ("attention", "lightning"):
+        p = os.path.join(cache, f"dobelix-{size}-{kind}")
+        if not os.path.exists(os.path.join(p, "model.safetensors")):
+            synth.write_dobelix(p, width=s["width"], kinds=(kind, kind), heads=s["heads"], kv_heads=s["kv"], dim=s["dim"],
+                                l_heads=s["heads"] // 2, l_dim=s["dim"], l_vdim=2 * s["dim"], taps=4, chunk=s["chunk"],
+                                ff=s["ff"], vocab=VOCAB)
+        out[f"dobelix-{kind}"] = p
+    near = _dadizen_models(size, cache)
+    out["dadizen-retention"], out["llama-dense"] = near["dadizen-retention"], near["llama-dense"]
+    return out
+
+
 def _models(size: str, cache: str) -> Dict[str, str]:
     from ..models import synth
     s = SIZES[size]
@@ -222,16 +242,17 @@ def _measure(path: str, n_seq: int, prompt: int, batch: int, context: int, iters
 
 def run(design: str, sizes: List[str], cache: str, n_seq: int = 4, prompt: int = 2048, batch: int = 64,
         context: int = 1536, iters: int = 5) -> dict:
-    if design not in ("suganex", "dadizen", "vinozen", "gosuvik"):
-        raise SystemExit(f"--design-compare: unknown design {design!r} (suganex, dadizen, vinozen, gosuvik)")
+    designs = {"suganex": _models, "dadizen": _dadizen_models, "vinozen": _vinozen_models, "gosuvik": _gosuvik_models,
+               "dobelix": _dobelix_models}
+    if design not in designs:
+        raise SystemExit(f"--design-compare: unknown design {design!r} ({', '.join(designs)})")
     os.makedirs(cache, exist_ok=True)
     res = {"design": design, "dtype": "bf16", "data": "synthetic", "layers": 2,
            "workload": {"prefill": f"{n_seq} x {prompt} tokens", "decode": f"batch {batch} at context {context}"},
            "sizes": {}}
     for size in sizes:
         t0 = time.time()
-        paths = {"suganex": _models, "dadizen": _dadizen_models, "vinozen": _vinozen_models,
-                 "gosuvik": _gosuvik_models}[design](size, cache)
+        paths = designs[design](size, cache)
         row = {}
         for name, p in paths.items():
             row[name] = {k: round(v, 3 if k.endswith("ms") else 1)
