@@ -1599,7 +1599,7 @@ def write_dobelix(out_dir: str, width: int = 256, kinds=("lightning", "attention
                   dim: int = 64, l_heads: int = 4, l_dim: int = 64, l_vdim: int = 64, taps: int = 4, chunk: int = 256,
                   ff: int = 1024, vocab: int = 32000, seed: int = 0) -> str:
     """Random-init Dobelix checkpoint directory (config.json + model.safetensors, bf16): one layer per entry of
-    `kinds`: lightning attention with l_heads heads of l_dim x l_vdim and decays between 0.6 and 0.999, or
+    `kinds`: lightning attention with l_heads heads of l_dim x l_vdim and decays between 0.5 and 0.998, or
     chunked sigmoid attention with `heads` query heads over kv_heads key heads of width dim; dense
     feed-forwards of width ff.  Benchmarks and smoke runs; the weights mean nothing."""
     import json
@@ -1625,8 +1625,8 @@ def write_dobelix(out_dir: str, width: int = 256, kinds=("lightning", "attention
         p = f"l{i}.mix."
         W[f"l{i}.norm1"], W[f"l{i}.norm2"], W[f"l{i}.canon1"] = norm(D), norm(D), rnd(D, taps, s=0.3)
         if kind == "lightning":
-            steps = [0.5 * (0.001 / 0.5) ** (k / max(1, l_heads - 1)) for k in range(l_heads)]
-            m = {"heads": l_heads, "dim": l_dim, "vdim": l_vdim, "decay": [2.718281828459045 ** -x for x in steps]}
+            m = {"heads": l_heads, "dim": l_dim, "vdim": l_vdim,
+                 "decay": [1.0 - 2.0 ** (-1.0 - 8.0 * k / max(1, l_heads - 1)) for k in range(l_heads)]}
             W[p + "q"], W[p + "k"], W[p + "v"] = lin(l_heads * l_dim, D), lin(l_heads * l_dim, D), lin(l_heads * l_vdim, D)
             W[p + "g"], W[p + "o"], W[p + "norm"] = lin(l_heads * l_vdim, D), lin(D, l_heads * l_vdim), norm(l_heads * l_vdim)
         elif kind == "attention":
