@@ -11,7 +11,8 @@ MODEL_CLASSES = {"suganex": ("localai_amd.models.suganex", "SuganexModel"),
                  "dadizen": ("localai_amd.models.dadizen", "DadizenModel"),
                  "vinozen": ("localai_amd.models.vinozen", "VinozenModel"),
                  "gosuvik": ("localai_amd.models.gosuvik", "GosuvikModel"),
-                 "dobelix": ("localai_amd.models.dobelix", "DobelixModel")}
+                 "dobelix": ("localai_amd.models.dobelix", "DobelixModel"),
+                 "bugapel": ("localai_amd.models.bugapel", "BugapelModel")}
 
 
 def model_class(arch: str):

@@ -87,8 +87,8 @@ def lib():
             "la_embed": [I, P, P, P, P, I, I, P, I, P, F, P],
             "la_dequant": [I, P, P, P, P, I, I, P, P],
             "la_attn_decode": [P, P, P, P, I, P, I, I, I, I, I, F, I, I, P, P, P, P, P, LNG, I, P, P, P, P, F, I, I, P, I, P,
-                               P, I, P, LNG, P],
-            "la_attn_prefill": [P, P, P, P, I, P, P, P, I, I, I, I, I, F, P, F, I, P, I, P, P, I, P, LNG, P],
+                               P, I, P, LNG, I, P],
+            "la_attn_prefill": [P, P, P, P, I, P, P, P, I, I, I, I, I, F, P, F, I, P, I, P, P, I, P, LNG, I, P],
             "la_sample": [P, LNG, I, I, P, P, P, P, P],
             "la_penalties": [P, LNG, I, P, I, P, P, I, P, P],
             "la_penalties_cols": [P, LNG, I, P, I, P, P, I, P, I, I, P],
@@ -121,11 +121,11 @@ def lib():
             "la_bsmoe": [I, I, P, I, I, I, P, P, I, P, I, I, I, P, P, I, LNG, I, I, P],
             "la_decode_advance": [P, P, P, P, P, P, I, I, I, P, I, P, P, P],
             "la_shortconv_kv": [I, I, P, I, P, P, I, I, I, I, P, P, P, P, P, P, P, P, P, I, I, I, I, P, P, P, I, I, P],
-            "la_attn_mix_rows": [I, P, P, P, P, P, P, I, I, I, I, I, I, I, F, F, P, P, I, I, P, I, I, P, P, I, P, P, P],
+            "la_attn_mix_rows": [I, P, P, P, P, P, P, I, I, I, I, I, I, I, F, F, P, P, I, I, P, I, I, P, P, I, P, P, I, P],
             "la_attn_mix_tiles": [P, P, P, P, I, P, P, P, I, I, I, I, I, I, F, F, P, P, I, I, P, I, I, P, I, P, P, I, P, I,
-                                  P, P, P],
+                                  P, P, I, P],
             "la_router_sigmoid": [I, P, LNG, P, P, I, I, I, I, I, P, P, P],
-            "la_router_topk": [I, I, P, LNG, P, P, I, I, I, I, I, P, P, P],
+            "la_router_topk": [I, I, P, LNG, P, P, I, I, I, I, I, I, I, F, P, P, P],
             "la_moe_pairs": [I, P, P, P, P, P, P, I, I, I, I, I, P, P, I, F, F, P],
             "la_sinusoid_add": [P, I, I, P, P, P],
             "la_qk_norm_pages": [I, P, I, I, I, I, I, I, I, P, P, F, F, I, P, P, P, I, P],
@@ -141,6 +141,10 @@ def lib():
             "la_stream_conv": [P, I, I, P, I, LNG, I, I, P, F, P, I, I, P, P, P, P, P, I, P, I, P],
             "la_glu_act": [P, I, LNG, I, I, I, I, P, I, P],
             "la_lightning": [I, P, I, I, I, I, I, I, P, P, P, P, I, P, P, F, P, P, P, I, P],
+            "la_hyper_streams": [P, I, I, I, P, P, I, LNG, I, P, P, P, P, P, P, F, P, I, P],
+            "la_head_rope_pages": [I, P, I, LNG, I, LNG, P, I, I, I, I, I, I, P, P, P, I, I, I, F, P, P, P, I, P],
+            "la_gla": [I, P, LNG, P, P, F, I, I, I, I, I, P, P, P, P, I, P, F, I, I, P, P, P, P, P, P, P],
+            "la_gla_width": [I],
             "la_rotate_heads": [I, P, I, I, I, P, P, F, F, P, LNG, P],
             "la_delta_rule": [I, P, LNG, P, P, I, I, I, I, I, I, I, I, P, P, P, P, P, F, F, P, P, P, P, P, I, P, P, P, P,
                               P, P, P],
@@ -1569,20 +1573,21 @@ def attn_decode(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, b
                 workspace: Optional[Tuple[torch.Tensor, ...]] = None, softcap: float = 0.0,
                 window: int = 0, dist_bias: Optional[torch.Tensor] = None,
                 sink: Optional[torch.Tensor] = None, sigmoid_bias: Optional[torch.Tensor] = None, chunk: int = 0,
-                gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+                gate: Optional[torch.Tensor] = None, keep: int = 0) -> torch.Tensor:
     """q [B,Hq,Dh] bf16; K cache [nblk,Hkv,BS,Dh]; V cache (grouped-transposed pages)
     [nblk,Hkv,BS/8,Dh,8]; block_tables [B,maxb] i32; seq_lens [B] i32.  softcap > 0: scores
     softcap * tanh(s / softcap); window > 0: only the last `window` keys are attended (Gemma-2).
     dist_bias (fp32 [N, Hq]) / sink (fp32 [Hq]): a bias per distance and head (constant from row
     N - 1 on) and a logit without key or value in the softmax denominator, as in attn_mix.
     sigmoid_bias (fp32 [Hq]), chunk, gate ([B, Hq Dh], any row stride): sigmoid weights instead of the
-    softmax, the chunked mask and a logit per output channel, as in attn_mix."""
+    softmax, the chunked mask and a logit per output channel, as in attn_mix.  keep: the first `keep` keys
+    stay visible beside the window's or chunk's (not with sigmoid_bias)."""
     B, Hq, Dh = q.shape
     nblk, Hkv, BS, Dh2 = k_cache.shape
     if Dh2 != Dh or Hq % Hkv or tuple(v_cache.shape) != (nblk, Hkv, BS // 8, Dh, 8):
         raise ValueError("attn_decode: head/cache shape mismatch")
     if not q.is_cuda:
-        if dist_bias is not None or sink is not None or sigmoid_bias is not None or chunk or gate is not None:
+        if dist_bias is not None or sink is not None or sigmoid_bias is not None or chunk or gate is not None or keep:
             raise ValueError("attn_decode: score extras, chunks and gates have no CPU path here (attn_mix has)")
         return _attn_ref_decode(q, k_cache, v_cache, block_tables, seq_lens, scale, softcap, window)
     ldg = _attn_extras("attn_decode", B, Hq, Dh, dist_bias, sink, sigmoid_bias, gate)
@@ -1598,7 +1603,7 @@ def attn_decode(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, b
                                 out.data_ptr(), po.data_ptr(), pml.data_ptr(), tk.data_ptr(), None, 0, 0, None, None,
                                 None, None, float(softcap), int(window), _dec_nw(B, Hkv), _ptr(dist_bias),
                                 dist_bias.shape[0] if dist_bias is not None else 0, _ptr(sink), _ptr(sigmoid_bias),
-                                int(chunk), _ptr(gate), ldg, _stream()),
+                                int(chunk), _ptr(gate), ldg, int(keep), _stream()),
            "la_attn_decode")
     return out
 
@@ -1643,7 +1648,7 @@ def attn_decode_rope(qkv: Partial, pos: torch.Tensor, slots: torch.Tensor, cos_s
                                 block_tables.shape[1], seq_lens.data_ptr(), T, Hq, Hkv, Dh, BS, float(scale), P, PS,
                                 out.data_ptr(), po.data_ptr(), pml.data_ptr(), tk.data_ptr(), a[0], a[1], a[2], a[3],
                                 pos.data_ptr(), slots.data_ptr(), cos_sin.data_ptr(), float(softcap), int(window),
-                                _dec_nw(T, Hkv), None, 0, None, None, 0, None, 0, _stream()),
+                                _dec_nw(T, Hkv), None, 0, None, None, 0, None, 0, 0, _stream()),
            "la_attn_decode(rope)")
     return out
 
@@ -1713,13 +1718,13 @@ def attn_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, 
                  out: Optional[torch.Tensor] = None, softcap: float = 0.0, window: int = 0,
                  dist_bias: Optional[torch.Tensor] = None, sink: Optional[torch.Tensor] = None,
                  sigmoid_bias: Optional[torch.Tensor] = None, chunk: int = 0,
-                 gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+                 gate: Optional[torch.Tensor] = None, keep: int = 0) -> torch.Tensor:
     """Causal attention for new tokens. q [T,Hq,Dh]; cu_q [nseq+1]; ctx_lens [nseq] (cached+new).
-    dist_bias (fp32 [N, Hq]) / sink / sigmoid_bias (fp32 [Hq]) / chunk / gate: as in attn_decode and attn_mix."""
+    dist_bias (fp32 [N, Hq]) / sink / sigmoid_bias (fp32 [Hq]) / chunk / gate / keep: as in attn_decode and attn_mix."""
     T, Hq, Dh = q.shape
     Hkv = k_cache.shape[1]
     if not q.is_cuda:
-        if dist_bias is not None or sink is not None or sigmoid_bias is not None or chunk or gate is not None:
+        if dist_bias is not None or sink is not None or sigmoid_bias is not None or chunk or gate is not None or keep:
             raise ValueError("attn_prefill: score extras, chunks and gates have no CPU path here (attn_mix has)")
         return _attn_ref_prefill(q, k_cache, v_cache, cu_q, ctx_lens, block_tables, scale, softcap, window)
     ldg = _attn_extras("attn_prefill", T, Hq, Dh, dist_bias, sink, sigmoid_bias, gate)
@@ -1733,7 +1738,7 @@ def attn_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, 
                                  block_tables.shape[1], Hq, Hkv, Dh, k_cache.shape[2], float(scale),
                                  out.data_ptr(), float(softcap), int(window), _ptr(dist_bias),
                                  dist_bias.shape[0] if dist_bias is not None else 0, _ptr(sink), _ptr(sigmoid_bias),
-                                 int(chunk), _ptr(gate), ldg, _stream()), "la_attn_prefill")
+                                 int(chunk), _ptr(gate), ldg, int(keep), _stream()), "la_attn_prefill")
     return out
 
 
@@ -1914,13 +1919,15 @@ def attn_mix(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, row_
              window: int = 0, gate: Optional[torch.Tensor] = None, tiles: Optional[torch.Tensor] = None,
              tile_rows: int = 0, cu_q: Optional[torch.Tensor] = None, key_splits: int = 1,
              v_width: int = 0, dist_bias: Optional[torch.Tensor] = None,
-             sink: Optional[torch.Tensor] = None, sigmoid_bias: Optional[torch.Tensor] = None) -> torch.Tensor:
+             sink: Optional[torch.Tensor] = None, sigmoid_bias: Optional[torch.Tensor] = None,
+             keep: int = 0) -> torch.Tensor:
     """Attention with reshaped scores over paged K ([blocks, G, BS, Dk]) and V ([blocks, G, BS / 8,
     Dv, 8], transposed per 8 keys: the operand layout of the P.V matrix instruction); one
     query row per token, row r belonging to sequence row_seq[r] (block_tables row) at position
     pos[r], its keys 0..pos[r] already in the pools.  Per head g: s = scale q.k, softcap tanh,
     minus slopes[g] * distance; then the heads' scores are mixed by talk [H, H]; keys are visible
-    within the query's chunk of `chunk` positions and the last `window` positions (0: no limit);
+    within the query's chunk of `chunk` positions and the last `window` positions (0: no limit), and the
+    first `keep` keys of the sequence beside those;
     softmax; values of width Dv; each head's output times sigmoid(gate[r, h]) (gate: [T, H] view,
     any row stride), or, with a [T, H Dv] gate, every output channel times the sigmoid of its own logit.  Returns [T, H * Dv] in q's dtype; scores and softmax in fp32.
     tiles / tile_rows / cu_q (attn_mix_tiles): the first tile_rows rows are whole prompt portions,
@@ -1947,6 +1954,8 @@ def attn_mix(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, row_
         raise ValueError("attn_mix: dist_bias is [N, H]")
     if sink is not None and sink.numel() != H:
         raise ValueError("attn_mix: sink is [H]")
+    if keep < 0 or (keep and v_cache is None):
+        raise ValueError("attn_mix: kept first keys are not combined with latent caches")
     if sigmoid_bias is not None and (sigmoid_bias.numel() != H or sink is not None or v_cache is None):
         raise ValueError("attn_mix: sigmoid_bias is [H], without sinks and latent caches")
     if v_cache is None:
@@ -1968,7 +1977,7 @@ def attn_mix(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, row_
             lo = (i // chunk) * chunk if chunk > 0 else 0
             if window > 0:
                 lo = max(lo, i - window + 1)
-            js = torch.arange(lo, i + 1)
+            js = torch.cat([torch.arange(0, min(keep, lo)), torch.arange(lo, i + 1)])
             tab = block_tables[int(row_seq[r])].long()
             blk, off = tab[js // BS], js % BS
             kk = k_cache[blk, :, off].float().repeat_interleave(rep, 1)     # [n, H, Dk]
@@ -2049,7 +2058,7 @@ def attn_mix(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, row_
                                      block_tables.shape[1], H, G, Dk, Dv, BS, float(scale), float(softcap), _ptr(slopes),
                                      _ptr(talk), int(chunk), int(window), _ptr(gate), ldg, gch, out.data_ptr(), ns,
                                      _ptr(po), _ptr(pml), tile_rows, _ptr(dist_bias), nbias, _ptr(sink),
-                                     _ptr(sigmoid_bias), _stream())
+                                     _ptr(sigmoid_bias), int(keep), _stream())
         if rc == 0:
             r0 = tile_rows
         elif rc != 1:
@@ -2062,7 +2071,7 @@ def attn_mix(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, row_
                                       float(scale), float(softcap), _ptr(slopes), _ptr(talk), int(chunk), int(window),
                                       None if gate is None else gate.data_ptr() + r0 * ldg * esz, ldg, gch,
                                       out.data_ptr() + r0 * H * Dv * esz, _ptr(dist_bias), nbias, _ptr(sink),
-                                      _ptr(sigmoid_bias), _stream()),
+                                      _ptr(sigmoid_bias), int(keep), _stream()),
                "la_attn_mix_rows")
     return out
 
@@ -2093,38 +2102,50 @@ def router_sigmoid(xn: torch.Tensor, router: torch.Tensor, corr: Optional[torch.
     return ids, wts
 
 
-def router_softmax(xn: torch.Tensor, router: torch.Tensor, bias: Optional[torch.Tensor], topk: int) -> Tuple[torch.Tensor, torch.Tensor]:
+def router_softmax(xn: torch.Tensor, router: torch.Tensor, bias: Optional[torch.Tensor], topk: int, groups: int = 1,
+                   keep: int = 1, scale: float = 1.0) -> Tuple[torch.Tensor, torch.Tensor]:
     """Logit router: z = xn @ router^T + bias in fp32; the topk experts with the largest z are
-    chosen (ties: lowest expert id) and weighted by the softmax over the chosen logits only.
+    chosen (ties: lowest expert id) and weighted by the softmax over the chosen logits only (which is
+    also the chosen scores of a softmax over all experts, over their sum), times scale.  groups > 1:
+    experts form that many equal groups of neighbours, a group's score is its largest z, and only
+    experts of the `keep` best groups can be chosen.
     Returns (ids [T, topk] int32, weights [T * topk] fp32)."""
     T, D = xn.shape
     E = router.shape[0]
+    if E % groups or (groups > 1 and not (1 <= keep <= groups and topk <= keep * (E // groups))):
+        raise ValueError("router_softmax: equal groups, whose best `keep` hold at least topk experts")
     if not xn.is_cuda:
         z = xn.float() @ router.float().t()
         if bias is not None:
             z = z + bias.float()
+        if groups > 1:
+            best = torch.topk(z.view(T, groups, -1).amax(-1), keep, -1).indices
+            ok = torch.zeros(T, groups, dtype=torch.bool).scatter_(1, best, True)
+            z = z.masked_fill(~ok.repeat_interleave(E // groups, 1), float("-inf"))
         val, idx = torch.topk(z, topk, -1)
-        return idx.to(torch.int32), torch.softmax(val, -1).reshape(-1).float()
+        return idx.to(torch.int32), (torch.softmax(val, -1) * scale).reshape(-1).float()
     assert xn.dtype in (torch.bfloat16, torch.float32) and xn.stride(1) == 1
     assert router.dtype == torch.float32 and router.is_contiguous() and router.shape[1] == D
     assert bias is None or (bias.dtype == torch.float32 and bias.numel() == E and bias.is_contiguous())
     ids = torch.empty(T, topk, dtype=torch.int32, device=xn.device)
     wts = torch.empty(T * topk, dtype=torch.float32, device=xn.device)
     _check(lib().la_router_topk(int(xn.dtype == torch.float32), 1, xn.data_ptr(), xn.stride(0), router.data_ptr(),
-                                _ptr(bias), E, D, T, topk, 1, ids.data_ptr(), wts.data_ptr(), _stream()),
+                                _ptr(bias), E, D, T, topk, 1, int(groups), int(keep), float(scale), ids.data_ptr(),
+                                wts.data_ptr(), _stream()),
            "la_router_topk")
     return ids, wts
 
 
-def moe_pairs(x: torch.Tensor, wg: torch.Tensor, wu: torch.Tensor, wd: torch.Tensor, ids: torch.Tensor,
+def moe_pairs(x: torch.Tensor, wg: Optional[torch.Tensor], wu: torch.Tensor, wd: torch.Tensor, ids: torch.Tensor,
               wts: torch.Tensor, clamp: Optional[Tuple[float, float]] = None) -> torch.Tensor:
     """Routed gated experts as (token, expert) pair GEMVs on dense stacked weights (small batches,
     any width, no host sync): y[t] = sum_k wts[t, k] * Wd[e] (silu(Wg[e] x[t]) * (Wu[e] x[t])),
     e = ids[t, k].  wg / wu [E, F, D], wd [E, D, F] in x's dtype (bf16 or fp32).  Returns fp32 [T, D].
     clamp = (limit, slope): the clamped unit of glu_clamp instead of SiLU gating, g = min(Wg x,
-    limit), u = clamp(Wu x, -limit, limit), g sigmoid(slope g) (u + 1)."""
+    limit), u = clamp(Wu x, -limit, limit), g sigmoid(slope g) (u + 1).  wg None: ungated experts,
+    Wd[e] max(Wu[e] x, 0)^2."""
     T, D = x.shape
-    E, F = wg.shape[0], wg.shape[1]
+    E, F = wu.shape[0], wu.shape[1]
     topk = ids.shape[1]
     if not x.is_cuda:
         xf = x.float()
@@ -2133,21 +2154,23 @@ def moe_pairs(x: torch.Tensor, wg: torch.Tensor, wu: torch.Tensor, wd: torch.Ten
         for t in range(T):
             for k in range(topk):
                 e = int(ids[t, k])
-                g_, u_ = wg[e].float() @ xf[t], wu[e].float() @ xf[t]
-                if clamp is None:
+                g_, u_ = (None if wg is None else wg[e].float() @ xf[t]), wu[e].float() @ xf[t]
+                if wg is None:
+                    h = torch.relu(u_).square()
+                elif clamp is None:
                     h = torch.nn.functional.silu(g_) * u_
                 else:
                     g_ = torch.clamp(g_, max=clamp[0])
                     h = g_ * torch.sigmoid(clamp[1] * g_) * (torch.clamp(u_, -clamp[0], clamp[0]) + 1.0)
                 y[t] += wv[t, k] * (wd[e].float() @ h.to(x.dtype).float())
         return y
-    for w_ in (wg, wu, wd):
+    for w_ in (wu, wd) if wg is None else (wg, wu, wd):
         assert w_.dtype == x.dtype and w_.is_contiguous()
-    assert tuple(wu.shape) == (E, F, D) and tuple(wd.shape) == (E, D, F) and x.is_contiguous()
+    assert (wg is None or wg.shape == wu.shape) and tuple(wu.shape) == (E, F, D) and tuple(wd.shape) == (E, D, F) and x.is_contiguous()
     assert ids.dtype == torch.int32 and ids.is_contiguous() and wts.dtype == torch.float32
     h = torch.empty(T * topk, F, dtype=x.dtype, device=x.device)
     y = torch.empty(T, D, dtype=torch.float32, device=x.device)
-    _check(lib().la_moe_pairs(int(x.dtype == torch.float32), x.data_ptr(), wg.data_ptr(), wu.data_ptr(), wd.data_ptr(),
+    _check(lib().la_moe_pairs(int(x.dtype == torch.float32), x.data_ptr(), _ptr(wg), wu.data_ptr(), wd.data_ptr(),
                               ids.data_ptr(), wts.data_ptr(), T, topk, D, F, E, h.data_ptr(), y.data_ptr(),
                               int(clamp is not None), float(clamp[0]) if clamp else 0.0, float(clamp[1]) if clamp else 0.0,
                               _stream()),
@@ -2292,11 +2315,19 @@ def rot_freqs(dims: int, base: float, scaling: Optional[dict] = None, device=Non
     d(t) = dims ln(original / (2 pi t)) / (2 ln base), lo = max(floor d(fast), 0), hi = min(ceil
     d(slow), dims - 1) and ramp_i = clamp((i - lo) / max(hi - lo, 0.001), 0, 1) the frequency is
     f_i / factor * ramp_i + f_i (1 - ramp_i), and cos / sin are scaled by 0.1 ln(factor) + 1.
+    scaling {"factor", "low", "high", "original"} (the Llama 3.1 rule, magnitude 1): by wavelength
+    l = 2 pi / f_i, f_i stays below original / high, is f_i / factor above original / low, and
+    (1 - s) f_i / factor + s f_i between, s = (original / l - low) / (high - low).
     Computed in float64 on the host; the kernels form angles position * f_i in fp32."""
     half = dims // 2
     f = np.power(float(base), -2.0 * np.arange(half, dtype=np.float64) / dims)
     mag = 1.0
-    if scaling:
+    if scaling and "low" in scaling:
+        factor, low, high, orig = (float(scaling[n]) for n in ("factor", "low", "high", "original"))
+        turns = orig * f / (2.0 * math.pi)            # original / wavelength
+        s = np.clip((turns - low) / (high - low), 0.0, 1.0) if high != low else (turns > high).astype(np.float64)
+        f = np.where(turns > high, f, np.where(turns < low, f / factor, (1.0 - s) * f / factor + s * f))
+    elif scaling:
         factor, orig = float(scaling["factor"]), float(scaling["original"])
         d_of = lambda turns: dims * math.log(orig / (2.0 * math.pi * turns)) / (2.0 * math.log(base))  # noqa: E731
         lo = max(math.floor(d_of(float(scaling["fast"]))), 0)
@@ -2985,6 +3016,172 @@ def lightning(src: torch.Tensor, H: int, Dk: int, Dv: int, pos: torch.Tensor, cu
                               pos.data_ptr(), cu_q.data_ptr(), sslots.data_ptr(), state.data_ptr(), state.shape[0],
                               decay.data_ptr(), norm_w.data_ptr(), float(eps), o.data_ptr(), out.data_ptr(), _ptr(seg),
                               max_rows, _stream()), "la_lightning")
+    return out
+
+
+# ---------------------------------------------------------------------------------------
+# Layer-list designs: a residual of several streams, biased and unit-normed rotated heads, gated linear attention
+# ---------------------------------------------------------------------------------------
+
+def _split_bias(src):
+    """(the source without its bias, the bias fp32 or None) of a projection result."""
+    if isinstance(src, Partial) and src.bias is not None:
+        return Partial(src.t), src.bias
+    return src, None
+
+
+def hyper_streams(X: torch.Tensor, branch=None, mix: Optional[torch.Tensor] = None, out_w: Optional[torch.Tensor] = None,
+                  in_w: Optional[torch.Tensor] = None, norm: Optional[tuple] = None, init: Optional[torch.Tensor] = None,
+                  out_dtype: torch.dtype = torch.bfloat16) -> Optional[torch.Tensor]:
+    """Sublayer boundary of a residual kept as n streams (hyper-connections), X fp32 [T, n, D] updated in place:
+    with a branch (a sublayer's result [T, D], Partial with or without bias) every stream becomes
+    sum_from mix[from, to] X_from + out_w[to] branch, all from the old streams; then the next sublayer's input
+    u = sum_s in_w[s] X_s (in_w None: the plain sum) is returned through norm = (w, b, eps), a layer norm with
+    weight and bias.  norm None: nothing is returned.  init (fp32 [T, D]): the streams all start as its rows
+    (what X holds is not read).  mix fp32 [n, n], out_w / in_w fp32 [n].  All arithmetic fp32, one launch."""
+    T, n, D = X.shape
+    branch, bias = _split_bias(branch)
+    if branch is not None and (mix is None or tuple(mix.shape) != (n, n) or out_w is None or out_w.numel() != n):
+        raise ValueError("hyper_streams: a branch needs mix [n, n] and out_w [n]")
+    if (in_w is not None and in_w.numel() != n) or (init is not None and tuple(init.shape) != (T, D)):
+        raise ValueError("hyper_streams: operand shapes do not fit")
+    if not X.is_cuda:
+        if init is not None:
+            X.copy_(init.float().unsqueeze(1).expand(T, n, D))
+        if branch is not None:
+            y = _branch_dense(branch)
+            y = y if bias is None else y + bias.float()
+            X.copy_(torch.einsum("st,xsd->xtd", mix.float(), X) + out_w.float().view(1, n, 1) * y.unsqueeze(1))
+        if norm is None:
+            return None
+        u = X.sum(1) if in_w is None else torch.einsum("s,xsd->xd", in_w.float(), X)
+        return (_ln_ref(u, norm[0], float(norm[2])) + norm[1].float()).to(out_dtype)
+    if X.dtype != torch.float32 or not X.is_contiguous() or out_dtype not in (torch.float32, torch.bfloat16) or n > 16:
+        raise ValueError("hyper_streams: up to 16 contiguous fp32 streams; outputs are bf16 or fp32")
+    nw, nb, eps = norm if norm is not None else (None, None, 0.0)
+    for t, k in ((mix, n * n), (out_w, n), (in_w, n), (nw, D), (nb, D), (bias, D), (init, T * D)):
+        if t is not None and (t.dtype != torch.float32 or t.numel() != k or not t.is_contiguous() or not t.is_cuda):
+            raise ValueError("hyper_streams: weights, biases and the initial rows are contiguous fp32 on the device")
+    a = _branch_args(branch, T, D) if branch is not None else (None, 0, 0, 0)
+    out = torch.empty(T, D, dtype=out_dtype, device=X.device) if norm is not None else None
+    _check(lib().la_hyper_streams(X.data_ptr(), T, n, D, _ptr(init), a[0], a[1], a[2], a[3], _ptr(bias), _ptr(mix), _ptr(out_w),
+                                  _ptr(in_w), _ptr(nw), _ptr(nb), float(eps), _ptr(out), int(out_dtype == torch.float32),
+                                  _stream()), "la_hyper_streams")
+    return out
+
+
+def head_rope_pages(src, H: int, Dq: int, G: int, Dk: int, Dv: int, pos: torch.Tensor, slots: Optional[torch.Tensor],
+                    freqs: torch.Tensor, rot: int, interleaved: bool, k_cache: Optional[torch.Tensor] = None,
+                    v_cache: Optional[torch.Tensor] = None, unit_eps: Optional[float] = None,
+                    dtype: torch.dtype = torch.bfloat16) -> torch.Tensor:
+    """Heads of a projection into the attention's operands in one launch: src [T, H Dq + G Dk + G Dv] (q | k | v; a
+    Partial -- fp32 slabs or one matrix, its bias added here -- or a dense tensor of any row stride).  The first
+    `rot` dims of every query and key head are rotated by pos * freqs (pairs (2i, 2i + 1) when interleaved, else
+    (i, i + rot / 2)); with unit_eps every query and key head is then divided by sqrt(mean x^2 + unit_eps).
+    Returns q [T, H Dq] in dtype; keys and values go to the paged pools at `slots` (-1: nowhere).  G = 0: queries
+    only.  fp32 arithmetic."""
+    src, bias = _split_bias(src)
+    t = src.t if isinstance(src, Partial) else src
+    T, W = t.shape[-2], H * Dq + G * Dk + G * Dv
+    if (t.shape[-1] < W or (isinstance(src, Partial) and t.shape[-1] != W) or rot % 2 or rot > Dq or (G and rot > Dk)
+            or freqs.numel() != rot // 2 or pos.shape[0] != T or t.stride(-1) != 1):
+        raise ValueError("head_rope_pages: operand shapes do not fit")
+    if G and (k_cache is None or v_cache is None or slots is None or tuple(k_cache.shape[1:]) != (G, k_cache.shape[2], Dk)
+              or tuple(v_cache.shape[1:]) != (G, k_cache.shape[2] // 8, Dv, 8)):
+        raise ValueError("head_rope_pages: pools do not fit the key / value widths")
+    if not t.is_cuda:
+        x = _branch_dense(src)[:, :W]
+        x = x if bias is None else x + bias.float()
+        unit = (lambda y: y) if unit_eps is None else (lambda y: y * torch.rsqrt(y.pow(2).mean(-1, keepdim=True) + unit_eps))
+        q = unit(_rotate_ref(x[:, :H * Dq].reshape(T, H, Dq), pos, freqs, 1.0, rot, 0, interleaved))
+        if G:
+            k = unit(_rotate_ref(x[:, H * Dq:H * Dq + G * Dk].reshape(T, G, Dk), pos, freqs, 1.0, rot, 0, interleaved))
+            _page_write_ref(k_cache, v_cache, slots, k, x[:, H * Dq + G * Dk:].reshape(T, G, Dv))
+        return q.reshape(T, H * Dq).to(dtype)
+    if t.dim() == 3 or isinstance(src, Partial):
+        a = _branch_args(src, T, W)
+        ld = W
+    else:
+        a, ld = (t.data_ptr(), int(t.dtype == torch.float32), 0, 1), t.stride(0)
+    if t.dtype not in (torch.float32, torch.bfloat16) or dtype not in (torch.float32, torch.bfloat16):
+        raise ValueError("head_rope_pages: bf16 or fp32 rows and results")
+    if G and (k_cache.dtype != dtype or v_cache.dtype != dtype):
+        raise ValueError("head_rope_pages: pools hold the result's dtype")
+    if bias is not None and (bias.dtype != torch.float32 or bias.numel() != W or not bias.is_contiguous()):
+        raise ValueError("head_rope_pages: the bias is contiguous fp32 [q | k | v]")
+    assert pos.dtype == torch.int32 and freqs.dtype == torch.float32 and freqs.is_contiguous()
+    assert slots is None or (slots.dtype == torch.int32 and slots.shape[0] == T)
+    q = torch.empty(T, H * Dq, dtype=dtype, device=t.device)
+    _check(lib().la_head_rope_pages(int(dtype == torch.float32), a[0], a[1], a[2], a[3], ld, _ptr(bias), T, H, Dq, G, Dk, Dv,
+                                    pos.data_ptr(), _ptr(slots), freqs.data_ptr() if rot else None, rot, int(interleaved),
+                                    int(unit_eps is not None), float(unit_eps or 0.0), q.data_ptr(), _ptr(k_cache),
+                                    _ptr(v_cache), k_cache.shape[2] if G else 0, _stream()), "la_head_rope_pages")
+    return q
+
+
+GLA_CHUNK = 16       # tokens per chunk of a portion (gla.hip GL_C)
+GLA_MAX_KEY = 256    # widest key head of the kernels
+
+
+def gla(src: torch.Tensor, z: torch.Tensor, z_bias: torch.Tensor, tau: float, H: int, Dk: int, Dv: int, pos: torch.Tensor,
+        cu_q: torch.Tensor, sslots: torch.Tensor, state: torch.Tensor, norm_w: torch.Tensor, eps: float,
+        max_rows: int = 0) -> torch.Tensor:
+    """Gated linear attention over projection rows src [T, >= 2 H Dk + 2 H Dv] (q | k | v | gate, any row stride) and
+    decay logits z [T, H Dk]: alpha = sigmoid(z + z_bias)^(1 / tau) per head and key channel; per head
+    S <- diag(alpha) S + k v^T, o = S^T q Dk^-1/2; every head's o divided by its root mean square (eps), times
+    norm_w (fp32 [Dv], shared by the heads), times silu(gate).  Portions, state slots (fp32, retention_state's
+    layout) and max_rows as in ops.retention; decays, state, read-outs and the norm are fp32.  Batches of one row
+    per sequence stream the state once; portions are computed chunk by chunk on the fp32 matrix
+    instructions.  Returns [T, H Dv] in src's dtype."""
+    T = src.shape[0]
+    nseq = cu_q.shape[0] - 1
+    Cq, Cv = H * Dk, H * Dv
+    if (src.dim() != 2 or src.shape[1] < 2 * Cq + 2 * Cv or src.stride(1) != 1 or tuple(z.shape) != (T, Cq)
+            or z_bias.numel() != Cq or tuple(state.shape[1:]) != (H, Dv, Dk) or norm_w.numel() != Dv
+            or sslots.shape[0] != nseq or pos.shape[0] != T or not tau > 0):
+        raise ValueError("gla: operand shapes do not fit")
+    if not src.is_cuda:
+        x = src[:, :2 * Cq + 2 * Cv].float()
+        q, k = x[:, :Cq].reshape(T, H, Dk) * Dk ** -0.5, x[:, Cq:2 * Cq].reshape(T, H, Dk)
+        v, g = x[:, 2 * Cq:2 * Cq + Cv].reshape(T, H, Dv), x[:, 2 * Cq + Cv:]
+        al = torch.exp(torch.nn.functional.logsigmoid(z.float() + z_bias.float()) / tau).view(T, H, Dk)
+        o = torch.zeros(T, H, Dv)
+        cu = cu_q.tolist()
+        for s in range(nseq):
+            a, b = cu[s], cu[s + 1]
+            if b <= a:
+                continue
+            ss = int(sslots[s])
+            S = torch.zeros(H, Dk, Dv) if int(pos[a]) == 0 or ss < 0 else state[ss].float().transpose(1, 2).clone()
+            for t in range(a, b):
+                S = al[t].unsqueeze(2) * S + k[t].unsqueeze(2) * v[t].unsqueeze(1)
+                o[t] = torch.einsum("hkv,hk->hv", S, q[t])
+            if ss >= 0:
+                state[ss] = S.transpose(1, 2)
+        return (_rms_ref(o, norm_w, eps).reshape(T, Cv) * torch.nn.functional.silu(g)).to(src.dtype)
+    if src.dtype not in (torch.float32, torch.bfloat16) or z.dtype != src.dtype or not z.is_contiguous():
+        raise ValueError("gla: bf16 or fp32 rows, contiguous decay logits of the same dtype")
+    if state.dtype != torch.float32 or not state.is_contiguous():
+        raise ValueError("gla: the state pool is contiguous fp32")
+    for t in (pos, cu_q, sslots):
+        assert t.dtype == torch.int32 and t.is_cuda and t.is_contiguous()
+    for t in (z_bias, norm_w):
+        assert t.dtype == torch.float32 and t.is_contiguous() and t.is_cuda
+    if Dk > GLA_MAX_KEY:
+        raise ValueError(f"gla: key heads up to {GLA_MAX_KEY} wide")
+    out = torch.empty(T, Cv, dtype=src.dtype, device=src.device)
+    max_rows = int(max_rows) if max_rows > 0 else T
+    single = T == nseq and max_rows == 1
+    qd = kd = dl = am = o = None
+    if not single:
+        n, W = (T // GLA_CHUNK + nseq) * H, int(lib().la_gla_width(Dk))
+        f32 = dict(dtype=torch.float32, device=src.device)
+        qd, kd = torch.empty(n * GLA_CHUNK * W, **f32), torch.empty(n * GLA_CHUNK * W, **f32)
+        dl, am, o = torch.empty(n * W, **f32), torch.empty(n * GLA_CHUNK * GLA_CHUNK, **f32), torch.empty(T, Cv, **f32)
+    _check(lib().la_gla(int(src.dtype == torch.float32), src.data_ptr(), src.stride(0), z.data_ptr(), z_bias.data_ptr(),
+                        float(tau), T, nseq, H, Dk, Dv, pos.data_ptr(), cu_q.data_ptr(), sslots.data_ptr(), state.data_ptr(),
+                        state.shape[0], norm_w.data_ptr(), float(eps), int(single), max_rows, _ptr(qd), _ptr(kd), _ptr(dl),
+                        _ptr(am), _ptr(o), out.data_ptr(), _stream()), "la_gla")
     return out
 
 

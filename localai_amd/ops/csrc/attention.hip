@@ -117,7 +117,8 @@ LA_DEV void rope_src_load(const DecRope& R, int b, int col, float (&v)[N]) {
 // denominator once, without key or value (counted by wave 0 of the first partition).
 // sig: a bias per head that replaces the softmax: a visible key's weight is sigmoid(score + sig[head]),
 // not normalised over the keys (the running maximum stays 0, the running sum 1).  chunk: keys of the
-// query's chunk of that many positions only (0: all).  gate: a logit per output channel (row stride
+// query's chunk of that many positions only (0: all).  keep: beside the window's or chunk's keys, the
+// first `keep` keys of the sequence are visible.  gate: a logit per output channel (row stride
 // ldg), the output times its sigmoid.
 struct DecExtra {
   const float* bias;
@@ -127,6 +128,7 @@ struct DecExtra {
   int chunk;
   const bf16* gate;
   long ldg;
+  int keep;
 };
 
 LA_DEV float gate_at(const DecExtra& E, long row, int col) {
@@ -136,7 +138,8 @@ LA_DEV float gate_at(const DecExtra& E, long row, int col) {
 // K/V are streamed once per decode step: non-temporal loads (the default) read them 12-14 %
 // faster at batch 256 (5.05 -> 5.70 TB/s at 256 keys, 5.21 -> 5.98 at 384;
 // profiles/r4_attn_decode_nt.md).  VAR bit 0 = ordinary cached loads (A/B only); bit 1 = keys
-// two tiles ahead (measured no faster; kept for the A/B); bit 2 = sigmoid weights (DecExtra sig).
+// two tiles ahead (measured no faster; kept for the A/B); bit 2 = sigmoid weights (DecExtra sig);
+// bit 3 = kept first keys (DecExtra keep).
 template <int DH, int GT, int NW, int VAR = 0>
 __global__ __launch_bounds__(NW * 64) __attribute__((amdgpu_waves_per_eu(2))) void attn_decode_kernel(
     const bf16* __restrict__ q, const bf16* __restrict__ kc, const bf16* __restrict__ vc,
@@ -168,6 +171,12 @@ __global__ __launch_bounds__(NW * 64) __attribute__((amdgpu_waves_per_eu(2))) vo
   const int nbt = (kend - t0 + BS - 1) / BS;
   const int* bt = block_tables + (long)b * max_blocks + t0 / BS;
   for (int i = tid; i < nbt; i += NT) sh.bt[i] = bt[i];
+  // Kept keys in front of the first partition: [0, klim), klim <= base.  They belong to partition 0, whose waves
+  // take their 32-key tiles before their own; the table entries follow the partition's in LDS.
+  constexpr bool KEEP = (VAR & 8) != 0;
+  const int klim = KEEP && p == 0 ? min(E.keep, base) : 0;
+  if constexpr (KEEP)
+    for (int i = tid; i * BS < klim; i += NT) sh.bt[nbt + i] = block_tables[(long)b * max_blocks + i];
 
   // Q^T fragments: lane holds Q[head r][d = 32c + 8g .. +8]
   bf16x8 qf[KC];
@@ -230,12 +239,17 @@ __global__ __launch_bounds__(NW * 64) __attribute__((amdgpu_waves_per_eu(2))) vo
     if constexpr (NTL) return __builtin_nontemporal_load((const bf16x8*)p);
     else return *(const bf16x8*)p;
   };
+  auto block_of = [&](int key) {
+    if constexpr (KEEP) return sh.bt[key < klim ? nbt + key / BS : (key - t0) / BS];
+    else return sh.bt[(key - t0) / BS];
+  };
+  auto limit_of = [&](int kb) { return KEEP && kb < klim ? klim : kend; };
   auto load_k = [&](int kb, bf16x8 (&K)[2][(DH + 31) / 32]) {
 #pragma unroll
     for (int t = 0; t < 2; ++t) {
       // K row r of MFMA t: key kb + 8(r>>2) + 4t + (r&3) (clamped to a real key)
-      const int kk = min(kb + 8 * (r >> 2) + 4 * t + (r & 3), kend - 1);
-      const long pk = (long)sh.bt[(kk - t0) / BS] * Hkv * BS * DH + head_off;
+      const int kk = min(kb + 8 * (r >> 2) + 4 * t + (r & 3), limit_of(kb) - 1);
+      const long pk = (long)block_of(kk) * Hkv * BS * DH + head_off;
       const bf16* krow = kc + pk + (long)(kk % BS) * DH;
 #pragma unroll
       for (int c = 0; c < KC; ++c) {
@@ -246,8 +260,8 @@ __global__ __launch_bounds__(NW * 64) __attribute__((amdgpu_waves_per_eu(2))) vo
   };
   auto load_v = [&](int kb, bf16x8 (&V)[DH / 16]) {
     // V^T: keys kb + 8g .. +7 at d (an 8-aligned run inside one page, clamped to a real key)
-    const int kv = min(kb + 8 * g, kend - 1) & ~7;
-    const long pv = (long)sh.bt[(kv - t0) / BS] * Hkv * BS * DH + head_off;
+    const int kv = min(kb + 8 * g, limit_of(kb) - 1) & ~7;
+    const long pv = (long)block_of(kv) * Hkv * BS * DH + head_off;
 #pragma unroll
     for (int nd = 0; nd < ND; ++nd) {
       const int d = 16 * nd + r;
@@ -281,23 +295,30 @@ __global__ __launch_bounds__(NW * 64) __attribute__((amdgpu_waves_per_eu(2))) vo
   constexpr bool DB = DH <= 128;
   // K2: keys two tiles ahead (V stays one ahead: a whole second tile does not fit in 256 VGPRs)
   constexpr bool K2 = (VAR & 2) != 0;
-  int kb = t0 + 32 * wave;
-  if (wlo > kb) kb += (wlo - kb) / (32 * NW) * (32 * NW);   // this wave's tiles that end before the first visible key
+  int kb0 = t0 + 32 * wave;
+  // this wave's tiles that end before the first visible key (unless there are kept keys among them)
+  if (wlo > kb0 && !(KEEP && E.keep > base)) kb0 += (wlo - kb0) / (32 * NW) * (32 * NW);
+  auto next_of = [&](int k) {          // the wave's tile after k (from its last kept tile to its first own)
+    const int n = k + 32 * NW;
+    return KEEP && k < klim && n >= klim ? kb0 : n;
+  };
+  int kb = KEEP && 32 * wave < klim ? 32 * wave : kb0;
   if (kb < kend) {
     DecTile<DH> cur, nxt;
     bf16x8 k2[2][(DH + 31) / 32];
     if constexpr (DB) {
       load_tile(kb, cur);
       if constexpr (K2)
-        if (kb + 32 * NW < kend) load_k(kb + 32 * NW, nxt.k);
+        if (next_of(kb) < kend) load_k(next_of(kb), nxt.k);
     }
-    for (; kb < kend; kb += 32 * NW) {
+    for (int kn; kb < kend; kb = kn) {
+      kn = next_of(kb);
       if constexpr (DB) {
         if constexpr (K2) {
-          if (kb + 2 * 32 * NW < kend) load_k(kb + 2 * 32 * NW, k2);
-          if (kb + 32 * NW < kend) load_v(kb + 32 * NW, nxt.v);
+          if (next_of(kn) < kend) load_k(next_of(kn), k2);
+          if (kn < kend) load_v(kn, nxt.v);
         } else {
-          if (kb + 32 * NW < kend) load_tile(kb + 32 * NW, nxt);
+          if (kn < kend) load_tile(kn, nxt);
         }
       } else {
         load_tile(kb, cur);
@@ -319,7 +340,7 @@ __global__ __launch_bounds__(NW * 64) __attribute__((amdgpu_waves_per_eu(2))) vo
           // sliding-window attention (keys at least `window` positions behind the query masked)
           float sv = cap_l2 > 0.f ? cap_l2 * tanhf(acc[i] * cap_mul) : acc[i] * scale_log2;
           if (E.bias) sv = fmaf(E.bias[(long)min(max(L - 1 - key, 0), E.nbias - 1) * Hq + hq_r], 1.4426950408889634f, sv);
-          s[t][i] = (key < kend && key >= wlo) ? sv : -INFINITY;
+          s[t][i] = (key < limit_of(kb) && (key >= wlo || (KEEP && key < E.keep))) ? sv : -INFINITY;
         }
       }
       bf16x8 pa;
@@ -511,7 +532,7 @@ __global__ __launch_bounds__(PF_T) void attn_prefill_kernel(
     const int* __restrict__ ctx_lens,       // [nseq] total keys (cached + new)
     const int* __restrict__ block_tables, int max_blocks, int Hq, int Hkv, int BS, float scale,
     bf16* __restrict__ out, float cap, int window, long ldq = 0, long ldk = 0, long ldv = 0, long ldo = 0,
-    DecExtra E = DecExtra{nullptr, 0, nullptr, nullptr, 0, nullptr, 0}) {
+    DecExtra E = DecExtra{nullptr, 0, nullptr, nullptr, 0, nullptr, 0, 0}) {
   constexpr int DP = (DH + 31) / 32 * 32;  // padded head dim for the MFMA k loop
   constexpr int KC = DP / 32;               // k-chunks of 32
   constexpr int ND = DP / 16;               // 16-wide output column tiles
@@ -566,7 +587,11 @@ __global__ __launch_bounds__(PF_T) void attn_prefill_kernel(
     if (window > 0) kbeg = max(kbeg, pos0 + r0 - window + 1);
     if (E.chunk > 0) kbeg = max(kbeg, (pos0 + r0) / E.chunk * E.chunk);
   }
-  for (int k0 = kbeg / PF_KT * PF_KT; k0 < kend; k0 += PF_KT) {
+  // tiles in order: those holding kept keys before kbeg, then kbeg's and after
+  const int tbeg = kbeg / PF_KT, tkeep = DENSE ? 0 : min((E.keep + PF_KT - 1) / PF_KT, tbeg);
+  for (int nt = 0;; ++nt) {
+    const int k0 = (nt < tkeep ? nt : tbeg + nt - tkeep) * PF_KT;
+    if (k0 >= kend) break;
     __syncthreads();
     // stage the K tile (row-major) and the V^T tile ([d][key], copied from the transposed cache)
     for (int cidx = tid; cidx < PF_KT * (DP / 8); cidx += PF_T) {
@@ -642,8 +667,8 @@ __global__ __launch_bounds__(PF_T) void attn_prefill_kernel(
       int wlo = window > 0 ? qpos - window + 1 : 0;
       if (!DENSE && E.chunk > 0) wlo = max(wlo, qpos / E.chunk * E.chunk);
       const bool causal = !DENSE;
-      if ((causal && key0 > qpos) || key0 >= kend || qr >= qlen || key0 < wlo) v0 = -INFINITY;
-      if ((causal && key1 > qpos) || key1 >= kend || qr >= qlen || key1 < wlo) v1 = -INFINITY;
+      if ((causal && key0 > qpos) || key0 >= kend || qr >= qlen || (key0 < wlo && key0 >= E.keep)) v0 = -INFINITY;
+      if ((causal && key1 > qpos) || key1 >= kend || qr >= qlen || (key1 < wlo && key1 >= E.keep)) v1 = -INFINITY;
       if constexpr (SIG) {   // weights of their own, no softmax; hidden keys: -inf, weight 0
         ps[wave][(4 * fq + i) * VS + fr] = (bf16)(1.f / (1.f + exp2f(-(v0 + sig_l2))));
         ps[wave][(4 * fq + i) * VS + 16 + fr] = (bf16)(1.f / (1.f + exp2f(-(v1 + sig_l2))));
@@ -710,7 +735,7 @@ extern "C" int la_attn_decode(const void* q, const void* kc, const void* vc, con
                               long rope_slab, int rope_S, const void* rope_bias, const int* pos, const int* slots,
                               const float* cos_sin, float softcap, int window, int nw, const float* dist_bias,
                               int nbias, const float* sink, const float* sig, int chunk, const void* gate, long ldg,
-                              void* stream) {
+                              int keep, void* stream) {
   // nw bit 8: split even short sequences over the grid's partitions (few sequences: the
   // parallelism is worth the merge); otherwise a sequence of <= DEC_ONE_PART keys is one partition
   const int one_part = (nw & 256) ? 0 : g_dec_one_part;
@@ -723,8 +748,8 @@ extern "C" int la_attn_decode(const void* q, const void* kc, const void* vc, con
   if (rope_p && ((Dh & 31) || !pos || !slots || !cos_sin || rope_S < 0)) return -1;
   if (!rope_p && !q) return -1;
   const la::DecRope R{rope_p, rope_slab, rope_S, (const float*)rope_bias, pos, slots, cos_sin, (Hq + 2 * Hkv) * Dh};
-  if ((dist_bias && nbias < 1) || (sink && sig) || chunk < 0 || (gate && ldg < (long)Hq * Dh)) return -1;
-  const la::DecExtra E{dist_bias, nbias, sink, sig, chunk, (const bf16*)gate, ldg};
+  if ((dist_bias && nbias < 1) || (sink && sig) || chunk < 0 || keep < 0 || (gate && ldg < (long)Hq * Dh)) return -1;
+  const la::DecExtra E{dist_bias, nbias, sink, sig, chunk, (const bf16*)gate, ldg, keep};
   const int G = Hq / Hkv;
   hipStream_t st = (hipStream_t)stream;
   dim3 grid(P, Hkv, B);
@@ -742,24 +767,34 @@ extern "C" int la_attn_decode(const void* q, const void* kc, const void* vc, con
   hipLaunchKernelGGL((la::attn_decode_kernel<D, GT, NW, V>), grid, dim3(NW * 64), 0, st, (const bf16*)q,        \
                      (const bf16*)kc, (const bf16*)vc, block_tables, max_blocks, seq_lens, Hkv, G, BS, sl2, PS,  \
                      (bf16*)out, po, pml, P, tk, R, cap_l2, cap_mul, window, one_part, E)
-  if (sig) {   // sigmoid weights: fewer instances (GT only sizes the cross-wave merge)
-#define DEC_SIG(D)                                             \
+  // sigmoid weights, kept keys: fewer instances (GT only sizes the cross-wave merge)
+#define DEC_FEW(D, V)                                          \
   case D:                                                      \
     if (G <= 4) {                                              \
-      if (nw == 1) DEC_LAUNCH(D, 4, 1, 4);                     \
-      else DEC_LAUNCH(D, 4, 4, 4);                             \
+      if (nw == 1) DEC_LAUNCH(D, 4, 1, V);                     \
+      else DEC_LAUNCH(D, 4, 4, V);                             \
     } else {                                                   \
-      if (nw == 1) DEC_LAUNCH(D, 16, 1, 4);                    \
-      else DEC_LAUNCH(D, 16, 4, 4);                            \
+      if (nw == 1) DEC_LAUNCH(D, 16, 1, V);                    \
+      else DEC_LAUNCH(D, 16, 4, V);                            \
     }                                                          \
     break;
-    switch (Dh) {
-      DEC_SIG(64) DEC_SIG(80) DEC_SIG(96) DEC_SIG(128) DEC_SIG(192) DEC_SIG(256)
-      default: return -2;
-    }
-#undef DEC_SIG
+#define DEC_FEWS(V)                                                                                    \
+  switch (Dh) {                                                                                        \
+    DEC_FEW(64, V) DEC_FEW(80, V) DEC_FEW(96, V) DEC_FEW(128, V) DEC_FEW(192, V) DEC_FEW(256, V)       \
+    default: return -2;                                                                                \
+  }
+  if (sig) {
+    if (keep) return -4;
+    DEC_FEWS(4)
     return (int)hipGetLastError();
   }
+  if (keep) {
+    if (PS / BS + (keep + BS - 1) / BS > la::DEC_MAXBT) return -4;
+    DEC_FEWS(8)
+    return (int)hipGetLastError();
+  }
+#undef DEC_FEWS
+#undef DEC_FEW
 #define DEC_NW(D, GT, NW)                                                  \
   do {                                                                     \
     if constexpr (D == 128 && GT == 4 && NW == 1) {                        \
@@ -826,9 +861,9 @@ extern "C" int la_attn_prefill(const void* q, const void* kc, const void* vc, co
                                const int* cu_q, const int* ctx_lens, const int* block_tables, int max_blocks, int Hq,
                                int Hkv, int Dh, int BS, float scale, void* out, float softcap, int window,
                                const float* dist_bias, int nbias, const float* sink, const float* sig, int chunk,
-                               const void* gate, long ldg, void* stream) {
-  if (Hq % Hkv || (dist_bias && nbias < 1) || (sink && sig) || chunk < 0 || (gate && ldg < (long)Hq * Dh)) return -1;
-  const la::DecExtra E{dist_bias, nbias, sink, sig, chunk, (const bf16*)gate, ldg};
+                               const void* gate, long ldg, int keep, void* stream) {
+  if (keep < 0 || Hq % Hkv || (dist_bias && nbias < 1) || (sink && sig) || chunk < 0 || (gate && ldg < (long)Hq * Dh)) return -1;
+  const la::DecExtra E{dist_bias, nbias, sink, sig, chunk, (const bf16*)gate, ldg, keep};
   hipStream_t st = (hipStream_t)stream;
   dim3 grid(ntiles, Hq);
 #define PF_LAUNCH(D, SG)                                                                                          \

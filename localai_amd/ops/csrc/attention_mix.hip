@@ -3,7 +3,8 @@
 //   s_g(i, j)  = softcap * tanh(scale * q_g(i) . k(j) / softcap)          (softcap 0: none)
 //                - slope_g * (i - j)                                       (slopes null: none)
 //   s'_h(i, j) = sum_g talk[h][g] * s_g(i, j)                              (talk null: identity)
-//   visible j:   j <= i, same chunk of `chunk` positions (chunk 0: all), within `window` (0: all)
+//   visible j:   j <= i, same chunk of `chunk` positions (chunk 0: all), within `window` (0: all);
+//                beside those, the first `keep` keys of the sequence (keep 0: none)
 //   o_h(i)     = gate_h(i) * sum_j softmax_j(s'_h(i, .)) v(j)              (gate null: 1)
 //
 // or, with a bias `sig` per head, without a softmax: the weight of a visible key is
@@ -63,7 +64,7 @@ __global__ __launch_bounds__(AM_NT) void attn_mix_rows_kernel(
     const int* __restrict__ pos, const int* __restrict__ bt, int maxb, int H, int G, int Dk, int Dv, int BS,
     float scale, float softcap, const float* __restrict__ slopes, const float* __restrict__ talk, int chunk,
     int window, const AT* __restrict__ gate, int ldg, int gch, AT* __restrict__ out, const float* __restrict__ dbias,
-    int nbias, const float* __restrict__ sink, const float* __restrict__ sig) {
+    int nbias, const float* __restrict__ sink, const float* __restrict__ sig, int keep) {
   extern __shared__ float lds[];
   float* qs = lds;                       // [H][Dk]
   float* s1 = qs + H * Dk;               // [H][KT] raw scores
@@ -91,14 +92,17 @@ __global__ __launch_bounds__(AM_NT) void attn_mix_rows_kernel(
 #pragma unroll
   for (int e = 0; e < AM_MAXO; ++e) acc[e] = 0.f;
   __syncthreads();
-  for (int j0 = lo; j0 <= i; j0 += AM_KT) {
-    const int nk = min(AM_KT, i + 1 - j0);
+  // the visible keys in order: the kept ones before lo, then lo .. i; n-th visible key -> its position
+  const int kept = min(keep, lo), nvis = kept + i + 1 - lo;
+  auto key_at = [&](int n) { return n < kept ? n : lo + n - kept; };
+  for (int j0 = 0; j0 < nvis; j0 += AM_KT) {
+    const int nk = min(AM_KT, nvis - j0);
     // raw scores of every (head, key) pair of the tile
     for (int e = tid; e < H * AM_KT; e += AM_NT) {
       const int h = e / AM_KT, jj = e - h * AM_KT;
       float s = -INFINITY;
       if (jj < nk) {
-        const int j = j0 + jj, blk = tab[j / BS], off = j % BS, g = h / rep;
+        const int j = key_at(j0 + jj), blk = tab[j / BS], off = j % BS, g = h / rep;
         s = dot_row<AT>(qs + h * Dk, kc + (((long)blk * G + g) * BS + off) * Dk, Dk, vec) * scale;
         if (softcap > 0.f) s = softcap * tanhf(s / softcap);
         if (slopes) s -= slopes[h] * (float)(i - j);
@@ -151,12 +155,12 @@ __global__ __launch_bounds__(AM_NT) void attn_mix_rows_kernel(
         float a = acc[e] * alpha[h];
         if (vc) {
           for (int jj = 0; jj < nk; ++jj) {
-            const int j = j0 + jj, blk = tab[j / BS], off = j % BS;
+            const int j = key_at(j0 + jj), blk = tab[j / BS], off = j % BS;
             a = fmaf(s2[h * AM_KT + jj], (float)vc[((((long)blk * G + g) * (BS >> 3) + (off >> 3)) * Dv + d) * 8 + (off & 7)], a);
           }
         } else {   // no V pages: a key row's first Dv columns are its value (latent caches)
           for (int jj = 0; jj < nk; ++jj) {
-            const int j = j0 + jj, blk = tab[j / BS], off = j % BS;
+            const int j = key_at(j0 + jj), blk = tab[j / BS], off = j % BS;
             a = fmaf(s2[h * AM_KT + jj], (float)kc[(((long)blk * G + g) * BS + off) * Dk + d], a);
           }
         }
@@ -204,7 +208,7 @@ __global__ __launch_bounds__(NW * 64) void attn_mix_tile_kernel(
     const float* __restrict__ slopes, const float* __restrict__ talk, int chunk, int window,
     const bf16* __restrict__ gate, int ldg, int gch, bf16* __restrict__ out, int nsplit, float* __restrict__ part_o,
     float* __restrict__ part_ml, const float* __restrict__ dbias, int nbias, const float* __restrict__ sink,
-    const float* __restrict__ sig) {
+    const float* __restrict__ sig, int keep) {
   extern __shared__ float lds[];
   float* s1 = lds;                           // [H][16][AT_SS]
   float* mrun = s1 + H * 16 * AT_SS;         // [H * 16]
@@ -255,19 +259,22 @@ __global__ __launch_bounds__(NW * 64) void attn_mix_tile_kernel(
   // blockIdx.y = key split: every nsplit-th key tile (decode rows: few query rows, many keys).
   // Block-table entries are read one tile ahead (K fragments) or a phase ahead (V fragments), so
   // no fragment load waits behind a dependent table load.
-  const int jfirst = (lo0 / AT_KT + (int)blockIdx.y) * AT_KT;
+  // Tiles in order: those holding kept keys before the first row's window, then the window's.
+  const int tlo = lo0 / AT_KT, tkeep = min((keep + AT_KT - 1) / AT_KT, tlo);
+  auto tile_at = [&](int n) { return (n < tkeep ? n : tlo + n - tkeep) * AT_KT; };
   int nextA[2];
 #pragma unroll
   for (int ns = 0; ns < 2; ++ns) {
-    const int key = jfirst + 16 * ns + fr;
+    const int key = tile_at(blockIdx.y) + 16 * ns + fr;
     nextA[ns] = key <= last ? tab[key / BS] : -1;
   }
-  for (int j0 = jfirst; j0 <= last; j0 += AT_KT * nsplit) {
+  for (int nt = blockIdx.y; tile_at(nt) <= last; nt += nsplit) {
+    const int j0 = tile_at(nt), jn = tile_at(nt + nsplit);
     int blkA[2];
 #pragma unroll
     for (int ns = 0; ns < 2; ++ns) {
       blkA[ns] = nextA[ns];
-      const int key = j0 + AT_KT * nsplit + 16 * ns + fr;
+      const int key = jn + 16 * ns + fr;
       nextA[ns] = key <= last ? tab[key / BS] : -1;
     }
     const int key8 = j0 + 8 * fq;
@@ -359,7 +366,7 @@ __global__ __launch_bounds__(NW * 64) void attn_mix_tile_kernel(
       const int key = j0 + kk, qpos = pos0 + qr;
       int lo = chunk > 0 ? (qpos / chunk) * chunk : 0;
       if (window > 0) lo = max(lo, qpos - window + 1);
-      const bool vis = qr < nrow && key <= qpos && key >= lo;
+      const bool vis = qr < nrow && key <= qpos && (key >= lo || key < keep);
 #pragma unroll
       for (int mb = 0; mb < 4; ++mb) {
         if (mb < MB) {
@@ -539,14 +546,14 @@ static int launch_tile(int nsplit, void* part_o, void* part_ml, int ntiles, size
                        const void* tiles, const void* cu_q, const void* pos, const void* bt, int maxb, int H, int G,
                        int Dk, int Dv, int BS, float scale, float softcap, const void* slopes, const void* talk,
                        int chunk, int window, const void* gate, int ldg, int gch, void* out, const void* dbias, int nbias,
-                       const void* sink, const void* sig) {
+                       const void* sink, const void* sig, int keep) {
   auto k = attn_mix_tile_kernel<NW, HPW, NDV>;
   if (shm > 48 * 1024) (void)hipFuncSetAttribute((const void*)k, hipFuncAttributeMaxDynamicSharedMemorySize, (int)shm);
   hipLaunchKernelGGL(k, dim3(ntiles, nsplit), dim3(NW * 64), shm, s, (const bf16*)q, (const bf16*)kc, (const bf16*)vc,
                      (const int*)tiles, (const int*)cu_q, (const int*)pos, (const int*)bt, maxb, H, G, Dk, Dv, BS, scale,
                      softcap, (const float*)slopes, (const float*)talk, chunk, window, (const bf16*)gate, ldg, gch,
                      (bf16*)out, nsplit, (float*)part_o, (float*)part_ml, (const float*)dbias, nbias, (const float*)sink,
-                     (const float*)sig);
+                     (const float*)sig, keep);
   return (int)hipGetLastError();
 }
 
@@ -556,8 +563,9 @@ extern "C" int la_attn_mix_rows(int f32, const void* q, const void* kc, const vo
                                 const void* pos, const void* bt, int maxb, int T, int H, int G, int Dk, int Dv, int BS,
                                 float scale, float softcap, const void* slopes, const void* talk, int chunk, int window,
                                 const void* gate, int ldg, int gch, void* out, const void* dbias, int nbias,
-                                const void* sink, const void* sig, void* stream) {
+                                const void* sink, const void* sig, int keep, void* stream) {
   using namespace la;
+  if (keep < 0) return -1;
   if (T <= 0 || H <= 0 || G <= 0 || H % G || H * Dv > AM_NT * AM_MAXO || (dbias && nbias < 1) || (sink && sig)) return -1;
   const size_t shm = sizeof(float) * ((size_t)H * Dk + 2 * (size_t)H * AM_KT + 3 * (size_t)H);
   if (shm > 160 * 1024) return -2;
@@ -568,14 +576,14 @@ extern "C" int la_attn_mix_rows(int f32, const void* q, const void* kc, const vo
     hipLaunchKernelGGL((attn_mix_rows_kernel<float>), dim3(T), dim3(AM_NT), shm, s, (const float*)q, (const float*)kc,
                        (const float*)vc, (const int*)row_seq, (const int*)pos, (const int*)bt, maxb, H, G, Dk, Dv, BS,
                        scale, softcap, (const float*)slopes, (const float*)talk, chunk, window, (const float*)gate, ldg, gch,
-                       (float*)out, (const float*)dbias, nbias, (const float*)sink, (const float*)sig);
+                       (float*)out, (const float*)dbias, nbias, (const float*)sink, (const float*)sig, keep);
   } else {
     if (shm > 48 * 1024)
       (void)hipFuncSetAttribute((const void*)attn_mix_rows_kernel<bf16>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)shm);
     hipLaunchKernelGGL((attn_mix_rows_kernel<bf16>), dim3(T), dim3(AM_NT), shm, s, (const bf16*)q, (const bf16*)kc,
                        (const bf16*)vc, (const int*)row_seq, (const int*)pos, (const int*)bt, maxb, H, G, Dk, Dv, BS,
                        scale, softcap, (const float*)slopes, (const float*)talk, chunk, window, (const bf16*)gate, ldg, gch,
-                       (bf16*)out, (const float*)dbias, nbias, (const float*)sink, (const float*)sig);
+                       (bf16*)out, (const float*)dbias, nbias, (const float*)sink, (const float*)sig, keep);
   }
   return (int)hipGetLastError();
 }
@@ -591,8 +599,9 @@ extern "C" int la_attn_mix_tiles(const void* q, const void* kc, const void* vc, 
                                  int Dv, int BS, float scale, float softcap, const void* slopes, const void* talk,
                                  int chunk, int window, const void* gate, int ldg, int gch, void* out, int nsplit,
                                  void* part_o, void* part_ml, int rows, const void* dbias, int nbias, const void* sink,
-                                 const void* sig, void* stream) {
+                                 const void* sig, int keep, void* stream) {
   using namespace la;
+  if (keep < 0) return -1;
   if (ntiles <= 0 || H <= 0 || G <= 0 || H % G || nsplit < 1 || nsplit > 64 || (nsplit > 1 && (!part_o || !part_ml)) ||
       (dbias && nbias < 1) || (sink && sig))
     return -1;
@@ -607,7 +616,7 @@ extern "C" int la_attn_mix_tiles(const void* q, const void* kc, const void* vc, 
   if (rc == 1 && nw == NW && hpw <= HPW && ndv == NDV)                                                             \
     rc = launch_tile<NW, HPW, NDV>(nsplit, part_o, part_ml, ntiles, shm, s, q, kc, vc, tiles, cu_q, pos, bt, maxb, H, \
                                    G, Dk, Dv, BS, scale, softcap, slopes, talk, chunk, window, gate, ldg, gch, out,       \
-                                   dbias, nbias, sink, sig);
+                                   dbias, nbias, sink, sig, keep);
   LA_TILE(4, 1, 2) LA_TILE(4, 1, 4) LA_TILE(4, 1, 8) LA_TILE(4, 2, 2) LA_TILE(4, 2, 4) LA_TILE(4, 2, 8)
   LA_TILE(8, 2, 2) LA_TILE(8, 2, 4) LA_TILE(8, 2, 8) LA_TILE(8, 4, 2) LA_TILE(8, 4, 4) LA_TILE(8, 4, 8)
 #undef LA_TILE

@@ -1,8 +1,10 @@
 // Mixture-of-experts pieces for dense (bf16 / fp32) expert weights of any width:
 //   * a router with sigmoid scores, an optional selection-only correction and normalised weights,
-//     or with biased logits and the softmax over the chosen logits as weights;
+//     or with biased logits and the softmax over the chosen logits as weights; optionally only experts of
+//     the best groups of neighbouring experts can be chosen;
 //   * the routed experts of small batches as (token, expert) pair GEMVs: gate|up with the SiLU
-//     gating fused, then the down projection with the weighted top-k combine fused, no atomics.
+//     gating fused (or an ungated up projection with relu squared), then the down projection with the
+//     weighted top-k combine fused, no atomics.
 // Larger batches group rows by expert and run library GEMMs (the caller's choice).
 #include "common.h"
 
@@ -13,13 +15,16 @@ namespace la {
 //         weights are s / (sum of the chosen s + 1e-20).
 // mode 1: s = z + corr (a bias that counts in the weights too); the `topk` largest s are chosen,
 //         their weights are the softmax over the chosen s.
+// groups > 1: experts form that many groups of neighbours; a group's score is its largest s (+ corr), and only
+// experts of the `keep` best groups can be chosen (ties: lowest group).  All weights times scale.
 template <typename AT>
 __global__ __launch_bounds__(256) void router_topk_kernel(const AT* __restrict__ x, long ldx,
                                                           const float* __restrict__ router,
                                                           const float* __restrict__ corr, int E, int D, int T,
-                                                          int topk, int renorm, int mode, int* __restrict__ ids,
-                                                          float* __restrict__ wts) {
+                                                          int topk, int renorm, int mode, int groups, int keep,
+                                                          float scale, int* __restrict__ ids, float* __restrict__ wts) {
   __shared__ float sc[4][256];
+  __shared__ uint8_t open[4][256];     // the expert's group can be chosen from
   const int w = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int t = blockIdx.x * 4 + w;
   const bool live = t < T;
@@ -55,6 +60,38 @@ __global__ __launch_bounds__(256) void router_topk_kernel(const AT* __restrict__
     }
   }
   __syncthreads();
+  if (groups > 1) {
+    const int n = E / groups;
+    float gm[4];                       // scores of groups lane, lane + 64, ..
+    for (int i = 0; i < 4; ++i) {
+      const int g = lane + 64 * i;
+      gm[i] = -INFINITY;
+      if (g < groups)
+        for (int e = g * n; e < (g + 1) * n; ++e) {
+          gm[i] = fmaxf(gm[i], sc[w][e] + ((corr && !mode) ? corr[e] : 0.f));
+          open[w][e] = 0;
+        }
+    }
+    uint32_t used = 0;
+    for (int k = 0; k < keep; ++k) {
+      float best = -INFINITY;
+      int bi = 0x7fffffff;
+      for (int i = 0; i < 4; ++i) {
+        const int g = lane + 64 * i;
+        if (g < groups && !((used >> i) & 1u) && (gm[i] > best || bi == 0x7fffffff)) { best = gm[i]; bi = g; }
+      }
+      for (int o = 32; o > 0; o >>= 1) {
+        const float ob = __shfl_xor(best, o, 64);
+        const int oi = __shfl_xor(bi, o, 64);
+        if (oi != 0x7fffffff && (bi == 0x7fffffff || ob > best || (ob == best && oi < bi))) { best = ob; bi = oi; }
+      }
+      if ((bi & 63) == lane) {
+        used |= 1u << (bi >> 6);
+        for (int e = bi * n; e < (bi + 1) * n; ++e) open[w][e] = 1;
+      }
+    }
+    __syncthreads();
+  }
   float sum = 0.f, my_s = 0.f, top0 = 0.f;
   int my_id = 0;
   uint32_t taken = 0;   // bit i: this lane's expert e = lane + 64 * i is already chosen
@@ -63,7 +100,7 @@ __global__ __launch_bounds__(256) void router_topk_kernel(const AT* __restrict__
     int bi = 0x7fffffff;
     for (int i = 0; i < 4; ++i) {
       const int e = lane + 64 * i;
-      if (e < E && !((taken >> i) & 1u)) {
+      if (e < E && !((taken >> i) & 1u) && (groups <= 1 || open[w][e])) {
         const float c = sc[w][e] + ((corr && !mode) ? corr[e] : 0.f);
         if (c > best || (c == best && e < bi)) { best = c; bi = e; }
       }
@@ -84,13 +121,31 @@ __global__ __launch_bounds__(256) void router_topk_kernel(const AT* __restrict__
   }
   if (live && lane < topk) {
     ids[(long)t * topk + lane] = my_id;
-    wts[(long)t * topk + lane] = (renorm || mode) ? my_s / (sum + 1e-20f) : my_s;
+    wts[(long)t * topk + lane] = ((renorm || mode) ? my_s / (sum + 1e-20f) : my_s) * scale;
   }
 }
 
 // h[p][f] = silu(Wg[e_p][f] . x[t_p]) * (Wu[e_p][f] . x[t_p]),  p = t * topk + slot; a wave per (p, f).
 // clamp: g = min(Wg x, limit), u = clamp(Wu x, -limit, limit), h = g sigmoid(slope g) (u + 1) instead.
-template <typename AT, typename WT>
+// Wg null: no gate, h = max(Wu x, 0)^2.  VEC values of a row per load.
+template <typename T, int VEC>
+LA_DEV float dot_slice(const T* __restrict__ w, const float (&x)[VEC]) {
+  typedef T vec __attribute__((ext_vector_type(VEC)));
+  const vec v = *(const vec*)w;
+  float a = 0.f;
+#pragma unroll
+  for (int j = 0; j < VEC; ++j) a = fmaf((float)v[j], x[j], a);
+  return a;
+}
+template <typename T, int VEC>
+LA_DEV void row_slice(const T* __restrict__ p, float (&x)[VEC]) {
+  typedef T vec __attribute__((ext_vector_type(VEC)));
+  const vec v = *(const vec*)p;
+#pragma unroll
+  for (int j = 0; j < VEC; ++j) x[j] = (float)v[j];
+}
+
+template <typename AT, typename WT, int VEC>
 __global__ __launch_bounds__(256) void moe_pair_glu_kernel(const AT* __restrict__ x, const WT* __restrict__ wg,
                                                            const WT* __restrict__ wu, const int* __restrict__ ids,
                                                            int topk, int D, int F, int E, AT* __restrict__ h, int clamp,
@@ -101,19 +156,24 @@ __global__ __launch_bounds__(256) void moe_pair_glu_kernel(const AT* __restrict_
   const int e = ids[p];
   if (e < 0 || e >= E) { if (lane == 0) h[(long)p * F + f] = (AT)0.f; return; }
   const AT* xr = x + (long)(p / topk) * D;
-  const WT* g = wg + ((long)e * F + f) * D;
+  const WT* g = wg ? wg + ((long)e * F + f) * D : nullptr;
   const WT* u = wu + ((long)e * F + f) * D;
   float a = 0.f, b = 0.f;
-  for (int d = lane; d < D; d += 64) {
-    const float xv = (float)xr[d];
-    a = fmaf((float)g[d], xv, a);
-    b = fmaf((float)u[d], xv, b);
+#pragma unroll 4
+  for (int d = lane * VEC; d < D; d += 64 * VEC) {
+    float xv[VEC];
+    row_slice<AT, VEC>(xr + d, xv);
+    if (g) a += dot_slice<WT, VEC>(g + d, xv);
+    b += dot_slice<WT, VEC>(u + d, xv);
   }
   a = wave_sum(a);
   b = wave_sum(b);
   if (lane == 0) {
     float v;
-    if (clamp) {
+    if (!g) {
+      const float r = fmaxf(b, 0.f);
+      v = r * r;
+    } else if (clamp) {
       const float g2 = fminf(a, limit), u2 = fminf(fmaxf(b, -limit), limit);
       v = g2 / (1.f + expf(-slope * g2)) * (u2 + 1.f);
     } else {
@@ -124,7 +184,7 @@ __global__ __launch_bounds__(256) void moe_pair_glu_kernel(const AT* __restrict_
 }
 
 // y[t][d] = sum_slot w[p] * (Wd[e_p][d] . h[p]); a wave per (t, d), slots in order (deterministic)
-template <typename AT, typename WT>
+template <typename AT, typename WT, int VEC>
 __global__ __launch_bounds__(256) void moe_pair_down_kernel(const AT* __restrict__ h, const WT* __restrict__ wd,
                                                             const int* __restrict__ ids, const float* __restrict__ wts,
                                                             int topk, int D, int F, int E, float* __restrict__ y) {
@@ -138,7 +198,12 @@ __global__ __launch_bounds__(256) void moe_pair_down_kernel(const AT* __restrict
     const WT* wr = wd + ((long)e * D + d) * F;
     const AT* hr = h + (long)p * F;
     float a = 0.f;
-    for (int f = lane; f < F; f += 64) a = fmaf((float)wr[f], (float)hr[f], a);
+#pragma unroll 4
+    for (int f = lane * VEC; f < F; f += 64 * VEC) {
+      float hv[VEC];
+      row_slice<AT, VEC>(hr + f, hv);
+      a += dot_slice<WT, VEC>(wr + f, hv);
+    }
     acc = fmaf(wts[p], wave_sum(a), acc);
   }
   if (lane == 0) y[(long)t * D + d] = acc;
@@ -147,25 +212,29 @@ __global__ __launch_bounds__(256) void moe_pair_down_kernel(const AT* __restrict
 }  // namespace la
 
 extern "C" int la_router_topk(int f32, int mode, const void* x, long ldx, const void* router, const void* corr, int E,
-                              int D, int T, int topk, int renorm, void* ids, void* wts, void* stream) {
+                              int D, int T, int topk, int renorm, int groups, int keep, float scale, void* ids,
+                              void* wts, void* stream) {
   using namespace la;
   if (E < 1 || E > 256 || topk < 1 || topk > E || topk > 64 || T <= 0 || mode < 0 || mode > 1) return -1;
+  if (groups < 1 || E % groups || (groups > 1 && (keep < 1 || keep > groups || topk > keep * (E / groups)))) return -2;
   dim3 grid((T + 3) / 4);
   if (f32)
     hipLaunchKernelGGL((router_topk_kernel<float>), grid, dim3(256), 0, (hipStream_t)stream, (const float*)x, ldx,
-                       (const float*)router, (const float*)corr, E, D, T, topk, renorm, mode, (int*)ids, (float*)wts);
+                       (const float*)router, (const float*)corr, E, D, T, topk, renorm, mode, groups, keep, scale, (int*)ids,
+                       (float*)wts);
   else
     hipLaunchKernelGGL((router_topk_kernel<bf16>), grid, dim3(256), 0, (hipStream_t)stream, (const bf16*)x, ldx,
-                       (const float*)router, (const float*)corr, E, D, T, topk, renorm, mode, (int*)ids, (float*)wts);
+                       (const float*)router, (const float*)corr, E, D, T, topk, renorm, mode, groups, keep, scale, (int*)ids,
+                       (float*)wts);
   return (int)hipGetLastError();
 }
 
 extern "C" int la_router_sigmoid(int f32, const void* x, long ldx, const void* router, const void* corr, int E, int D,
                                  int T, int topk, int renorm, void* ids, void* wts, void* stream) {
-  return la_router_topk(f32, 0, x, ldx, router, corr, E, D, T, topk, renorm, ids, wts, stream);
+  return la_router_topk(f32, 0, x, ldx, router, corr, E, D, T, topk, renorm, 1, 1, 1.f, ids, wts, stream);
 }
 
-// f32: activations and weights fp32 (else both bf16).  x [T, D], wg / wu [E, F, D], wd [E, D, F],
+// f32: activations and weights fp32 (else both bf16).  wg null: ungated experts, relu squared.  x [T, D], wg / wu [E, F, D], wd [E, D, F],
 // ids [T * topk], wts [T * topk] -> h [T * topk, F] (scratch, activation type), y [T, D] fp32.
 extern "C" int la_moe_pairs(int f32, const void* x, const void* wg, const void* wu, const void* wd, const void* ids,
                             const void* wts, int T, int topk, int D, int F, int E, void* h, void* y, int clamp, float limit,
@@ -176,16 +245,21 @@ extern "C" int la_moe_pairs(int f32, const void* x, const void* wg, const void* 
   if (P > 65535 || T > 65535) return -2;
   dim3 g1((F + 3) / 4, P), g2((D + 3) / 4, T);
   hipStream_t s = (hipStream_t)stream;
-  if (f32) {
-    hipLaunchKernelGGL((moe_pair_glu_kernel<float, float>), g1, dim3(256), 0, s, (const float*)x, (const float*)wg,
-                       (const float*)wu, (const int*)ids, topk, D, F, E, (float*)h, clamp, limit, slope);
-    hipLaunchKernelGGL((moe_pair_down_kernel<float, float>), g2, dim3(256), 0, s, (const float*)h, (const float*)wd,
-                       (const int*)ids, (const float*)wts, topk, D, F, E, (float*)y);
-  } else {
-    hipLaunchKernelGGL((moe_pair_glu_kernel<bf16, bf16>), g1, dim3(256), 0, s, (const bf16*)x, (const bf16*)wg,
-                       (const bf16*)wu, (const int*)ids, topk, D, F, E, (bf16*)h, clamp, limit, slope);
-    hipLaunchKernelGGL((moe_pair_down_kernel<bf16, bf16>), g2, dim3(256), 0, s, (const bf16*)h, (const bf16*)wd,
-                       (const int*)ids, (const float*)wts, topk, D, F, E, (float*)y);
+  if (!x || !wu || !wd || !ids || !wts || !h || !y || (clamp && !wg)) return -3;
+#define LA_MP(AT, VEC)                                                                                                    \
+  {                                                                                                                       \
+    hipLaunchKernelGGL((moe_pair_glu_kernel<AT, AT, VEC>), g1, dim3(256), 0, s, (const AT*)x, (const AT*)wg,              \
+                       (const AT*)wu, (const int*)ids, topk, D, F, E, (AT*)h, clamp, limit, slope);                       \
+    hipLaunchKernelGGL((moe_pair_down_kernel<AT, AT, VEC>), g2, dim3(256), 0, s, (const AT*)h, (const AT*)wd,             \
+                       (const int*)ids, (const float*)wts, topk, D, F, E, (float*)y);                                     \
   }
+  // whole vectors of 16 bytes where both widths allow
+  const bool al = (((uintptr_t)x | (uintptr_t)wg | (uintptr_t)wu | (uintptr_t)wd | (uintptr_t)h) & 15) == 0;
+  if (f32) {
+    if (al && !((D | F) & 3)) LA_MP(float, 4) else LA_MP(float, 1)
+  } else {
+    if (al && !((D | F) & 7)) LA_MP(bf16, 8) else LA_MP(bf16, 1)
+  }
+#undef LA_MP
   return (int)hipGetLastError();
 }

@@ -21,59 +21,9 @@
 //
 // Sources are GEMM results as the framework hands them on: fp32 split-K slabs [S][T][N] (summed
 // here), or one bf16 / fp32 matrix.  All arithmetic is fp32; outputs bf16 or fp32.
-#include "common.h"
+#include "row_src.h"
 
 namespace la {
-
-struct RowSrc {
-  const void* p;
-  int f32;
-  long slab;
-  int S;
-};
-
-LA_DEV float src_at(const RowSrc& s, long idx) {
-  if (s.f32) {
-    const float* f = (const float*)s.p;
-    float a = f[idx];
-    for (int k = 1; k < s.S; ++k) a += f[idx + k * s.slab];
-    return a;
-  }
-  return (float)((const bf16*)s.p)[idx];
-}
-
-// four neighbouring columns; slabs are requested four at a time (clamped index, masked: no branch between loads)
-LA_DEV f32x4 src4_at(const RowSrc& s, long idx) {
-  if (!s.f32) {
-    const bf16x4 b = *(const bf16x4*)((const bf16*)s.p + idx);
-    return f32x4{(float)b[0], (float)b[1], (float)b[2], (float)b[3]};
-  }
-  const float* f = (const float*)s.p + idx;
-  if (s.S <= 1) return *(const f32x4*)f;
-  f32x4 a = {0.f, 0.f, 0.f, 0.f};
-  for (int k0 = 0; k0 < s.S; k0 += 4) {
-    f32x4 t[4];
-#pragma unroll
-    for (int k = 0; k < 4; ++k) t[k] = *(const f32x4*)(f + (long)min(k0 + k, s.S - 1) * s.slab);
-#pragma unroll
-    for (int k = 0; k < 4; ++k) {
-      const float m = k0 + k < s.S ? 1.f : 0.f;
-#pragma unroll
-      for (int j = 0; j < 4; ++j) a[j] = fmaf(m, t[k][j], a[j]);
-    }
-  }
-  return a;
-}
-
-LA_DEV void put4(void* out, int out_f32, long idx, const f32x4& v) {
-  if (out_f32) *(f32x4*)((float*)out + idx) = v;
-  else *(bf16x4*)((bf16*)out + idx) = bf16x4{(bf16)v[0], (bf16)v[1], (bf16)v[2], (bf16)v[3]};
-}
-
-LA_DEV void put(void* out, int out_f32, long idx, float v) {
-  if (out_f32) ((float*)out)[idx] = v;
-  else ((bf16*)out)[idx] = (bf16)v;
-}
 
 enum { NC_NONE = 0, NC_DYT = 1, NC_RMS = 2, NC_CAST = 3, NC_LN = 4 };
 constexpr int NC_NT = 256;

@@ -16,10 +16,13 @@
 //   qk_row_norm_rope_pages: q and k normed over the WHOLE projection (all heads together) with a
 //                weight per channel, rotated like rope_pages' half layout, q times a number per head; the
 //                values are the raw keys (before norm and rotation).
+//   head_rope_pages: q | k | v as fp32 split-K slabs or one matrix of any row stride, a bias per column, either
+//                pair layout, and optionally every rotated query and key head divided by its root mean square
+//                (no weight); a group of lanes per head, V values per access.
 //   sinusoid_add: additive positions on the fp32 stream, column 2i += sin(pos f_i), 2i + 1 += cos.
 //
 // A workgroup per token; the token's cos / sin are computed once into LDS.
-#include "common.h"
+#include "row_src.h"
 
 namespace la {
 
@@ -316,6 +319,107 @@ __global__ __launch_bounds__(RP_NT) void qk_row_norm_rope_pages_kernel(
   }
 }
 
+// Row [q (H x Dq) | k (G x Dk) | v (G x Dv)] plus bias.  A unit is V pairs of the rotated span (2 V dims) or V dims
+// of the rest; the LG lanes of a head take its units in turn.  unit: the head divided by sqrt(mean x^2 + eps);
+// a rotation keeps the sum of squares, so it is taken from the values as they are read.
+template <typename AT, int V>
+__global__ __launch_bounds__(RP_NT) void head_rope_pages_kernel(
+    RowSrc src, long ld, const float* __restrict__ bias, int H, int Dq, int G, int Dk, int Dv,
+    const int* __restrict__ pos, const int* __restrict__ slots, const float* __restrict__ freqs, int rot, int interleaved,
+    int unit, float eps, int LG, AT* __restrict__ q_out, AT* __restrict__ kc, AT* __restrict__ vc, int BS) {
+  typedef typename RowVec<V>::type fvec;
+  typedef AT avec __attribute__((ext_vector_type(V)));
+  extern __shared__ float cs[];          // [rot / 2][2]
+  const int t = blockIdx.x, tid = threadIdx.x, half = rot >> 1;
+  const int Cq = H * Dq, Ck = G * Dk, Cv = G * Dv;
+  const long row = (long)t * ld;
+  const int p = pos[t];
+  for (int i = tid; i < half; i += RP_NT) sincosf((float)p * freqs[i], &cs[2 * i + 1], &cs[2 * i]);
+  __syncthreads();
+  const int slot = G ? slots[t] : -1;
+  const int blk = slot >= 0 ? slot / BS : 0, off = slot >= 0 ? slot - blk * BS : 0;
+  auto value = [&](int c) -> fvec {
+    fvec x = srcv_at<V>(src, row + c);
+    if (bias) {
+      const fvec b = *(const fvec*)(bias + c);
+#pragma unroll
+      for (int j = 0; j < V; ++j) x[j] += b[j];
+    }
+    return x;
+  };
+  auto store = [](AT* p, const fvec& x) {
+    avec y;
+#pragma unroll
+    for (int j = 0; j < V; ++j) y[j] = (AT)x[j];
+    *(avec*)p = y;
+  };
+  const int lane = tid % LG, nh = slot >= 0 ? H + G : H, pairs = half / V;
+  for (int u = tid / LG; u < nh; u += RP_NT / LG) {
+    const bool isq = u < H;
+    const int D = isq ? Dq : Dk, c0 = isq ? u * Dq : Cq + (u - H) * Dk, per = pairs + (D - rot) / V;
+    AT* dst = isq ? q_out + (long)t * Cq + (long)u * Dq : kc + (((long)blk * G + (u - H)) * BS + off) * Dk;
+    // columns of unit k: a, and for a rotated unit also b
+    auto first = [&](int k) { return k < pairs ? (interleaved ? 2 * k * V : k * V) : rot + (k - pairs) * V; };
+    auto second = [&](int k) { return interleaved ? (2 * k + 1) * V : k * V + half; };
+    fvec a = fvec(0.f), b = fvec(0.f);
+    auto load = [&](int k) {
+      a = value(c0 + first(k));
+      b = k < pairs ? value(c0 + second(k)) : fvec(0.f);
+    };
+    float inv = 1.f;
+    if (lane < per) load(lane);
+    if (unit) {
+      float ss = 0.f;
+      for (int k = lane; k < per; k += LG) {
+        if (k != lane) load(k);
+#pragma unroll
+        for (int j = 0; j < V; ++j) ss = fmaf(a[j], a[j], fmaf(b[j], b[j], ss));
+      }
+      for (int o = LG >> 1; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+      inv = 1.f / sqrtf(ss / (float)D + eps);
+      if (per > LG && lane < per) load(lane);
+    }
+    for (int k = lane; k < per; k += LG) {
+      if (k != lane) load(k);
+      if (k < pairs) {
+        fvec ya, yb;
+        if (V == 1 || !interleaved) {
+#pragma unroll
+          for (int j = 0; j < V; ++j) {
+            const float c = cs[2 * (k * V + j)], s = cs[2 * (k * V + j) + 1];
+            ya[j] = (a[j] * c - b[j] * s) * inv;
+            yb[j] = (b[j] * c + a[j] * s) * inv;
+          }
+        } else {
+          const float* f = cs + 2 * k * V;   // V pairs: the first half of them in a, the others in b
+#pragma unroll
+          for (int j = 0; j + 1 < V; j += 2) {
+            ya[j] = (a[j] * f[j] - a[j + 1] * f[j + 1]) * inv;
+            ya[j + 1] = (a[j + 1] * f[j] + a[j] * f[j + 1]) * inv;
+            yb[j] = (b[j] * f[V + j] - b[j + 1] * f[V + j + 1]) * inv;
+            yb[j + 1] = (b[j + 1] * f[V + j] + b[j] * f[V + j + 1]) * inv;
+          }
+        }
+        store(dst + first(k), ya);
+        store(dst + second(k), yb);
+      } else {
+        fvec y;
+#pragma unroll
+        for (int j = 0; j < V; ++j) y[j] = a[j] * inv;
+        store(dst + first(k), y);
+      }
+    }
+  }
+  if (slot < 0) return;
+  for (int e = tid * V; e < Cv; e += RP_NT * V) {
+    const int g = e / Dv, d = e - g * Dv;
+    const fvec x = value(Cq + Ck + e);
+    AT* dst = vc + ((((long)blk * G + g) * (BS >> 3) + (off >> 3)) * Dv + d) * 8 + (off & 7);
+#pragma unroll
+    for (int j = 0; j < V; ++j) dst[j * 8] = (AT)x[j];
+  }
+}
+
 // every head of a row turned over its whole width, dims m and m + Dv / 2 by sign * pos * freqs[m], times scale
 template <typename AT>
 __global__ __launch_bounds__(RP_NT) void rotate_heads_kernel(const AT* __restrict__ x, int H, int Dv,
@@ -340,6 +444,37 @@ __global__ __launch_bounds__(RP_NT) void rotate_heads_kernel(const AT* __restric
 }
 
 }  // namespace la
+
+// sp: fp32 slabs (src_f32, S of them `slab` elements apart) or one bf16 matrix, rows ld apart; bias fp32 or null
+extern "C" int la_head_rope_pages(int f32, const void* sp, int src_f32, long slab, int S, long ld, const void* bias, int T,
+                                  int H, int Dq, int G, int Dk, int Dv, const void* pos, const void* slots,
+                                  const void* freqs, int rot, int interleaved, int unit, float eps, void* q_out, void* kc,
+                                  void* vc, int BS, void* stream) {
+  using namespace la;
+  if (T <= 0 || H <= 0 || Dq <= 0 || G < 0 || (rot & 1) || rot < 0 || rot > Dq) return -1;
+  if (G && (Dk <= 0 || Dv <= 0 || rot > Dk || !kc || !vc || !slots || BS <= 0 || (BS & 7))) return -2;
+  if (!sp || !pos || (rot > 0 && !freqs) || !q_out || (src_f32 && S < 1) || ld < (long)H * Dq + (long)G * (Dk + Dv)) return -3;
+  RowSrc s{sp, src_f32, slab, S};
+  const size_t shm = (size_t)(rot + 2) * sizeof(float);
+  const bool vec = !((Dq | Dk | Dv | ld | slab) & 3) && !(rot & 7) &&
+                   (((uintptr_t)sp | (uintptr_t)bias | (uintptr_t)q_out | (uintptr_t)kc) & 15) == 0;
+  const int v = vec ? 4 : 1, D = Dq > Dk ? Dq : Dk, per = rot / 2 / v + (D - rot) / v;
+  int LG = 4;
+  while (LG < 64 && LG < per) LG <<= 1;
+#define LA_HRP(AT, V)                                                                                                    \
+  hipLaunchKernelGGL((head_rope_pages_kernel<AT, V>), dim3(T), dim3(RP_NT), shm, (hipStream_t)stream, s, ld,             \
+                     (const float*)bias, H, Dq, G, Dk, Dv, (const int*)pos, (const int*)slots, (const float*)freqs, rot, \
+                     interleaved, unit, eps, LG, (AT*)q_out, (AT*)kc, (AT*)vc, BS)
+  if (f32) {
+    if (vec) LA_HRP(float, 4);
+    else LA_HRP(float, 1);
+  } else {
+    if (vec) LA_HRP(bf16, 4);
+    else LA_HRP(bf16, 1);
+  }
+#undef LA_HRP
+  return (int)hipGetLastError();
+}
 
 extern "C" int la_qk_norm_rope_pages(int f32, const void* src, long ld, int T, int H, int D, int G, int Dv, const void* pos,
                                      const void* slots, const void* qw, const void* kw, float eps, const void* freqs,
