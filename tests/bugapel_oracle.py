@@ -162,19 +162,36 @@ def route(z, top, groups, keep, scale):
     return ids, [float(s[e]) / tot * scale for e in ids]
 
 
-def experts(W, p, f, h):
+def margin(z, top, groups, keep):
+    """How far one token's choice is from another one, in logits: between the last kept and the first dropped
+    group, and the last chosen and the first passed-over expert."""
+    n = z.shape[0] // groups
+    gs = sorted(range(groups), key=lambda g: -float(z[g * n:(g + 1) * n].max()))
+    es = sorted((float(z[e]) for g in gs[:keep] for e in range(g * n, (g + 1) * n)), reverse=True)
+    gaps = [es[top - 1] - es[top]] if top < len(es) else []
+    if keep < groups:
+        a, b = (float(z[g * n:(g + 1) * n].max()) for g in gs[keep - 1:keep + 1])
+        gaps.append(a - b)
+    return min(gaps, default=math.inf)
+
+
+def experts(W, p, f, h, margins=None):
+    """margins: a list of one number per token that is lowered to the token's margin here."""
     r = f["router"]
     gr = r.get("groups") or {"count": 1, "keep": 1}
     y = torch.zeros_like(h)
     for t in range(h.shape[0]):
+        if margins is not None:
+            margins[t] = min(margins[t], margin(W[p + "router"] @ h[t], r["top"], gr["count"], gr["keep"]))
         for e, w in zip(*route(W[p + "router"] @ h[t], r["top"], gr["count"], gr["keep"], r["scale"])):
             y[t] += w * (W[p + f"e{e}.down"] @ torch.relu(W[p + f"e{e}.up"] @ h[t]) ** 2)
     return y
 
 
 # ------------------------------------------------------------------------------------------ model
-def forward(cfg, W, tokens, streams=None):
-    """logits [T, vocab] (float64); streams: a list that receives the sum of the streams after every layer."""
+def forward(cfg, W, tokens, streams=None, margins=None):
+    """logits [T, vocab] (float64); streams: a list that receives the sum of the streams after every layer;
+    margins: a list of one number per token that is lowered to the token's smallest router margin."""
     eps, n = cfg["norm"]["eps"], cfg["streams"]
     x = W["embed"][torch.as_tensor(tokens).long()] * cfg["embedding"]["scale"]
     X = x.unsqueeze(1).repeat(1, n, 1)
@@ -182,7 +199,7 @@ def forward(cfg, W, tokens, streams=None):
         p = f"l{i}."
         subs = [lambda h: MIXERS[L["type"]](W, p + "mix.", L["mixer"], h, eps)]
         if L.get("mlp"):
-            subs.append(lambda h: experts(W, p + "mlp.", L["mlp"], h))
+            subs.append(lambda h: experts(W, p + "mlp.", L["mlp"], h, margins))
         for q, f in enumerate(subs, 1):
             y = f(layer_norm(streams_in(X, W[p + f"hc{q}.in"]), W[p + f"norm{q}"], W[p + f"norm{q}.b"], eps))
             X = streams_out(X, y, W[p + f"hc{q}.mix"], W[p + f"hc{q}.out"])
