@@ -88,19 +88,23 @@ def visible(i, window, keep):
     return [j for j in range(i + 1) if not window or i - j < window or j < keep]
 
 
+def attend(q, k, v, scale, one=False):
+    """One query q [H, d] over keys k [n, G, d] and values v [n, G, dv]; one: a 1 is added to the denominator."""
+    H = q.shape[0]
+    rep = H // k.shape[1]
+    o = torch.zeros(H, v.shape[2], dtype=F64)
+    for hd in range(H):
+        s = (k[:, hd // rep] @ q[hd]) * scale
+        m = max(float(s.max()), 0.0)
+        e = torch.exp(s - m)
+        o[hd] = (e / (e.sum() + (math.exp(-m) if one else 0.0))) @ v[:, hd // rep]
+    return o
+
+
 def softmax_attention(q, k, v, scale, window=0, keep=0, one=False):
     """q [T, H, d], k [T, G, d], v [T, G, dv]; one: a 1 is added to the denominator."""
-    T, H, _ = q.shape
-    rep = H // k.shape[1]
-    o = torch.zeros(T, H, v.shape[2], dtype=F64)
-    for i in range(T):
-        js = visible(i, window, keep)
-        for hd in range(H):
-            s = (k[js, hd // rep] @ q[i, hd]) * scale
-            m = max(float(s.max()), 0.0)
-            e = torch.exp(s - m)
-            o[i, hd] = (e / (e.sum() + (math.exp(-m) if one else 0.0))) @ v[js, hd // rep]
-    return o
+    seen = [visible(i, window, keep) for i in range(q.shape[0])]
+    return torch.stack([attend(q[i], k[js], v[js], scale, one) for i, js in enumerate(seen)])
 
 
 def attention(W, p, m, h, eps):

@@ -75,11 +75,11 @@ CONFIGS = {
                    bare(attention_2(heads=3, kv=1, dim=9, vdim=11, rot=6, window=18, keep=17))], 51, 35, 5, eps=1e-6),
     # widths the GPU's specialised paths take: split-KV decode and prefill kernels, matrix-core tiles, the vectorised
     # page append, the grouped expert GEMMs, several blocks of key channels
-    "wide": config([moe(attention(heads=8, kv=2, dim=64, vdim=64, rot=32, scale=0.3, scaling=SCALING), ff=256),
-                    moe(attention_2(heads=4, kv=1, dim=128, vdim=128, rot=128, scale=0.2, window=37, keep=4), ff=256, groups=1, keep=1),
+    "wide": config([moe(attention(heads=8, kv=2, dim=64, vdim=64, rot=32, scale=0.12, scaling=SCALING), ff=256),
+                    moe(attention_2(heads=4, kv=1, dim=128, vdim=128, rot=128, scale=0.1, window=37, keep=4), ff=256, groups=1, keep=1),
                     bare(gla(heads=4, dim=64, vdim=96, rank=16)), moe(gla(heads=2, dim=80, vdim=32, rank=8), ff=64),
-                    bare(attention_2(heads=4, kv=2, dim=32, vdim=64, rot=32, window=24, keep=20)),
-                    moe(attention(heads=4, kv=4, dim=96, vdim=32, rot=96), ff=256)], 97, 256, 2),
+                    bare(attention_2(heads=4, kv=2, dim=32, vdim=64, rot=32, scale=0.2, window=24, keep=20)),
+                    moe(attention(heads=4, kv=4, dim=96, vdim=32, rot=96, scale=0.1), ff=256)], 97, 256, 2),
 }
 
 
@@ -180,8 +180,8 @@ class Want:
 
 def close(got, want, dtype):
     """Every position, its mean taken off, in units of the wanted logits' spread.  fp32: to rounding.  bf16: to 16-bit
-    rounding; a position whose routing is a close call counts in the median only, and of the others one in ten
-    may stand out (it reads what a close call changed)."""
+    rounding; a position whose routing is a close call, or that of one of the 6 before it (whose change it reads),
+    counts in the median only, and of the others one in ten may stand out."""
     got, logits = got.detach().double().cpu(), want.logits.double()
     d = got - logits
     d = d - d.mean(-1, keepdim=True)
@@ -189,7 +189,8 @@ def close(got, want, dtype):
     if dtype == "float32":
         assert float(err.max()) < 4e-4 and float(err.median()) < 1e-5, (int(err.argmax()), float(err.max()), float(err.median()))
         return
-    sure = err[want.margins > MARGIN]
+    m = want.margins
+    sure = err[torch.stack([m[max(0, t - 6):t + 1].min() for t in range(m.shape[0])]) > MARGIN]
     out = int((sure > 0.12).sum())
     assert out <= max(1, sure.numel() // 10) and (err.numel() < 10 or float(err.median()) < 0.04), (out, sure.numel(), float(err.max()), float(err.median()))
 
