@@ -1647,3 +1647,79 @@ def write_dobelix(out_dir: str, width: int = 256, kinds=("lightning", "attention
         json.dump(cfg, f_)
     save_file(W, os.path.join(out_dir, "model.safetensors"))
     return out_dir
+
+
+def write_bugapel(out_dir: str, width: int = 256, kinds=("gla", "attention", "attention_2"), heads: int = 4, kv_heads: int = 2,
+                  dim: int = 64, g_heads: int = 4, g_dim: int = 64, g_vdim: int = 64, rank: int = 16, window: int = 256,
+                  keep: int = 4, streams: int = 2, experts: int = 8, top: int = 2, groups: int = 2, keep_groups: int = 1,
+                  expert_ff: int = 256, vocab: int = 32000, seed: int = 0) -> str:
+    """Random-init Bugapel checkpoint directory (config.json + model.safetensors, bf16): one layer per entry of
+    `kinds`: gated linear attention with g_heads heads of g_dim x g_vdim, or one of the two attention mixers with
+    `heads` query heads over kv_heads key heads of width dim; routed experts of width expert_ff (experts 0: no
+    feed-forward).  Benchmarks and smoke runs; the weights mean nothing."""
+    import json
+
+    import torch
+    from safetensors.torch import save_file
+    os.makedirs(out_dir, exist_ok=True)
+    g = torch.Generator().manual_seed(seed)
+    D = width
+
+    def rnd(*shape, s):
+        return (torch.randn(*shape, generator=g, dtype=torch.float32) * s).to(torch.bfloat16)
+
+    def lin(a, b):
+        return rnd(a, b, s=b ** -0.5)
+
+    def norm(name, k):
+        W[name] = (1.0 + rnd(k, s=0.05).float()).to(torch.bfloat16)
+
+    W = {"embed": rnd(vocab, D, s=D ** -0.5), "final.norm.b": rnd(D, s=0.05)}
+    norm("final.norm", D)
+    layers = []
+    for i, kind in enumerate(kinds):
+        for q in (1, 2) if experts else (1,):
+            norm(f"l{i}.norm{q}", D)
+            W[f"l{i}.norm{q}.b"] = rnd(D, s=0.05)
+            h = f"l{i}.hc{q}."
+            W[h + "in"], W[h + "out"] = (1.0 / streams + rnd(streams, s=0.05).float()).to(torch.bfloat16), (1.0 + rnd(streams, s=0.05).float()).to(torch.bfloat16)
+            W[h + "mix"] = (torch.eye(streams) + rnd(streams, streams, s=0.05).float()).to(torch.bfloat16)
+        p = f"l{i}.mix."
+        if kind == "gla":
+            m = {"heads": g_heads, "dim": g_dim, "vdim": g_vdim, "tau": 16.0}
+            for n, k in (("q", g_dim), ("k", g_dim), ("v", g_vdim), ("g", g_vdim)):
+                W[p + n] = lin(g_heads * k, D)
+            W[p + "a1"], W[p + "a2"], W[p + "a2.b"] = lin(rank, D), lin(g_heads * g_dim, rank), rnd(g_heads * g_dim, s=1.0)
+            norm(p + "norm", g_vdim)
+            wide = g_heads * g_vdim
+        elif kind in ("attention", "attention_2"):
+            m = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5,
+                 "rot": {"dims": dim, "base": 10000.0}}
+            rows = (("q", heads * dim), ("k", kv_heads * dim), ("v", kv_heads * dim))
+            for n, k in rows:
+                W[p + n] = lin(k, D)
+            if kind == "attention":
+                m["rot"]["scaling"] = {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}
+            else:
+                m["mask"] = {"size": window, "keep_first": keep}
+                for n, k in rows + (("o", D),):
+                    W[f"{p}{n}.b"] = rnd(k, s=0.1)
+            wide = heads * dim
+        else:
+            raise ValueError(f"unknown mixer kind {kind!r}")
+        W[p + "o"] = lin(D, wide)
+        mlp = None
+        if experts:
+            p = f"l{i}.mlp."
+            W[p + "router"] = lin(experts, D)
+            for e in range(experts):
+                W[p + f"e{e}.up"], W[p + f"e{e}.down"] = lin(expert_ff, D), lin(D, expert_ff)
+            mlp = {"kind": "moe", "expert": {"ff": expert_ff},
+                   "router": {"experts": experts, "top": top, "scale": 1.0, "groups": {"count": groups, "keep": keep_groups}}}
+        layers.append({"type": kind, "mixer": m, "mlp": mlp})
+    cfg = {"architecture": "Bugapel", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "streams": streams,
+           "embedding": {"scale": D ** 0.5}, "logit_softcap": 30.0, "layers": layers}
+    with open(os.path.join(out_dir, "config.json"), "w") as f_:
+        json.dump(cfg, f_)
+    save_file(W, os.path.join(out_dir, "model.safetensors"))
+    return out_dir

@@ -7,7 +7,9 @@ kind (windowed attention, latent attention, retention) beside the llama checkpoi
 attention with a dense feed-forward, attention with routed experts, the state-space mixer, beside
 the llama and Mixtral-style checkpoints; Gosuvik: the delta rule, latent attention with routed experts,
 the parallel mixer, beside the same two; Dobelix: one model per mixer kind (lightning attention, chunked
-sigmoid attention) beside the llama checkpoint and Dadizen's retention -- all stored as
+sigmoid attention) beside the llama checkpoint and Dadizen's retention; Bugapel: one model per mixer kind (attention,
+windowed attention with kept tokens, gated linear attention), each with routed experts, beside the
+Mixtral-style checkpoint and Gosuvik's delta rule -- all stored as
 dense bf16 weights so every GEMM takes the same library path, and each is timed through its engine's own
 batch construction (native scheduler, paged KV pool, state slots) and `model.forward`:
   prefill: `n_seq` prompts of `prompt` tokens in one batch, tokens/s;
@@ -136,6 +138,26 @@ def _dobelix_models(size: str, cache: str) -> Dict[str, str]:
     return out
 
 
+def _bugapel_models(size: str, cache: str) -> Dict[str, str]:
+    """Two equal layers of one mixer kind each with two streams and routed experts: both attention mixers with the
+    size's heads (window = the size's chunk), gated linear attention with as many heads of the size's width as
+    the delta rule it is compared with.  The experts have no gates: their width is one and a half times the
+    Mixtral-style model's, so that the expert weights are equally large."""
+    from ..models import synth
+    s = SIZES[size]
+    out = {}
+    for kind in ("attention", "attention_2", "gla"):
+        p = os.path.join(cache, f"bugapel-{size}-{kind}")
+        if not os.path.exists(os.path.join(p, "model.safetensors")):
+            synth.write_bugapel(p, width=s["width"], kinds=(kind, kind), heads=s["heads"], kv_heads=s["kv"], dim=s["dim"],
+                                g_heads=s["heads"], g_dim=s["dim"], g_vdim=s["dim"], window=s["chunk"], experts=s["experts"],
+                                top=s["top"], expert_ff=-(-s["eff"] * 3 // 2 // 256) * 256, vocab=VOCAB)
+        out[f"bugapel-{kind}"] = p
+    out["mixtral-moe"] = _llama(size, cache, moe=True)
+    out["gosuvik-channel_delta-dense"] = _gosuvik_models(size, cache)["gosuvik-channel_delta-dense"]
+    return out
+
+
 def _models(size: str, cache: str) -> Dict[str, str]:
     from ..models import synth
     s = SIZES[size]
@@ -243,7 +265,7 @@ def _measure(path: str, n_seq: int, prompt: int, batch: int, context: int, iters
 def run(design: str, sizes: List[str], cache: str, n_seq: int = 4, prompt: int = 2048, batch: int = 64,
         context: int = 1536, iters: int = 5) -> dict:
     designs = {"suganex": _models, "dadizen": _dadizen_models, "vinozen": _vinozen_models, "gosuvik": _gosuvik_models,
-               "dobelix": _dobelix_models}
+               "dobelix": _dobelix_models, "bugapel": _bugapel_models}
     if design not in designs:
         raise SystemExit(f"--design-compare: unknown design {design!r} ({', '.join(designs)})")
     os.makedirs(cache, exist_ok=True)
