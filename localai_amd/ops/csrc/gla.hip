@@ -108,10 +108,34 @@ __global__ __launch_bounds__(GL_NT) void gla_step_kernel(const AT* __restrict__ 
 // Chunk c of the portion of sequence seq that starts at row a has the number a / 16 + seq + c (unique, below T / 16 + nseq).
 LA_DEV long chunk_no(int a, int seq, int c) { return a / GL_C + seq + c; }
 
+// Sum over W lanes (16 or 32 neighbours) of 16 values at once: at every level a lane hands half of its values to its
+// partner and keeps the other half, so lane l ends with the total of value l & 15.
+template <int W>
+LA_DEV float fold16(float (&v)[16], int lane) {
+  if constexpr (W == 32) {
+#pragma unroll
+    for (int j = 0; j < 16; ++j) v[j] += __shfl_xor(v[j], 16, 64);
+  }
+#pragma unroll
+  for (int m = 8; m > 0; m >>= 1) {
+    const bool up = lane & m;
+#pragma unroll
+    for (int j = 0; j < 8; ++j)
+      if (j < m) {
+        const float keep = up ? v[j + m] : v[j], give = up ? v[j] : v[j + m];
+        v[j] = keep + __shfl_xor(give, m, 64);
+      }
+  }
+  return v[0];
+}
+
 // qd [chunk][H][16][DkP]: q e^b (times qscale);  kd [chunk][H][DkP][16]: k e^(b_last - b);  dl [chunk][H][DkP]: e^(b_last);
 // am [chunk][H][16][16]: A.  DkP = Dk rounded up to 16, filled up with zeros (dl: ones).  Rows past the portion's
-// end count as q = k = 0 with decay 1.  A workgroup per (chunk, head); LDS: q, k, b as [16][DkP + 1].
-template <typename AT>
+// end count as q = k = 0 with decay 1.  A workgroup per (chunk, head); LDS: q, k, b as [16][DkP + 1], then the sums of
+// a over the 16 / TPT token ranges of every channel (a thread takes TPT tokens of one channel).
+// A in 4 x 4 tiles of (t, s): the four on the diagonal pair by pair (16 lanes each, wave 0), the six below it (32
+// lanes each, waves 1 - 3) through the sum b at the tile's first row, c: e^(b_t - b_s) = e^(b_t - c) e^(c - b_s), neither above 1.
+template <typename AT, int TPT>
 __global__ __launch_bounds__(GL_NT) void gla_chunk_kernel(const AT* __restrict__ src, long ld, const AT* __restrict__ z,
                                                           const float* __restrict__ zb, float inv_tau, int H, int Dk,
                                                           int DkP, const int* __restrict__ cu_q, int maxchunk, float qscale,
@@ -122,67 +146,112 @@ __global__ __launch_bounds__(GL_NT) void gla_chunk_kernel(const AT* __restrict__
   float* qs = lds;
   float* ks = qs + GL_C * W;
   float* bs = ks + GL_C * W;
+  float* tot = bs + GL_C * W;            // [16 / TPT][DkP]
   const int seq = blockIdx.x / maxchunk, c = blockIdx.x - seq * maxchunk, h = blockIdx.y, tid = threadIdx.x;
   const int a0 = cu_q[seq], a = a0 + c * GL_C, n = min(GL_C, cu_q[seq + 1] - a);
   if (n <= 0) return;
   const long no = chunk_no(a0, seq, c) * H + h;
-  for (int d = tid; d < DkP; d += GL_NT) {
-    const bool in = d < Dk;
+  constexpr int SP = GL_C / TPT;
+  const int d = tid % DkP, part = tid / DkP, t0 = part * TPT;
+  const bool mine = part < SP, in = mine && d < Dk;     // DkP SP <= GL_NT
+  float q[TPT], k[TPT], b[TPT], run = 0.f;
+  if (mine) {
+#pragma unroll
+    for (int i = 0; i < TPT; ++i) {
+      const int t = t0 + i;
+      const long r = (long)(a + min(t, n - 1));           // rows past the end: loaded, not used
+      const int dd = min(d, Dk - 1);
+      q[i] = (float)src[r * ld + (long)h * Dk + dd];
+      k[i] = (float)src[r * ld + (long)(H + h) * Dk + dd];
+      b[i] = (float)z[r * H * Dk + (long)h * Dk + dd];
+    }
     const float zbv = in ? zb[h * Dk + d] : 0.f;
-    float q[GL_C], k[GL_C], b[GL_C], run = 0.f;
 #pragma unroll
-    for (int t = 0; t < GL_C; ++t) {
-      const bool live = in && t < n;
-      const long r = (long)(a + (t < n ? t : 0));
-      q[t] = live ? (float)src[r * ld + (long)h * Dk + d] * qscale : 0.f;
-      k[t] = live ? (float)src[r * ld + (long)(H + h) * Dk + d] : 0.f;
-      b[t] = live ? (float)z[r * H * Dk + (long)h * Dk + d] : 0.f;
+    for (int i = 0; i < TPT; ++i) {
+      const bool live = in && t0 + i < n;
+      q[i] = live ? q[i] * qscale : 0.f;
+      k[i] = live ? k[i] : 0.f;
+      if (live) run += gl_log_decay(b[i] + zbv, inv_tau);
+      b[i] = run;
     }
-#pragma unroll
-    for (int t = 0; t < GL_C; ++t) {
-      if (in && t < n) run += gl_log_decay(b[t] + zbv, inv_tau);
-      b[t] = run;
-      qs[t * W + d] = q[t];
-      ks[t * W + d] = k[t];
-      bs[t * W + d] = run;
-      qd[(no * GL_C + t) * DkP + d] = q[t] * exp2f(run);
-    }
-#pragma unroll
-    for (int t = 0; t < GL_C; t += 4) {
-      f32x4 y;
-#pragma unroll
-      for (int j = 0; j < 4; ++j) y[j] = k[t + j] * exp2f(run - b[t + j]);
-      *(f32x4*)(kd + (no * DkP + d) * GL_C + t) = y;
-    }
-    dl[no * DkP + d] = exp2f(run);
+    tot[part * DkP + d] = run;
   }
   __syncthreads();
-  // A below and on the diagonal: 136 (t, s) pairs, 8 lanes each; above it zeros
-  float* ar = am + no * GL_C * GL_C;
-  constexpr int NP = GL_C * (GL_C + 1) / 2, ROUNDS = (NP * 8 + GL_NT - 1) / GL_NT;
-  for (int e = tid; e < GL_C * GL_C; e += GL_NT)
-    if ((e & (GL_C - 1)) > e / GL_C) ar[e] = 0.f;
+  if (mine) {
+    float before = 0.f, last = 0.f;
 #pragma unroll
-  for (int i = 0; i < ROUNDS; ++i) {
-    const int e = i * GL_NT + tid, p = min(e >> 3, NP - 1), part = e & 7;
-    int t = (int)((sqrtf(8.f * p + 1.f) - 1.f) * 0.5f);     // p = t (t + 1) / 2 + s
-    if ((t + 1) * (t + 2) / 2 <= p) ++t;
-    if (t * (t + 1) / 2 > p) --t;
-    const int s = p - t * (t + 1) / 2;
-    const float* qr = qs + t * W;
-    const float* kr = ks + s * W;
-    const float* bt = bs + t * W;
-    const float* bq = bs + s * W;
-    float acc = 0.f;
-    for (int d = part; d < DkP; d += 8) acc = fmaf(qr[d] * kr[d], exp2f(bt[d] - bq[d]), acc);
-    acc = group_sum<8>(acc);
-    if (part == 0 && (e >> 3) < NP) ar[t * GL_C + s] = acc;
+    for (int s = 0; s < SP; ++s) {
+      const float x = tot[s * DkP + d];
+      if (s < part) before += x;
+      last += x;
+    }
+#pragma unroll
+    for (int i = 0; i < TPT; ++i) {
+      const int t = t0 + i;
+      b[i] += before;
+      qs[t * W + d] = q[i];
+      ks[t * W + d] = k[i];
+      bs[t * W + d] = b[i];
+      qd[(no * GL_C + t) * DkP + d] = q[i] * exp2f(b[i]);
+    }
+#pragma unroll
+    for (int i = 0; i < TPT; i += 4) {
+      f32x4 y;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) y[j] = k[i + j] * exp2f(fminf(last - b[i + j], 0.f));
+      *(f32x4*)(kd + (no * DkP + d) * GL_C + t0 + i) = y;
+    }
+    if (part == 0) dl[no * DkP + d] = exp2f(last);
+  }
+  __syncthreads();
+  float* ar = am + no * GL_C * GL_C;
+  const int lane = tid & 63, wave = tid >> 6;
+  float acc[16];
+#pragma unroll
+  for (int e = 0; e < 16; ++e) acc[e] = 0.f;
+  if (wave == 0) {
+    const int T4 = (lane >> 4) * 4;
+    for (int x = lane & 15; x < DkP; x += 16) {
+      float qv[4], kv[4], bv[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        qv[i] = qs[(T4 + i) * W + x];
+        kv[i] = ks[(T4 + i) * W + x];
+        bv[i] = bs[(T4 + i) * W + x];
+      }
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j <= i; ++j) acc[4 * i + j] = fmaf(qv[i] * kv[j], i == j ? 1.f : exp2f(bv[i] - bv[j]), acc[4 * i + j]);
+    }
+    const float v = fold16<16>(acc, lane);
+    ar[(T4 + ((lane & 15) >> 2)) * GL_C + T4 + (lane & 3)] = v;
+  } else {
+    const int u = 2 * (wave - 1) + (lane >> 5);           // tiles (1,0) (2,0) (2,1) (3,0) (3,1) (3,2)
+    const int I = u == 0 ? 1 : (u < 3 ? 2 : 3), J = u - I * (I - 1) / 2;
+    for (int x = lane & 31; x < DkP; x += 32) {
+      const float cb = bs[4 * I * W + x];
+      float qv[4], kv[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        qv[i] = qs[(4 * I + i) * W + x] * exp2f(bs[(4 * I + i) * W + x] - cb);
+        kv[i] = ks[(4 * J + i) * W + x] * exp2f(cb - bs[(4 * J + i) * W + x]);
+      }
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) acc[4 * i + j] = fmaf(qv[i], kv[j], acc[4 * i + j]);
+    }
+    const float v = fold16<32>(acc, lane);
+    const int i = (lane & 15) >> 2, j = lane & 3;
+    if (lane & 16) ar[(4 * J + j) * GL_C + 4 * I + i] = 0.f;      // its mirror above the diagonal
+    else ar[(4 * I + i) * GL_C + 4 * J + j] = v;
   }
 }
 
 // grid (H, nseq, column groups), blockDim / 64 waves: one (portion, head, 16 value columns) per wave
 template <typename AT, int KB>
-__global__ __launch_bounds__(GL_NT) void gla_scan_kernel(const AT* __restrict__ src, long ld, int H, int Dk, int Dv,
+__global__ __launch_bounds__(GL_NT) __attribute__((amdgpu_waves_per_eu(1))) void gla_scan_kernel(const AT* __restrict__ src, long ld, int H, int Dk, int Dv,
                                                          const int* __restrict__ pos, const int* __restrict__ cu_q,
                                                          const int* __restrict__ sslots, float* __restrict__ state,
                                                          const float* __restrict__ qd, const float* __restrict__ kd,
@@ -205,62 +274,66 @@ __global__ __launch_bounds__(GL_NT) void gla_scan_kernel(const AT* __restrict__ 
       const int d = 16 * kb + 4 * g + i;
       S[kb][i] = st && !zero && d < Dk ? st[d] : 0.f;
     }
-  const AT* vp = src + 2L * H * Dk + (long)h * Dv + col;
+  // v of rows past the portion's end and of columns past Dv is some other element: their k and A are 0, their column is
+  // not stored.  No load behind a branch, so that a chunk's operands fly during the chunk before.
+  const AT* vp = src + 2L * H * Dk + (long)h * Dv + min(col, Dv - 1);
   const int nch = (b - a + GL_C - 1) / GL_C;
-  f32x4 qf[KB], kf[KB], df[KB], af;
-  float vf[4];
-  auto load = [&](int c, f32x4 (&Q)[KB], f32x4 (&K)[KB], f32x4 (&D)[KB], f32x4& A, float (&Vv)[4]) {
+  struct Ops {
+    f32x4 q[KB], k[KB], d[KB], a;
+    AT v[4];
+  };
+  auto load = [&](int c, Ops& x) {
     const long no = chunk_no(a, seq, c) * H + h;
     const float* qp = qd + (no * GL_C + r) * DkP + 4 * g;
     const float* kp = kd + (no * DkP + r) * GL_C + 4 * g;
     const float* dp = dl + no * DkP + 4 * g;
 #pragma unroll
-    for (int kb = 0; kb < KB; ++kb) {
-      Q[kb] = *(const f32x4*)(qp + 16 * kb);
-      K[kb] = *(const f32x4*)(kp + 16 * kb * GL_C);
-      D[kb] = *(const f32x4*)(dp + 16 * kb);
-    }
-    A = *(const f32x4*)(am + (no * GL_C + r) * GL_C + 4 * g);
+    for (int i = 0; i < 4; ++i) x.v[i] = vp[(long)min(a + c * GL_C + 4 * g + i, b - 1) * ld];
+    x.a = *(const f32x4*)(am + (no * GL_C + r) * GL_C + 4 * g);
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int t = a + c * GL_C + 4 * g + i;
-      Vv[i] = mine && t < b ? (float)vp[(long)t * ld] : 0.f;
+    for (int kb = 0; kb < KB; ++kb) {
+      x.q[kb] = *(const f32x4*)(qp + 16 * kb);
+      x.d[kb] = *(const f32x4*)(dp + 16 * kb);
+      x.k[kb] = *(const f32x4*)(kp + 16 * kb * GL_C);
     }
   };
-  load(0, qf, kf, df, af, vf);
-  for (int c = 0; c < nch; ++c) {
-    f32x4 qn[KB], kn[KB], dn[KB], an;
-    float vn[4];
-    load(min(c + 1, nch - 1), qn, kn, dn, an, vn);   // the next chunk's operands fly during this one
+  auto step = [&](int c, const Ops& x) {
     f32x4 oc[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};   // two chains of the read-out's sum
+    float vf[4];
 #pragma unroll
-    for (int i = 0; i < 4; ++i) oc[i & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(af[i], vf[i], oc[i & 1], 0, 0, 0);
+    for (int i = 0; i < 4; ++i) {
+      vf[i] = (float)x.v[i];
+      oc[i & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.a[i], vf[i], oc[i & 1], 0, 0, 0);
+    }
 #pragma unroll
     for (int kb = 0; kb < KB; ++kb) {
 #pragma unroll
-      for (int i = 0; i < 4; ++i)
-        oc[i & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(qf[kb][i], S[kb][i], oc[i & 1], 0, 0, 0);
+      for (int i = 0; i < 4; ++i) oc[i & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.q[kb][i], S[kb][i], oc[i & 1], 0, 0, 0);
 #pragma unroll
-      for (int i = 0; i < 4; ++i) S[kb][i] *= df[kb][i];
+      for (int i = 0; i < 4; ++i) S[kb][i] *= x.d[kb][i];
     }
 #pragma unroll
     for (int i = 0; i < 4; ++i)
 #pragma unroll
-      for (int kb = 0; kb < KB; ++kb) S[kb] = __builtin_amdgcn_mfma_f32_16x16x4f32(kf[kb][i], vf[i], S[kb], 0, 0, 0);
+      for (int kb = 0; kb < KB; ++kb) S[kb] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.k[kb][i], vf[i], S[kb], 0, 0, 0);
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int t = a + c * GL_C + 4 * g + i;
       if (mine && t < b) o[((long)t * H + h) * Dv + col] = oc[0][i] + oc[1][i];
     }
-#pragma unroll
-    for (int kb = 0; kb < KB; ++kb) {
-      qf[kb] = qn[kb];
-      kf[kb] = kn[kb];
-      df[kb] = dn[kb];
-    }
-    af = an;
-#pragma unroll
-    for (int i = 0; i < 4; ++i) vf[i] = vn[i];
+  };
+  Ops x0, x1;
+  load(0, x0);
+  for (int c = 0; c < nch; c += 2) {
+    load(min(c + 1, nch - 1), x1);
+    __builtin_amdgcn_sched_barrier(0);     // the loads stay ahead of the chunk they fly over
+    step(c, x0);
+    __builtin_amdgcn_sched_barrier(0);
+    if (c + 1 >= nch) break;
+    load(min(c + 2, nch - 1), x0);
+    __builtin_amdgcn_sched_barrier(0);
+    step(c + 1, x1);
+    __builtin_amdgcn_sched_barrier(0);
   }
   if (!st) return;
 #pragma unroll
@@ -338,11 +411,18 @@ static int gla_launch(const AT* src, long ld, const AT* z, const float* zb, floa
     if (v >= KB) break;
   }
   const int DkP = kbt * 16;
-  const size_t shm = (size_t)3 * GL_C * (DkP + 1) * sizeof(float);
-  if (shm > 48 * 1024)
-    (void)hipFuncSetAttribute((const void*)gla_chunk_kernel<AT>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)shm);
-  hipLaunchKernelGGL(gla_chunk_kernel<AT>, dim3(nseq * maxchunk, H), dim3(GL_NT), shm, st, src, ld, z, zb, inv_tau, H, Dk,
-                     DkP, cu_q, maxchunk, qscale, qd, kd, dl, am);
+  const int sp = DkP <= 64 ? 4 : (DkP <= 128 ? 2 : 1);      // threads a channel
+  const size_t shm = (size_t)(3 * GL_C * (DkP + 1) + sp * DkP) * sizeof(float);
+#define LA_GLK(TPT)                                                                                                      \
+  {                                                                                                                      \
+    if (shm > 48 * 1024)                                                                                                 \
+      (void)hipFuncSetAttribute((const void*)gla_chunk_kernel<AT, TPT>, hipFuncAttributeMaxDynamicSharedMemorySize,      \
+                                (int)shm);                                                                               \
+    hipLaunchKernelGGL((gla_chunk_kernel<AT, TPT>), dim3(nseq * maxchunk, H), dim3(GL_NT), shm, st, src, ld, z, zb,      \
+                       inv_tau, H, Dk, DkP, cu_q, maxchunk, qscale, qd, kd, dl, am);                                     \
+  }
+  if (sp == 4) LA_GLK(4) else if (sp == 2) LA_GLK(8) else LA_GLK(16)
+#undef LA_GLK
   const int blocks = (Dv + 15) / 16, waves = blocks < 4 ? blocks : 4;
 #define LA_GLC(KBT)                                                                                                    \
   if (kbt == KBT)                                                                                                      \

@@ -17,28 +17,32 @@ namespace la {
 //         their weights are the softmax over the chosen s.
 // groups > 1: experts form that many groups of neighbours; a group's score is its largest s (+ corr), and only
 // experts of the `keep` best groups can be chosen (ties: lowest group).  All weights times scale.
-template <typename AT>
-__global__ __launch_bounds__(256) void router_topk_kernel(const AT* __restrict__ x, long ldx,
+// SPREAD (batches of few rows): a workgroup per token whose waves take two experts each at a time, wave 0 chooses.
+template <typename AT, bool SPREAD>
+__global__ __launch_bounds__(SPREAD ? 1024 : 256) void router_topk_kernel(const AT* __restrict__ x, long ldx,
                                                           const float* __restrict__ router,
                                                           const float* __restrict__ corr, int E, int D, int T,
                                                           int topk, int renorm, int mode, int groups, int keep,
                                                           float scale, int* __restrict__ ids, float* __restrict__ wts) {
-  __shared__ float sc[4][256];
-  __shared__ uint8_t open[4][256];     // the expert's group can be chosen from
-  const int w = threadIdx.x >> 6, lane = threadIdx.x & 63;
-  const int t = blockIdx.x * 4 + w;
+  constexpr int NR = SPREAD ? 1 : 4, KE = SPREAD ? 2 : 8;     // tokens a workgroup, experts a pass of a wave
+  __shared__ float sc[NR][256];
+  __shared__ uint8_t open[NR][256];    // the expert's group can be chosen from
+  const int wave = threadIdx.x >> 6, w = SPREAD ? 0 : wave, lane = threadIdx.x & 63;
+  const int t = blockIdx.x * NR + w;
+  const bool chooses = !SPREAD || wave == 0;
   const bool live = t < T;
   const AT* xr = x + (long)(live ? t : 0) * ldx;
-  // 8 experts at a time: x is read once per pass and the 8 router rows give independent loads
-  for (int e0 = 0; e0 < E; e0 += 8) {
-    float a[8];
+  // KE experts at a time: x is read once per pass and the router rows give independent loads
+  for (int e0 = SPREAD ? wave * KE : 0; e0 < E; e0 += SPREAD ? (int)(blockDim.x >> 6) * KE : KE) {
+    float a[KE];
 #pragma unroll
-    for (int k = 0; k < 8; ++k) a[k] = 0.f;
+    for (int k = 0; k < KE; ++k) a[k] = 0.f;
     if ((D & 3) == 0) {
+#pragma unroll(SPREAD ? 8 : 1)
       for (int d = lane * 4; d < D; d += 256) {
         const float x0 = (float)xr[d], x1 = (float)xr[d + 1], x2 = (float)xr[d + 2], x3 = (float)xr[d + 3];
 #pragma unroll
-        for (int k = 0; k < 8; ++k) {
+        for (int k = 0; k < KE; ++k) {
           if (e0 + k < E) {
             const float4 r = *(const float4*)(router + (long)(e0 + k) * D + d);
             a[k] = fmaf(r.x, x0, fmaf(r.y, x1, fmaf(r.z, x2, fmaf(r.w, x3, a[k]))));
@@ -49,18 +53,18 @@ __global__ __launch_bounds__(256) void router_topk_kernel(const AT* __restrict__
       for (int d = lane; d < D; d += 64) {
         const float xv = (float)xr[d];
 #pragma unroll
-        for (int k = 0; k < 8; ++k)
+        for (int k = 0; k < KE; ++k)
           if (e0 + k < E) a[k] = fmaf(router[(long)(e0 + k) * D + d], xv, a[k]);
       }
     }
 #pragma unroll
-    for (int k = 0; k < 8; ++k) {
+    for (int k = 0; k < KE; ++k) {
       const float v = wave_sum(a[k]);
       if (lane == 0 && e0 + k < E) sc[w][e0 + k] = mode ? v + (corr ? corr[e0 + k] : 0.f) : 1.f / (1.f + __expf(-v));
     }
   }
   __syncthreads();
-  if (groups > 1) {
+  if (groups > 1 && chooses) {
     const int n = E / groups;
     float gm[4];                       // scores of groups lane, lane + 64, ..
     for (int i = 0; i < 4; ++i) {
@@ -90,8 +94,9 @@ __global__ __launch_bounds__(256) void router_topk_kernel(const AT* __restrict__
         for (int e = bi * n; e < (bi + 1) * n; ++e) open[w][e] = 1;
       }
     }
-    __syncthreads();
   }
+  if (groups > 1) __syncthreads();
+  if (!chooses) return;
   float sum = 0.f, my_s = 0.f, top0 = 0.f;
   int my_id = 0;
   uint32_t taken = 0;   // bit i: this lane's expert e = lane + 64 * i is already chosen
@@ -217,15 +222,18 @@ extern "C" int la_router_topk(int f32, int mode, const void* x, long ldx, const 
   using namespace la;
   if (E < 1 || E > 256 || topk < 1 || topk > E || topk > 64 || T <= 0 || mode < 0 || mode > 1) return -1;
   if (groups < 1 || E % groups || (groups > 1 && (keep < 1 || keep > groups || topk > keep * (E / groups)))) return -2;
-  dim3 grid((T + 3) / 4);
-  if (f32)
-    hipLaunchKernelGGL((router_topk_kernel<float>), grid, dim3(256), 0, (hipStream_t)stream, (const float*)x, ldx,
-                       (const float*)router, (const float*)corr, E, D, T, topk, renorm, mode, groups, keep, scale, (int*)ids,
-                       (float*)wts);
-  else
-    hipLaunchKernelGGL((router_topk_kernel<bf16>), grid, dim3(256), 0, (hipStream_t)stream, (const bf16*)x, ldx,
-                       (const float*)router, (const float*)corr, E, D, T, topk, renorm, mode, groups, keep, scale, (int*)ids,
-                       (float*)wts);
+  const bool spread = T <= 512;
+  const int nw = E > 32 ? 16 : (E + 1) / 2;
+#define LA_RT(AT, SP)                                                                                                   \
+  hipLaunchKernelGGL((router_topk_kernel<AT, SP>), dim3(SP ? T : (T + 3) / 4), dim3(SP ? 64 * nw : 256), 0,             \
+                     (hipStream_t)stream, (const AT*)x, ldx, (const float*)router, (const float*)corr, E, D, T, topk,   \
+                     renorm, mode, groups, keep, scale, (int*)ids, (float*)wts)
+  if (f32) {
+    if (spread) LA_RT(float, true); else LA_RT(float, false);
+  } else {
+    if (spread) LA_RT(bf16, true); else LA_RT(bf16, false);
+  }
+#undef LA_RT
   return (int)hipGetLastError();
 }
 
