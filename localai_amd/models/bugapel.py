@@ -158,8 +158,7 @@ class BugapelModel(LayeredModel):
     arch = "bugapel"
     # what this family launches from ops/csrc (ops.require_kernels: a first run compiles only these)
     kernel_sources = ("elementwise.hip", "hyper_streams.hip", "rope_pages.hip", "gla.hip", "attention_mix.hip", "attention.hip",
-                      "moe_dense.hip", "moe.hip", "norm_chain.hip", "shortconv.hip", "sampling.hip", "decode_loop.hip",
-                      "gemm_skinny.hip")
+                      "moe_dense.hip", "moe.hip", "sampling.hip", "decode_loop.hip", "gemm_skinny.hip")
 
     def __init__(self, reader, device: torch.device, tp: Optional[TPInfo] = None, max_pos: Optional[int] = None,
                  rope_overrides: Optional[dict] = None, lora=None, dtype: torch.dtype = torch.bfloat16):

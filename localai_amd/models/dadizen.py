@@ -31,14 +31,13 @@ from __future__ import annotations
 
 import os
 from dataclasses import dataclass, field
-from typing import Dict, List, Optional, Tuple
+from typing import List, Optional, Tuple
 
-import numpy as np
 import torch
 
 from .. import ops
-from ..gguf import dequantize
 from .decoder import ForwardBatch, KVCache, TPInfo
+from .layered import LayeredModel
 
 # decode rows of softmax attention through the matrix-core tile kernel where the shape allows
 DECODE_TILES = os.environ.get("LOCALAI_AMD_DADIZEN_DECODE_TILES", "1") == "1"
@@ -163,28 +162,17 @@ class _Layer:
     uv_t: Optional[torch.Tensor] = None         # [H, kv_rank, vdim]
 
 
-class DadizenModel:
+class DadizenModel(LayeredModel):
+    arch = "dadizen"
     # what this family launches from ops/csrc (ops.require_kernels: a first run compiles only these)
     kernel_sources = ("elementwise.hip", "norm_chain.hip", "rope_pages.hip", "retention.hip", "attention_mix.hip",
                       "attention.hip", "attention_latent.hip", "sampling.hip", "decode_loop.hip", "gemm_skinny.hip")
-    stateful = True         # retention state per sequence: state slots, no prefix-cache reuse
-    mixed_batches = True    # prompt portions and decode rows of different sequences in one forward
 
     def __init__(self, reader, device: torch.device, tp: Optional[TPInfo] = None, max_pos: Optional[int] = None,
                  rope_overrides: Optional[dict] = None, lora=None, dtype: torch.dtype = torch.bfloat16):
-        self.tp = tp or TPInfo()
-        if self.tp.world > 1:
-            raise ValueError("dadizen: tensor parallelism is not implemented for this design")
-        if lora is not None:
-            raise ValueError("dadizen: LoRA adapters are not supported")
-        if dtype not in (torch.bfloat16, torch.float32):
-            raise ValueError("dadizen: serving dtype is bfloat16 or float32")
-        self.device, self.dtype = device, dtype
-        self.f32 = dtype == torch.float32
+        self._begin(reader, device, tp, max_pos, lora, dtype)
         self.hp = hp = DadizenHParams.from_config(reader.config, str(reader.kv.get("general.name", "")))
-        self.max_pos = max_pos or 1 << 20
         self.vocab_local = hp.n_vocab
-        self.T = reader.tensors
         D = hp.n_embd
         raw, f32, qw = self._raw, self._f32, self._qw
         emb = raw("embed")
@@ -217,28 +205,11 @@ class DadizenModel:
             self.layers.append(L)
         self.out_norm = self._dyt("final.norm")
         self.output = qw(self._shaped("head", (hp.n_vocab, D)))
-        self._aranges: Dict[int, tuple] = {}
         self.T = None
 
     # --------------------------------------------------------------------------- loading
-    def _raw(self, name: str) -> torch.Tensor:
-        if name not in self.T:
-            raise KeyError(f"dadizen: missing tensor {name}")
-        t = self.T[name]
-        return torch.from_numpy(dequantize(t.data, t.ggml_type, t.shape).astype(np.float32).reshape(t.shape))
-
-    def _shaped(self, name: str, shape) -> torch.Tensor:
-        w = self._raw(name)
-        if tuple(w.shape) != tuple(shape):
-            raise ValueError(f"dadizen: {name} is {tuple(w.shape)}, the config asks for {tuple(shape)}")
-        return w
-
     def _f32(self, name: str) -> torch.Tensor:
         return self._raw(name).to(self.device).contiguous()
-
-    def _qw(self, w: torch.Tensor) -> ops.QWeight:
-        w = w.to(self.device)
-        return ops.QWeight.from_f32(w) if self.f32 else ops.QWeight.from_float(w)
 
     def _dyt(self, name: str) -> tuple:
         return ("dyt", float(self._raw(name + ".alpha").reshape(-1)[0]), self._f32(name), self._f32(name + ".b"))
@@ -290,22 +261,8 @@ class DadizenModel:
                 out.append((0, 0, 0, (m.heads, m.vdim, m.dim), torch.float32))
         return out
 
-    def kv_bytes_per_token(self) -> int:
-        es = 4 if self.f32 else 2
-        return max(es, sum(g * (dk + dv) * es for g, dk, dv, *_ in self._run_specs()))
-
-    def new_kv_cache(self, num_blocks: int, block_size: int, state_slots: int = 0) -> KVCache:
-        return KVCache.layered(self._run_specs(), num_blocks, block_size, self.device, self.dtype, state_slots)
-
-    def decode_workspace(self, Bp: int, ctx: int, block_size: int):
-        """Split-KV buffers of the decode attention kernel per (heads, kv heads, width) of the layers it serves."""
-        out = {}
-        for m in self.hp.mixers:
-            if m.kind == "attention" and self._decode_kernel_ok(m, block_size):
-                key = (m.heads, m.kv_heads, m.dim)
-                if key not in out:
-                    out[key] = ops.decode_workspace(Bp, m.heads, m.kv_heads, m.dim, ctx, self.device, block_size)
-        return out or None
+    def _attention_specs(self):
+        return [m for m in self.hp.mixers if m.kind == "attention"]
 
     def prefill_tiles(self, q_lens, device):
         """(16-row work tiles of the leading prompt portions for ops.attn_mix, rows they cover)."""
@@ -313,39 +270,12 @@ class DadizenModel:
             return None, 0
         return ops.attn_mix_tiles(q_lens, device)
 
-    def _single_rows(self, T: int):
-        """(row -> sequence, row ranges, one-row work tiles) of a batch with one row per sequence."""
-        a = self._aranges.get(T)
-        if a is None:
-            r = torch.arange(T + 1, dtype=torch.int32, device=self.device)
-            tiles = torch.stack([r[:T], torch.zeros_like(r[:T])], 1).contiguous()
-            a = self._aranges[T] = (r[:T].contiguous(), r, tiles)
-        return a
-
     # --------------------------------------------------------------------------- forward
-    def _dense(self, p: ops.Partial) -> torch.Tensor:
-        """A projection's rows as one contiguous [T, N] matrix of the activation dtype."""
-        t = p.t
-        if p.bias is None and t.dim() == 3 and t.shape[0] == 1:
-            t = t[0]
-        elif p.bias is not None or t.dim() == 3:
-            if t.is_cuda and p.N % 4 == 0:
-                return ops.reduce(p, dtype=self.dtype)
-            t = p.dense()
-        return t if t.dtype == self.dtype else t.to(self.dtype)
-
     def _rms(self, x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
         """Rows of a projection slice divided by their root mean square, times w (fp32 inside)."""
         y = torch.empty(x.shape[0], x.shape[1], dtype=torch.float32, device=x.device)
         return ops.norm_chain(y, x.contiguous(), post=("rms", w, self.hp.norm_eps), pre=("cast",), replace=True,
                               out_dtype=self.dtype)
-
-    def _decode_kernel_ok(self, m: MixSpec, block_size: int) -> bool:
-        """Decode batches of this layer on the framework's split-KV decode attention kernel (the llama
-        families'): bf16, equal key and value widths it is instantiated for; it takes the window."""
-        return (not self.f32 and self.device.type == "cuda" and m.dim == m.vdim and m.dim in (64, 80, 96, 128, 192, 256)
-                and m.heads // m.kv_heads <= 16 and block_size % 16 == 0 and (128 % block_size == 0 or block_size % 128 == 0)
-                and ops._has("la_attn_decode"))
 
     def _attention(self, L: _Layer, m: MixSpec, xn, fb, kv, run, row_seq, cu_q, tiles, tile_rows, splits, ws=None):
         proj = self._dense(ops.linear(xn, L.win))

@@ -27,20 +27,18 @@ from __future__ import annotations
 
 import os
 from dataclasses import dataclass, field
-from typing import Dict, List, Optional, Tuple
+from typing import List, Optional, Tuple
 
-import numpy as np
 import torch
 
 from .. import ops
-from ..gguf import dequantize
 from .decoder import ForwardBatch, KVCache, TPInfo
+from .layered import LayeredModel
 
 # decode rows of attention layers outside the split-KV decode kernel's widths: matrix-core tiles, keys dealt to
 # about this many workgroups a batch
 DECODE_TILES = os.environ.get("LOCALAI_AMD_DOBELIX_DECODE_TILES", "1") == "1"
 DECODE_WGS = int(os.environ.get("LOCALAI_AMD_DOBELIX_DECODE_WGS", "1024"))
-ATTN_WIDTHS = (64, 80, 96, 128, 192, 256)     # head widths the decode / prefill attention kernels are instantiated for
 
 
 @dataclass
@@ -125,28 +123,17 @@ class _Layer:
     down: Optional[ops.QWeight] = None
 
 
-class DobelixModel:
+class DobelixModel(LayeredModel):
+    arch = "dobelix"
     # what this family launches from ops/csrc (ops.require_kernels: a first run compiles only these)
     kernel_sources = ("elementwise.hip", "norm_chain.hip", "shortconv.hip", "rope_pages.hip", "retention.hip",
                       "attention_mix.hip", "attention.hip", "sampling.hip", "decode_loop.hip", "gemm_skinny.hip")
-    stateful = True         # convolution tails and recurrent state per sequence: state slots, no prefix-cache reuse
-    mixed_batches = True    # prompt portions and decode rows of different sequences in one forward
 
     def __init__(self, reader, device: torch.device, tp: Optional[TPInfo] = None, max_pos: Optional[int] = None,
                  rope_overrides: Optional[dict] = None, lora=None, dtype: torch.dtype = torch.bfloat16):
-        self.tp = tp or TPInfo()
-        if self.tp.world > 1:
-            raise ValueError("dobelix: tensor parallelism is not implemented for this design")
-        if lora is not None:
-            raise ValueError("dobelix: LoRA adapters are not supported")
-        if dtype not in (torch.bfloat16, torch.float32):
-            raise ValueError("dobelix: serving dtype is bfloat16 or float32")
-        self.device, self.dtype = device, dtype
-        self.f32 = dtype == torch.float32
+        self._begin(reader, device, tp, max_pos, lora, dtype)
         self.hp = hp = DobelixHParams.from_config(reader.config, str(reader.kv.get("general.name", "")))
-        self.max_pos = max_pos or 1 << 20
         self.vocab_local = hp.n_vocab
-        self.T = reader.tensors
         D = hp.n_embd
         sh, qw = self._shaped, self._qw
         self.tok_embd = ops.QWeight.from_float(sh("embed", (hp.n_vocab, D)).to(device))   # bf16 table, exact
@@ -161,29 +148,9 @@ class DobelixModel:
             self.layers.append(L)
         self.out_norm = ("rms", self._f32("final.norm", (D,)), hp.norm_eps)
         self.output = qw(sh("head", (hp.n_vocab, D)))
-        self._aranges: Dict[int, tuple] = {}
         self.T = None
 
     # --------------------------------------------------------------------------- loading
-    def _raw(self, name: str) -> torch.Tensor:
-        if name not in self.T:
-            raise KeyError(f"dobelix: missing tensor {name}")
-        t = self.T[name]
-        return torch.from_numpy(dequantize(t.data, t.ggml_type, t.shape).astype(np.float32).reshape(t.shape))
-
-    def _shaped(self, name: str, shape) -> torch.Tensor:
-        w = self._raw(name)
-        if tuple(w.shape) != tuple(shape):
-            raise ValueError(f"dobelix: {name} is {tuple(w.shape)}, the config asks for {tuple(shape)}")
-        return w
-
-    def _f32(self, name: str, shape) -> torch.Tensor:
-        return self._shaped(name, shape).to(self.device).contiguous()
-
-    def _qw(self, w: torch.Tensor) -> ops.QWeight:
-        w = w.to(self.device)
-        return ops.QWeight.from_f32(w) if self.f32 else ops.QWeight.from_float(w)
-
     def _layer(self, p: str, win: torch.Tensor, wo: torch.Tensor) -> _Layer:
         D, taps = self.hp.n_embd, self.hp.taps
         conv = self._shaped(p + "canon1", (D, taps)).t().contiguous().to(self.device)
@@ -210,73 +177,17 @@ class DobelixModel:
         return L
 
     # --------------------------------------------------------------------------- engine interface
-    def _specs(self):
+    def _run_specs(self):
         """KVCache.layered spec of every layer: the stream's convolution tail (fp32), beside pages for an
         attention layer or the recurrent state of a lightning layer."""
         tail = ((self.hp.taps - 1, self.hp.n_embd), torch.float32)
         return [(m.kv_heads, m.dim, m.vdim, [tail]) if m.kind == "attention"
                 else (0, 0, 0, [tail, ((m.heads, m.vdim, m.dim), torch.float32)]) for m in self.hp.mixers]
 
-    def kv_bytes_per_token(self) -> int:
-        es = 4 if self.f32 else 2
-        return max(es, sum(g * (dk + dv) * es for g, dk, dv, *_ in self._specs()))
-
-    def new_kv_cache(self, num_blocks: int, block_size: int, state_slots: int = 0) -> KVCache:
-        return KVCache.layered(self._specs(), num_blocks, block_size, self.device, self.dtype, state_slots)
-
-    def decode_workspace(self, Bp: int, ctx: int, block_size: int):
-        """Split-KV buffers of the decode attention kernel per (heads, kv heads, width) of the layers it serves."""
-        out = {}
-        for m in self.hp.mixers:
-            if m.kind == "attention" and self._decode_kernel_ok(m, block_size):
-                key = (m.heads, m.kv_heads, m.dim)
-                if key not in out:
-                    out[key] = ops.decode_workspace(Bp, m.heads, m.kv_heads, m.dim, ctx, self.device, block_size)
-        return out or None
-
-    def _decode_kernel_ok(self, m: MixSpec, block_size: int) -> bool:
-        """Decode batches of this layer on the framework's split-KV decode attention kernel (the llama
-        families'): bf16 and a head width it is instantiated for."""
-        return (not self.f32 and self.device.type == "cuda" and m.dim in ATTN_WIDTHS and m.heads // m.kv_heads <= 16
-                and block_size % 16 == 0 and (128 % block_size == 0 or block_size % 128 == 0) and ops._has("la_attn_decode"))
-
-    def _prefill_kernel_ok(self, m: MixSpec) -> bool:
-        """Batches of prompt portions only, for this layer, on the framework's prefill attention kernel (64
-        query rows of one head per workgroup)."""
-        return (not self.f32 and self.device.type == "cuda" and m.dim in ATTN_WIDTHS and ops._has("la_attn_prefill"))
-
-    def prefill_tiles(self, q_lens, device):
-        """((16-row work tiles of the leading prompt portions for ops.attn_mix, 64-row tiles of the same
-        portions for ops.attn_prefill where a layer has the widths that kernel takes), rows they cover)."""
-        if device.type != "cuda" or self.f32:
-            return None, 0
-        mix, rows = ops.attn_mix_tiles(q_lens, device)
-        pf = None
-        if any(m.kind == "attention" and self._prefill_kernel_ok(m) for m in self.hp.mixers):
-            pf = ops.prefill_tiles(q_lens, device)
-        return (mix, pf), rows
-
-    def _single_rows(self, T: int):
-        """(row -> sequence, row ranges, one-row work tiles) of a batch with one row per sequence."""
-        a = self._aranges.get(T)
-        if a is None:
-            r = torch.arange(T + 1, dtype=torch.int32, device=self.device)
-            tiles = torch.stack([r[:T], torch.zeros_like(r[:T])], 1).contiguous()
-            a = self._aranges[T] = (r[:T].contiguous(), r, tiles)
-        return a
+    def _attention_specs(self):
+        return [m for m in self.hp.mixers if m.kind == "attention"]
 
     # --------------------------------------------------------------------------- forward
-    def _dense(self, p: ops.Partial) -> torch.Tensor:
-        """A projection's rows as one contiguous [T, N] matrix of the activation dtype."""
-        t = p.t
-        if p.bias is None and t.dim() == 3 and t.shape[0] == 1:
-            t = t[0]
-        elif p.bias is not None or t.dim() == 3:
-            if t.is_cuda and p.N % 4 == 0:
-                return ops.reduce(p, dtype=self.dtype)
-            t = p.dense()
-        return t if t.dtype == self.dtype else t.to(self.dtype)
-
     def _attention(self, L: _Layer, m: MixSpec, h, fb, kv, i, row_seq, cu_q, tiles, tile_rows, splits, ws=None):
         proj = self._dense(ops.linear(h, L.win))             # [T, q | k | gate]
         kc, vc = kv.k[i], kv.v[i]

@@ -37,19 +37,14 @@ from __future__ import annotations
 
 import os
 from dataclasses import dataclass, field
-from typing import Dict, List, Optional, Tuple
+from typing import List, Optional, Tuple
 
-import numpy as np
 import torch
 
 from .. import ops
-from ..gguf import dequantize
 from .decoder import ForwardBatch, KVCache, TPInfo
+from .layered import LayeredModel, RoutedExperts
 
-# routed experts: (token, expert) pair GEMVs up to this many rows, grouped rows + library GEMMs beyond
-MOE_PAIR_MAX_T = int(os.environ.get("LOCALAI_AMD_GOSUVIK_PAIR_MAX_T", "32"))
-# from this many rows on the grouped expert kernels give way to library GEMMs per expert
-MOE_DENSE_MIN_T = 6144
 DECODE_TILES = os.environ.get("LOCALAI_AMD_GOSUVIK_DECODE_TILES", "1") == "1"
 DECODE_WGS = int(os.environ.get("LOCALAI_AMD_GOSUVIK_DECODE_WGS", "1024"))
 UNIT_EPS = 1e-6      # inside the root of the delta rule's unit-length q and k
@@ -170,12 +165,6 @@ class GosuvikHParams:
 
 
 @dataclass
-class _Expert:
-    gate_up: ops.QWeight
-    down: ops.QWeight
-
-
-@dataclass
 class _Layer:
     norm1: torch.Tensor
     win: ops.QWeight                   # the mixer's fused input projections (see the loaders)
@@ -209,37 +198,21 @@ class _Layer:
     down: Optional[ops.QWeight] = None
     poly: Optional[torch.Tensor] = None          # fp32 [4]
     router: Optional[torch.Tensor] = None        # fp32 [E, D]
-    wg: Optional[torch.Tensor] = None            # stacked expert weights [E, F, D] / [E, D, F], activation dtype
-    wu: Optional[torch.Tensor] = None
-    wd: Optional[torch.Tensor] = None
-    experts: Optional[List[_Expert]] = None
-    moe_gu: Optional[object] = None              # ops.MoEWeights where the grouped expert GEMMs take the shape
-    moe_down: Optional[object] = None
+    experts: Optional[RoutedExperts] = None
 
 
-class GosuvikModel:
+class GosuvikModel(LayeredModel):
+    arch = "gosuvik"
     # what this family launches from ops/csrc (ops.require_kernels: a first run compiles only these)
     kernel_sources = ("elementwise.hip", "norm_chain.hip", "rope_pages.hip", "retention.hip", "delta_rule.hip",
                       "matrix_memory.hip", "attention_mix.hip", "attention.hip", "attention_latent.hip", "moe_dense.hip",
                       "moe.hip", "sampling.hip", "decode_loop.hip", "gemm_skinny.hip")
-    stateful = True         # convolution tails and recurrent state per sequence: state slots, no prefix-cache reuse
-    mixed_batches = True    # prompt portions and decode rows of different sequences in one forward
 
     def __init__(self, reader, device: torch.device, tp: Optional[TPInfo] = None, max_pos: Optional[int] = None,
                  rope_overrides: Optional[dict] = None, lora=None, dtype: torch.dtype = torch.bfloat16):
-        self.tp = tp or TPInfo()
-        if self.tp.world > 1:
-            raise ValueError("gosuvik: tensor parallelism is not implemented for this design")
-        if lora is not None:
-            raise ValueError("gosuvik: LoRA adapters are not supported")
-        if dtype not in (torch.bfloat16, torch.float32):
-            raise ValueError("gosuvik: serving dtype is bfloat16 or float32")
-        self.device, self.dtype = device, dtype
-        self.f32 = dtype == torch.float32
+        self._begin(reader, device, tp, max_pos, lora, dtype)
         self.hp = hp = GosuvikHParams.from_config(reader.config, str(reader.kv.get("general.name", "")))
-        self.max_pos = max_pos or 1 << 20
         self.vocab_local = hp.n_vocab
-        self.T = reader.tensors
         D = hp.n_embd
         self.tok_embd = ops.QWeight.from_float(self._shaped("embed", (hp.n_vocab, D)).to(device))   # bf16 table, exact
         self.layers: List[_Layer] = []
@@ -254,29 +227,9 @@ class GosuvikModel:
             self.layers.append(L)
         self.out_norm = self._f32("final.norm", (D,))
         self.output = self._qw(self._shaped("head", (hp.n_vocab, D)))
-        self._aranges: Dict[int, tuple] = {}
         self.T = None
 
     # --------------------------------------------------------------------------- loading
-    def _raw(self, name: str) -> torch.Tensor:
-        if name not in self.T:
-            raise KeyError(f"gosuvik: missing tensor {name}")
-        t = self.T[name]
-        return torch.from_numpy(dequantize(t.data, t.ggml_type, t.shape).astype(np.float32).reshape(t.shape))
-
-    def _shaped(self, name: str, shape) -> torch.Tensor:
-        w = self._raw(name)
-        if tuple(w.shape) != tuple(shape):
-            raise ValueError(f"gosuvik: {name} is {tuple(w.shape)}, the config asks for {tuple(shape)}")
-        return w
-
-    def _f32(self, name: str, shape) -> torch.Tensor:
-        return self._shaped(name, shape).to(self.device).contiguous()
-
-    def _qw(self, w: torch.Tensor) -> ops.QWeight:
-        w = w.to(self.device)
-        return ops.QWeight.from_f32(w) if self.f32 else ops.QWeight.from_float(w)
-
     def _freqs(self, r: RotSpec):
         """(frequencies, magnitude) of a rotation: YaRN when the scaling names an original length,
         positions divided by the factor when it gives a factor alone."""
@@ -357,16 +310,8 @@ class GosuvikModel:
         if not 1 <= f.top <= f.experts:
             raise ValueError(f"{p}: top must lie in 1 .. experts")
         L.router = self._f32(p + "router", (f.experts, D))
-        ws = [(sh(p + f"e{e}.gate", (f.ff, D)), sh(p + f"e{e}.up", (f.ff, D)), sh(p + f"e{e}.down", (D, f.ff)))
-              for e in range(f.experts)]
-        L.wg, L.wu, L.wd = (torch.stack([w[k] for w in ws]).to(device=self.device, dtype=self.dtype).contiguous()
-                            for k in range(3))
-        L.experts = [_Expert(qw(torch.cat([g, u], 0)), qw(d)) for g, u, d in ws]
-        if not self.f32 and self.device.type == "cuda" and D % 256 == 0 and f.ff % 256 == 0:
-            # the framework's grouped expert GEMMs (one weight stream per active expert, device
-            # routing, no host sync) read [gate; up] fused per expert
-            L.moe_gu = ops.MoEWeights([e.gate_up for e in L.experts])
-            L.moe_down = ops.MoEWeights([e.down for e in L.experts])
+        L.experts = RoutedExperts([(sh(p + f"e{e}.gate", (f.ff, D)), sh(p + f"e{e}.up", (f.ff, D)), sh(p + f"e{e}.down", (D, f.ff)))
+                                   for e in range(f.experts)], self.device, self.dtype, "silu")
 
     # --------------------------------------------------------------------------- engine interface
     def _run_specs(self):
@@ -386,69 +331,10 @@ class GosuvikModel:
                                                         ((r.heads,), torch.float32)]))
         return out
 
-    def kv_bytes_per_token(self) -> int:
-        es = 4 if self.f32 else 2
-        return max(es, sum(g * (dk + dv) * es for g, dk, dv, *_ in self._run_specs()))
-
-    def new_kv_cache(self, num_blocks: int, block_size: int, state_slots: int = 0) -> KVCache:
-        return KVCache.layered(self._run_specs(), num_blocks, block_size, self.device, self.dtype, state_slots)
-
-    def decode_workspace(self, Bp: int, ctx: int, block_size: int):
-        """Split-KV buffers of the decode attention kernel per (heads, kv heads, width) of the layers it serves."""
-        out = {}
-        for m in self.hp.mixers:
-            l = m.left
-            if l is not None and self._decode_kernel_ok(l, block_size):
-                key = (l.heads, l.kv_heads, l.dim)
-                if key not in out:
-                    out[key] = ops.decode_workspace(Bp, l.heads, l.kv_heads, l.dim, ctx, self.device, block_size)
-        return out or None
-
-    def _decode_kernel_ok(self, l: MixSpec, block_size: int) -> bool:
-        """Decode batches of this attention on the framework's split-KV decode attention kernel (the llama
-        families'): bf16, equal key and value widths it is instantiated for; it takes the window and the sink."""
-        return (not self.f32 and self.device.type == "cuda" and l.dim == l.vdim and l.dim in (64, 80, 96, 128, 192, 256)
-                and l.heads // l.kv_heads <= 16 and block_size % 16 == 0 and (128 % block_size == 0 or block_size % 128 == 0)
-                and ops._has("la_attn_decode"))
-
-    def _prefill_kernel_ok(self, l: MixSpec) -> bool:
-        """Batches of prompt portions only, for this attention, on the framework's prefill attention kernel
-        (64 query rows of one head per workgroup): bf16, equal key and value widths it is instantiated for."""
-        return (not self.f32 and self.device.type == "cuda" and l.dim == l.vdim and l.dim in (64, 80, 96, 128, 192, 256)
-                and ops._has("la_attn_prefill"))
-
-    def prefill_tiles(self, q_lens, device):
-        """((16-row work tiles of the leading prompt portions for ops.attn_mix, 64-row tiles of the same
-        portions for ops.attn_prefill where a layer has the widths that kernel takes), rows they cover)."""
-        if device.type != "cuda" or self.f32:
-            return None, 0
-        mix, rows = ops.attn_mix_tiles(q_lens, device)
-        pf = None
-        if any(m.left is not None and self._prefill_kernel_ok(m.left) for m in self.hp.mixers):
-            pf = ops.prefill_tiles(q_lens, device)
-        return (mix, pf), rows
-
-    def _single_rows(self, T: int):
-        """(row -> sequence, row ranges, one-row work tiles) of a batch with one row per sequence."""
-        a = self._aranges.get(T)
-        if a is None:
-            r = torch.arange(T + 1, dtype=torch.int32, device=self.device)
-            tiles = torch.stack([r[:T], torch.zeros_like(r[:T])], 1).contiguous()
-            a = self._aranges[T] = (r[:T].contiguous(), r, tiles)
-        return a
+    def _attention_specs(self):
+        return [m.left for m in self.hp.mixers if m.left is not None]
 
     # --------------------------------------------------------------------------- forward
-    def _dense(self, p: ops.Partial) -> torch.Tensor:
-        """A projection's rows as one contiguous [T, N] matrix of the activation dtype."""
-        t = p.t
-        if p.bias is None and t.dim() == 3 and t.shape[0] == 1:
-            t = t[0]
-        elif p.bias is not None or t.dim() == 3:
-            if t.is_cuda and p.N % 4 == 0:
-                return ops.reduce(p, dtype=self.dtype)
-            t = p.dense()
-        return t if t.dtype == self.dtype else t.to(self.dtype)
-
     def _delta(self, L: _Layer, m: MixSpec, xn, fb, kv, run, cu_q):
         proj = self._dense(ops.linear(xn, L.win))            # [T, q | k | v | beta | decay rank | gate rank]
         c0 = 2 * m.kv_heads * m.dim + m.heads * m.vdim + m.heads
@@ -508,50 +394,10 @@ class GosuvikModel:
                           max_rows=1 if fb.decode else fb.max_q, out=both, col0=nl)
         return both
 
-    def _unit(self, x: torch.Tensor, e: _Expert, ff: int):
-        """One gated expert on rows x: down(silu(gate x) * up x)."""
-        gu = ops.linear(x, e.gate_up)
-        if not self.f32 and (ff % 4 == 0 or not x.is_cuda):
-            h = ops.act(gu, ff, ops.ACT_SWIGLU)
-        else:
-            g = self._dense(gu).float()
-            h = (torch.nn.functional.silu(g[:, :ff]) * g[:, ff:]).to(self.dtype)
-        return ops.linear(h, e.down)
-
-    def _routed(self, L: _Layer, f: FfSpec, xn: torch.Tensor):
-        """The weighted sum of every row's chosen experts (fp32 [T, D], or a Partial of it)."""
-        T = xn.shape[0]
-        ids, wts = ops.router_softmax(xn, L.router, None, f.top)
-        capturing = xn.is_cuda and torch.cuda.is_current_stream_capturing()
-        if L.moe_gu is not None and (T < MOE_DENSE_MIN_T or capturing) and T > 2:
-            order, off = ops.moe_route(ids, f.experts)
-            gu = ops.moe_linear(xn, L.moe_gu, order, off, f.top, T)
-            h = ops.act(gu, f.ff, ops.ACT_SWIGLU)
-            return ops.moe_linear(h, L.moe_down, order, off, f.top, T, down=True, wts=wts)
-        if T <= MOE_PAIR_MAX_T or capturing:
-            return ops.moe_pairs(xn, L.wg, L.wu, L.wd, ids, wts)
-        # rows grouped by expert (device), one host read of the group offsets, then per expert
-        # gate|up and down as library GEMMs over its rows and a weighted scatter-add in fp32
-        order, off = ops.moe_route(ids, f.experts)
-        off_h = off.cpu().tolist()
-        order_l = order.long()
-        tok = order_l // f.top
-        xs = xn.index_select(0, tok)
-        wsel = wts.index_select(0, order_l)
-        out = torch.zeros(T, self.hp.n_embd, dtype=torch.float32, device=xn.device)
-        with ops.blas_tuning_paused():
-            for e in range(f.experts):
-                r0, r1 = off_h[e], off_h[e + 1]
-                if r1 <= r0:
-                    continue
-                y = self._dense(self._unit(xs[r0:r1].contiguous(), L.experts[e], f.ff)).float()
-                out.index_add_(0, tok[r0:r1], y * wsel[r0:r1].unsqueeze(1))
-        return out
-
     def _mlp(self, L: _Layer, f: FfSpec, xn: torch.Tensor):
         if f.kind == "dense":
             return ops.linear(ops.poly_norm_act(ops.linear(xn, L.up), L.poly, self.hp.norm_eps, self.dtype), L.down)
-        return self._routed(L, f, xn)
+        return L.experts(xn, *ops.router_softmax(xn, L.router, None, f.top))
 
     def forward(self, fb: ForwardBatch, kv: KVCache, attn_workspace=None, return_hidden: bool = False,
                 local_logits: bool = False, layer_out: Optional[list] = None) -> torch.Tensor:

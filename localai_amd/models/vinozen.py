@@ -33,19 +33,14 @@ from __future__ import annotations
 
 import os
 from dataclasses import dataclass, field
-from typing import Dict, List, Optional, Tuple
+from typing import List, Optional, Tuple
 
-import numpy as np
 import torch
 
 from .. import ops
-from ..gguf import dequantize
 from .decoder import ForwardBatch, KVCache, TPInfo
+from .layered import LayeredModel, RoutedExperts
 
-# routed experts: (token, expert) pair GEMVs up to this many rows, grouped rows + library GEMMs beyond
-MOE_PAIR_MAX_T = int(os.environ.get("LOCALAI_AMD_VINOZEN_PAIR_MAX_T", "32"))
-# from this many rows on the grouped expert kernels give way to library GEMMs per expert
-MOE_DENSE_MIN_T = 6144
 DECODE_TILES = os.environ.get("LOCALAI_AMD_VINOZEN_DECODE_TILES", "1") == "1"
 DECODE_WGS = int(os.environ.get("LOCALAI_AMD_VINOZEN_DECODE_WGS", "1024"))
 
@@ -163,41 +158,25 @@ class _Layer:
     down: Optional[ops.QWeight] = None
     router: Optional[torch.Tensor] = None        # fp32 [E, D]
     router_b: Optional[torch.Tensor] = None
-    wg: Optional[torch.Tensor] = None            # stacked expert weights [E, F, D] / [E, D, F], activation dtype
-    wu: Optional[torch.Tensor] = None
-    wd: Optional[torch.Tensor] = None
-    experts: Optional[List[_Expert]] = None
-    moe_gu: Optional[object] = None              # ops.MoEWeights where the grouped expert GEMMs take the shape
-    moe_down: Optional[object] = None
+    experts: Optional[RoutedExperts] = None
     shared: Optional[_Expert] = None
     side_gate: Optional[ops.QWeight] = None
     side_proj: Optional[ops.QWeight] = None
     side_norm: Optional[torch.Tensor] = None
 
 
-class VinozenModel:
+class VinozenModel(LayeredModel):
+    arch = "vinozen"
     # what this family launches from ops/csrc (ops.require_kernels: a first run compiles only these)
     kernel_sources = ("elementwise.hip", "norm_chain.hip", "rope_pages.hip", "retention.hip", "mamba2.hip",
                       "attention_mix.hip", "attention.hip", "moe_dense.hip", "moe.hip", "sampling.hip", "decode_loop.hip",
                       "gemm_skinny.hip")
-    stateful = True         # convolution tails and recurrent state per sequence: state slots, no prefix-cache reuse
-    mixed_batches = True    # prompt portions and decode rows of different sequences in one forward
 
     def __init__(self, reader, device: torch.device, tp: Optional[TPInfo] = None, max_pos: Optional[int] = None,
                  rope_overrides: Optional[dict] = None, lora=None, dtype: torch.dtype = torch.bfloat16):
-        self.tp = tp or TPInfo()
-        if self.tp.world > 1:
-            raise ValueError("vinozen: tensor parallelism is not implemented for this design")
-        if lora is not None:
-            raise ValueError("vinozen: LoRA adapters are not supported")
-        if dtype not in (torch.bfloat16, torch.float32):
-            raise ValueError("vinozen: serving dtype is bfloat16 or float32")
-        self.device, self.dtype = device, dtype
-        self.f32 = dtype == torch.float32
+        self._begin(reader, device, tp, max_pos, lora, dtype)
         self.hp = hp = VinozenHParams.from_config(reader.config, str(reader.kv.get("general.name", "")))
-        self.max_pos = max_pos or 1 << 20
         self.vocab_local = hp.n_vocab
-        self.T = reader.tensors
         D = hp.n_embd
         f32, qw, sh = self._f32, self._qw, self._shaped
         emb = sh("embed", (hp.n_vocab, D))
@@ -220,29 +199,9 @@ class VinozenModel:
                 L.side_norm = f32(p + "side.norm", (D,))
             self.layers.append(L)
         self.out_norm = ("ln", f32("final.norm", (D,)), hp.norm_eps)
-        self._aranges: Dict[int, tuple] = {}
         self.T = None
 
     # --------------------------------------------------------------------------- loading
-    def _raw(self, name: str) -> torch.Tensor:
-        if name not in self.T:
-            raise KeyError(f"vinozen: missing tensor {name}")
-        t = self.T[name]
-        return torch.from_numpy(dequantize(t.data, t.ggml_type, t.shape).astype(np.float32).reshape(t.shape))
-
-    def _shaped(self, name: str, shape) -> torch.Tensor:
-        w = self._raw(name)
-        if tuple(w.shape) != tuple(shape):
-            raise ValueError(f"vinozen: {name} is {tuple(w.shape)}, the config asks for {tuple(shape)}")
-        return w
-
-    def _f32(self, name: str, shape) -> torch.Tensor:
-        return self._shaped(name, shape).to(self.device).contiguous()
-
-    def _qw(self, w: torch.Tensor) -> ops.QWeight:
-        w = w.to(self.device)
-        return ops.QWeight.from_f32(w) if self.f32 else ops.QWeight.from_float(w)
-
     def _load_attention(self, p: str, m: MixSpec) -> _Layer:
         D, H = self.hp.n_embd, m.heads
         sh = self._shaped
@@ -289,21 +248,14 @@ class VinozenModel:
             raise ValueError(f"{p}: top must lie in 1 .. experts")
         L.router = self._f32(p + "router", (f.experts, D))
         L.router_b = self._f32(p + "router.b", (f.experts,)) if p + "router.b" in self.T else None
-        ws = [self._expert(p + f"e{e}.", f.ff) for e in range(f.experts)]
-        L.wg, L.wu, L.wd = (torch.stack([w[k] for w in ws]).to(device=self.device, dtype=self.dtype).contiguous()
-                            for k in range(3))
-        L.experts = [_Expert(qw(torch.cat([g, u], 0)), qw(d)) for g, u, d in ws]
-        if not self.f32 and self.device.type == "cuda" and D % 256 == 0 and f.ff % 256 == 0:
-            # the framework's grouped expert GEMMs (one weight stream per active expert, device
-            # routing, no host sync) read [gate; up] fused per expert
-            L.moe_gu = ops.MoEWeights([e.gate_up for e in L.experts])
-            L.moe_down = ops.MoEWeights([e.down for e in L.experts])
+        L.experts = RoutedExperts([self._expert(p + f"e{e}.", f.ff) for e in range(f.experts)], self.device, self.dtype,
+                                  ("clamp", f.limit, 1.702))
         if f.shared_ff:
             g, u, d = self._expert(p + "shared.", f.shared_ff)
             L.shared = _Expert(qw(torch.cat([g, u], 0)), qw(d))
 
     # --------------------------------------------------------------------------- engine interface
-    def _specs(self):
+    def _run_specs(self):
         """KVCache.layered spec of every layer: pages for attention layers with projections of their
         own, (convolution tail, recurrent state) for mamba2 layers."""
         out = []
@@ -315,104 +267,13 @@ class VinozenModel:
                 out.append((0, 0, 0, [((max(m.taps - 1, 0), C), None), ((m.heads, m.vdim, m.state), torch.float32)]))
         return out
 
-    def kv_bytes_per_token(self) -> int:
-        es = 4 if self.f32 else 2
-        return max(es, sum(g * (dk + dv) * es for g, dk, dv, *_ in self._specs()))
-
-    def new_kv_cache(self, num_blocks: int, block_size: int, state_slots: int = 0) -> KVCache:
-        return KVCache.layered(self._specs(), num_blocks, block_size, self.device, self.dtype, state_slots)
-
-    def decode_workspace(self, Bp: int, ctx: int, block_size: int):
-        """Split-KV buffers of the decode attention kernel per (heads, kv heads, width) of the layers it serves."""
-        out = {}
-        for m in self.hp.mixers:
-            if m.kind == "attention" and self._decode_kernel_ok(m, block_size):
-                key = (m.heads, m.kv_heads, m.dim)
-                if key not in out:
-                    out[key] = ops.decode_workspace(Bp, m.heads, m.kv_heads, m.dim, ctx, self.device, block_size)
-        return out or None
-
-    def _decode_kernel_ok(self, m: MixSpec, block_size: int) -> bool:
-        """Decode batches of this layer on the framework's split-KV decode attention kernel (the llama
-        families'): bf16, equal key and value widths it is instantiated for; it takes the bias table and the sink."""
-        return (not self.f32 and self.device.type == "cuda" and m.dim == m.vdim and m.dim in (64, 80, 96, 128, 192, 256)
-                and m.heads // m.kv_heads <= 16 and block_size % 16 == 0 and (128 % block_size == 0 or block_size % 128 == 0)
-                and ops._has("la_attn_decode"))
-
-    def prefill_tiles(self, q_lens, device):
-        """((16-row work tiles of the leading prompt portions for ops.attn_mix, 64-row tiles of the same
-        portions for ops.attn_prefill where a layer has the widths that kernel takes), rows they cover)."""
-        if device.type != "cuda" or self.f32:
-            return None, 0
-        mix, rows = ops.attn_mix_tiles(q_lens, device)
-        pf = None
-        if any(m.kind == "attention" and self._prefill_kernel_ok(m) for m in self.hp.mixers):
-            pf = ops.prefill_tiles(q_lens, device)
-        return (mix, pf), rows
-
-    def _prefill_kernel_ok(self, m: MixSpec) -> bool:
-        """Batches of prompt portions only, for this layer, on the framework's prefill attention kernel (the
-        llama families': 64 query rows of one head per workgroup): bf16, equal key and value widths it is
-        instantiated for; it takes the bias table and the sink."""
-        return (not self.f32 and self.device.type == "cuda" and m.dim == m.vdim and m.dim in (64, 80, 96, 128, 192, 256)
-                and ops._has("la_attn_prefill"))
-
-    def _single_rows(self, T: int):
-        """(row -> sequence, row ranges, one-row work tiles) of a batch with one row per sequence."""
-        a = self._aranges.get(T)
-        if a is None:
-            r = torch.arange(T + 1, dtype=torch.int32, device=self.device)
-            tiles = torch.stack([r[:T], torch.zeros_like(r[:T])], 1).contiguous()
-            a = self._aranges[T] = (r[:T].contiguous(), r, tiles)
-        return a
+    def _attention_specs(self):
+        return [m for m in self.hp.mixers if m.kind == "attention"]
 
     # --------------------------------------------------------------------------- forward
-    def _dense(self, p: ops.Partial) -> torch.Tensor:
-        """A projection's rows as one contiguous [T, N] matrix of the activation dtype."""
-        t = p.t
-        if p.bias is None and t.dim() == 3 and t.shape[0] == 1:
-            t = t[0]
-        elif p.bias is not None or t.dim() == 3:
-            if t.is_cuda and p.N % 4 == 0:
-                return ops.reduce(p, dtype=self.dtype)
-            t = p.dense()
-        return t if t.dtype == self.dtype else t.to(self.dtype)
-
     def _unit(self, x: torch.Tensor, e: _Expert, ff: int, limit: float):
         """One clamped gated expert on rows x: down(glu_clamp(gate|up x))."""
         return ops.linear(ops.glu_clamp(ops.linear(x, e.gate_up), ff, limit, out_dtype=self.dtype), e.down)
-
-    def _routed(self, L: _Layer, f: FfSpec, xn: torch.Tensor) -> torch.Tensor:
-        """fp32 [T, D]: the weighted sum of every row's chosen experts."""
-        T = xn.shape[0]
-        ids, wts = ops.router_softmax(xn, L.router, L.router_b, f.top)
-        capturing = xn.is_cuda and torch.cuda.is_current_stream_capturing()
-        if L.moe_gu is not None and (T < MOE_DENSE_MIN_T or capturing) and T > 2:
-            # grouped expert GEMMs on the routed rows, as the Mixtral path: gate|up, the clamped unit,
-            # then the down projection with the routing weights
-            order, off = ops.moe_route(ids, f.experts)
-            gu = ops.moe_linear(xn, L.moe_gu, order, off, f.top, T)
-            h = ops.glu_clamp(gu, f.ff, f.limit, out_dtype=self.dtype)
-            return ops.moe_linear(h, L.moe_down, order, off, f.top, T, down=True, wts=wts).dense()
-        if T <= MOE_PAIR_MAX_T or capturing:
-            return ops.moe_pairs(xn, L.wg, L.wu, L.wd, ids, wts, clamp=(f.limit, 1.702))
-        # rows grouped by expert (device), one host read of the group offsets, then per expert
-        # gate|up and down as library GEMMs over its rows and a weighted scatter-add in fp32
-        order, off = ops.moe_route(ids, f.experts)
-        off_h = off.cpu().tolist()
-        order_l = order.long()
-        tok = order_l // f.top
-        xs = xn.index_select(0, tok)
-        wsel = wts.index_select(0, order_l)
-        out = torch.zeros(T, self.hp.n_embd, dtype=torch.float32, device=xn.device)
-        with ops.blas_tuning_paused():
-            for e in range(f.experts):
-                r0, r1 = off_h[e], off_h[e + 1]
-                if r1 <= r0:
-                    continue
-                y = self._dense(self._unit(xs[r0:r1].contiguous(), L.experts[e], f.ff, f.limit)).float()
-                out.index_add_(0, tok[r0:r1], y * wsel[r0:r1].unsqueeze(1))
-        return out
 
     def _mlp(self, L: _Layer, f: FfSpec, xn: torch.Tensor):
         if f.kind == "dense":
@@ -423,7 +284,8 @@ class VinozenModel:
                 x = self._dense(gu).float()
                 h = (torch.nn.functional.silu(x[:, :f.ff]) * x[:, f.ff:]).to(self.dtype)
             return ops.linear(h, L.down)
-        y = self._routed(L, f, xn)
+        y = L.experts(xn, *ops.router_softmax(xn, L.router, L.router_b, f.top))
+        y = y.dense() if isinstance(y, ops.Partial) else y
         if L.shared is not None:
             y = y + self._dense(self._unit(xn, L.shared, f.shared_ff, f.shared_limit)).float()
         return y
