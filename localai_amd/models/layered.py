@@ -163,8 +163,12 @@ class LayeredModel:
         """fp32 logits of the rows fb.logits_idx selects (all when None), softcap tanh(. / softcap) when given."""
         rows = x if fb.logits_idx is None else x.index_select(0, fb.logits_idx)
         lp = ops.linear(rows.contiguous(), self.output)
-        lg = lp.t[0] if (lp.t.dim() == 3 and lp.t.shape[0] == 1 and lp.t.dtype == torch.float32) else self._dense(lp).float()
-        return lg.div_(softcap).tanh_().mul_(softcap) if softcap > 0 else lg
+        if softcap <= 0 and lp.t.dim() == 3 and lp.t.shape[0] == 1:
+            return lp.t[0]
+        if lp.N % 4 == 0 or not lp.t.is_cuda:
+            return ops.reduce(lp, softcap=softcap)       # slabs, soft cap and fp32 rows in one launch
+        lg = lp.dense()
+        return torch.tanh(lg / softcap) * softcap if softcap > 0 else lg
 
     def _attend(self, q: torch.Tensor, m, kc: torch.Tensor, vc: torch.Tensor, fb: ForwardBatch, b: BatchRows, splits: int = 1,
                 workspace=None, **kw) -> torch.Tensor:

@@ -83,7 +83,7 @@ def lib():
             "la_groupnorm_nhwc": [P, P, P, P, P, I, I, I, I, I, I, F, I, P],
             "la_mamba_ssm_step": [P, P, P, P, LNG, I, I, P, P, P, LNG, P, I, I, I, P],
             "la_act": [P, LNG, I, P, P, I, I, I, P],
-            "la_reduce_slabs": [P, LNG, I, P, I, I, P, P, P],
+            "la_reduce_slabs": [P, LNG, I, P, I, I, P, P, F, P],
             "la_embed": [I, P, P, P, P, I, I, P, I, P, F, P],
             "la_dequant": [I, P, P, P, P, I, I, P, P],
             "la_attn_decode": [P, P, P, P, I, P, I, I, I, I, I, F, I, I, P, P, P, P, P, LNG, I, P, P, P, P, F, I, I, P, I, P,
@@ -1430,14 +1430,15 @@ def act_linear(src: Partial, F: int, mode: int, w: QWeight) -> Partial:
     return linear(act(src, F, mode), w)
 
 
-def reduce(src: Partial, dtype=torch.float32, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+def reduce(src: Partial, dtype=torch.float32, out: Optional[torch.Tensor] = None, softcap: float = 0.0) -> torch.Tensor:
     """Sum of the split-K slabs (+ bias) as one dense [M, N] matrix (into `out`, a contiguous
-    [M, N] tensor of `dtype`, when given)."""
+    [M, N] tensor of `dtype`, when given); softcap > 0: softcap * tanh(sum / softcap)."""
     if out is not None:
         dtype = out.dtype
         assert out.is_contiguous() and tuple(out.shape) == (src.M, src.N)
     if not src.t.is_cuda:
-        d = src.dense().to(dtype)
+        d = src.dense()
+        d = (torch.tanh(d / softcap) * softcap if softcap > 0 else d).to(dtype)
         if out is None:
             return d
         out.copy_(d)
@@ -1448,7 +1449,8 @@ def reduce(src: Partial, dtype=torch.float32, out: Optional[torch.Tensor] = None
     a = src.src_args()
     f32 = out.data_ptr() if dtype == torch.float32 else None
     b16 = out.data_ptr() if dtype == torch.bfloat16 else None
-    _check(lib().la_reduce_slabs(a[0], a[1], a[2], a[3], T, N, f32, b16, _stream()), "la_reduce_slabs")
+    _check(lib().la_reduce_slabs(a[0], a[1], a[2], a[3], T, N, f32, b16, float(softcap), _stream()),
+           "la_reduce_slabs")
     return out
 
 

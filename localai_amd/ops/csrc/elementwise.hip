@@ -507,14 +507,18 @@ __global__ __launch_bounds__(256) void act8_kernel(const bf16* __restrict__ src,
   *(bf16x8*)(out + (long)t * F + c) = ob;
 }
 
-// sum split-K slabs (+bias) -> f32 or bf16 matrix [T][N]
+// sum split-K slabs (+bias) -> f32 or bf16 matrix [T][N]; cap > 0: cap * tanh(sum / cap)
 __global__ __launch_bounds__(256) void reduce_slabs_kernel(Src src, int N, float* __restrict__ out_f32,
-                                                           bf16* __restrict__ out_bf16) {
+                                                           bf16* __restrict__ out_bf16, float cap) {
   const int t = blockIdx.y;
   const int c = (blockIdx.x * blockDim.x + threadIdx.x) * 4;
   if (c >= N) return;
   float a[4];
   load4(src, (long)t * N + c, c, a);
+  if (cap > 0.f) {
+#pragma unroll
+    for (int j = 0; j < 4; ++j) a[j] = cap * tanhf(a[j] / cap);
+  }
   if (out_f32) *(float4*)(out_f32 + (long)t * N + c) = make_float4(a[0], a[1], a[2], a[3]);
   if (out_bf16) {
     bf16x4 ob = {(bf16)a[0], (bf16)a[1], (bf16)a[2], (bf16)a[3]};
@@ -681,12 +685,12 @@ extern "C" int la_act(const void* p, long slab, int S, const void* bias, void* o
 }
 
 extern "C" int la_reduce_slabs(const void* p, long slab, int S, const void* bias, int T, int N, void* out_f32,
-                               void* out_bf16, void* stream) {
+                               void* out_bf16, float cap, void* stream) {
   if (N & 3) return -1;
   Src s{p, slab, S, (const float*)bias};
   dim3 grid((N / 4 + 255) / 256, T);
   hipLaunchKernelGGL(la::reduce_slabs_kernel, grid, dim3(256), 0, (hipStream_t)stream, s, N, (float*)out_f32,
-                     (bf16*)out_bf16);
+                     (bf16*)out_bf16, cap);
   return (int)hipGetLastError();
 }
 

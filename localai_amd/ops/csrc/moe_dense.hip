@@ -42,11 +42,9 @@ __global__ __launch_bounds__(SPREAD ? 1024 : 256) void router_topk_kernel(const 
       for (int d = lane * 4; d < D; d += 256) {
         const float x0 = (float)xr[d], x1 = (float)xr[d + 1], x2 = (float)xr[d + 2], x3 = (float)xr[d + 3];
 #pragma unroll
-        for (int k = 0; k < KE; ++k) {
-          if (e0 + k < E) {
-            const float4 r = *(const float4*)(router + (long)(e0 + k) * D + d);
-            a[k] = fmaf(r.x, x0, fmaf(r.y, x1, fmaf(r.z, x2, fmaf(r.w, x3, a[k]))));
-          }
+        for (int k = 0; k < KE; ++k) {     // past the last expert: its row again, the sum unused (no branch between loads)
+          const float4 r = *(const float4*)(router + (long)min(e0 + k, E - 1) * D + d);
+          a[k] = fmaf(r.x, x0, fmaf(r.y, x1, fmaf(r.z, x2, fmaf(r.w, x3, a[k]))));
         }
       }
     } else {

@@ -322,20 +322,19 @@ __global__ __launch_bounds__(RP_NT) void qk_row_norm_rope_pages_kernel(
 // Row [q (H x Dq) | k (G x Dk) | v (G x Dv)] plus bias.  A unit is V pairs of the rotated span (2 V dims) or V dims
 // of the rest; the LG lanes of a head take its units in turn.  unit: the head divided by sqrt(mean x^2 + eps);
 // a rotation keeps the sum of squares, so it is taken from the values as they are read.
+// The workgroup has RP_NT threads, or four times as many where the batch has few rows (every head at once).
 template <typename AT, int V>
-__global__ __launch_bounds__(RP_NT) void head_rope_pages_kernel(
+__global__ __launch_bounds__(4 * RP_NT) void head_rope_pages_kernel(
     RowSrc src, long ld, const float* __restrict__ bias, int H, int Dq, int G, int Dk, int Dv,
     const int* __restrict__ pos, const int* __restrict__ slots, const float* __restrict__ freqs, int rot, int interleaved,
     int unit, float eps, int LG, AT* __restrict__ q_out, AT* __restrict__ kc, AT* __restrict__ vc, int BS) {
   typedef typename RowVec<V>::type fvec;
   typedef AT avec __attribute__((ext_vector_type(V)));
   extern __shared__ float cs[];          // [rot / 2][2]
-  const int t = blockIdx.x, tid = threadIdx.x, half = rot >> 1;
+  const int t = blockIdx.x, tid = threadIdx.x, half = rot >> 1, NT = blockDim.x;
   const int Cq = H * Dq, Ck = G * Dk, Cv = G * Dv;
   const long row = (long)t * ld;
   const int p = pos[t];
-  for (int i = tid; i < half; i += RP_NT) sincosf((float)p * freqs[i], &cs[2 * i + 1], &cs[2 * i]);
-  __syncthreads();
   const int slot = G ? slots[t] : -1;
   const int blk = slot >= 0 ? slot / BS : 0, off = slot >= 0 ? slot - blk * BS : 0;
   auto value = [&](int c) -> fvec {
@@ -354,33 +353,40 @@ __global__ __launch_bounds__(RP_NT) void head_rope_pages_kernel(
     *(avec*)p = y;
   };
   const int lane = tid % LG, nh = slot >= 0 ? H + G : H, pairs = half / V;
-  for (int u = tid / LG; u < nh; u += RP_NT / LG) {
+  // columns of unit k of a head: first, and for a rotated unit also second
+  auto first = [&](int k) { return k < pairs ? (interleaved ? 2 * k * V : k * V) : rot + (k - pairs) * V; };
+  auto second = [&](int k) { return interleaved ? (2 * k + 1) * V : k * V + half; };
+  auto column = [&](int u) { return u < H ? u * Dq : Cq + (u - H) * Dk; };
+  auto units = [&](int u) { return pairs + ((u < H ? Dq : Dk) - rot) / V; };
+  fvec a = fvec(0.f), b = fvec(0.f);
+  auto load = [&](int c0, int k) {
+    a = value(c0 + first(k));
+    b = k < pairs ? value(c0 + second(k)) : fvec(0.f);
+  };
+  // the first head's values are on their way while the angles are evaluated
+  const int u0 = tid / LG;
+  if (u0 < nh && lane < units(u0)) load(column(u0), lane);
+  for (int i = tid; i < half; i += NT) sincosf((float)p * freqs[i], &cs[2 * i + 1], &cs[2 * i]);
+  __syncthreads();
+  for (int u = u0; u < nh; u += NT / LG) {
     const bool isq = u < H;
-    const int D = isq ? Dq : Dk, c0 = isq ? u * Dq : Cq + (u - H) * Dk, per = pairs + (D - rot) / V;
+    const int D = isq ? Dq : Dk, c0 = column(u), per = units(u);
     AT* dst = isq ? q_out + (long)t * Cq + (long)u * Dq : kc + (((long)blk * G + (u - H)) * BS + off) * Dk;
-    // columns of unit k: a, and for a rotated unit also b
-    auto first = [&](int k) { return k < pairs ? (interleaved ? 2 * k * V : k * V) : rot + (k - pairs) * V; };
-    auto second = [&](int k) { return interleaved ? (2 * k + 1) * V : k * V + half; };
-    fvec a = fvec(0.f), b = fvec(0.f);
-    auto load = [&](int k) {
-      a = value(c0 + first(k));
-      b = k < pairs ? value(c0 + second(k)) : fvec(0.f);
-    };
     float inv = 1.f;
-    if (lane < per) load(lane);
+    if (u != u0 && lane < per) load(c0, lane);
     if (unit) {
       float ss = 0.f;
       for (int k = lane; k < per; k += LG) {
-        if (k != lane) load(k);
+        if (k != lane) load(c0, k);
 #pragma unroll
         for (int j = 0; j < V; ++j) ss = fmaf(a[j], a[j], fmaf(b[j], b[j], ss));
       }
       for (int o = LG >> 1; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
       inv = 1.f / sqrtf(ss / (float)D + eps);
-      if (per > LG && lane < per) load(lane);
+      if (per > LG && lane < per) load(c0, lane);
     }
     for (int k = lane; k < per; k += LG) {
-      if (k != lane) load(k);
+      if (k != lane) load(c0, k);
       if (k < pairs) {
         fvec ya, yb;
         if (V == 1 || !interleaved) {
@@ -411,7 +417,7 @@ __global__ __launch_bounds__(RP_NT) void head_rope_pages_kernel(
     }
   }
   if (slot < 0) return;
-  for (int e = tid * V; e < Cv; e += RP_NT * V) {
+  for (int e = tid * V; e < Cv; e += NT * V) {
     const int g = e / Dv, d = e - g * Dv;
     const fvec x = value(Cq + Ck + e);
     AT* dst = vc + ((((long)blk * G + g) * (BS >> 3) + (off >> 3)) * Dv + d) * 8 + (off & 7);
@@ -461,8 +467,9 @@ extern "C" int la_head_rope_pages(int f32, const void* sp, int src_f32, long sla
   const int v = vec ? 4 : 1, D = Dq > Dk ? Dq : Dk, per = rot / 2 / v + (D - rot) / v;
   int LG = 4;
   while (LG < 64 && LG < per) LG <<= 1;
+  const int nt = T <= 512 && (H + G) * LG > RP_NT ? 4 * RP_NT : RP_NT;
 #define LA_HRP(AT, V)                                                                                                    \
-  hipLaunchKernelGGL((head_rope_pages_kernel<AT, V>), dim3(T), dim3(RP_NT), shm, (hipStream_t)stream, s, ld,             \
+  hipLaunchKernelGGL((head_rope_pages_kernel<AT, V>), dim3(T), dim3(nt), shm, (hipStream_t)stream, s, ld,                \
                      (const float*)bias, H, Dq, G, Dk, Dv, (const int*)pos, (const int*)slots, (const float*)freqs, rot, \
                      interleaved, unit, eps, LG, (AT*)q_out, (AT*)kc, (AT*)vc, BS)
   if (f32) {

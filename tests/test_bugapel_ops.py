@@ -137,6 +137,33 @@ def test_rotated_heads_into_pages(device, interleaved, H, G, D, Dv, rot):
             assert float(kc[1, :, 2:].float().min()) == 7.0 and float(vc[3, :, 0, :, :7].float().min()) == 7.0
 
 
+@pytest.mark.parametrize("device", DEVICES)
+def test_rotated_heads_of_many_rows(device):
+    """More rows than the few that get large workgroups: the same numbers as row by row."""
+    H, G, D, Dv, rot, T, BS = 8, 2, 64, 32, 32, 530, 16
+    g = torch.Generator().manual_seed(3)
+    src = torch.randn(T, H * D + G * (D + Dv), generator=g).to(device)
+    fq, _ = ops.rot_freqs(rot, 50.0, None, device)
+    pools = [(torch.zeros(34, G, BS, D, device=device), torch.zeros(34, G, BS // 8, Dv, 8, device=device)) for _ in range(2)]
+    pos, slots = i32(range(T), device), i32(range(T), device)
+    q = ops.head_rope_pages(src, H, D, G, D, Dv, pos, slots, fq, rot, True, *pools[0], unit_eps=1e-4, dtype=torch.float32)
+    parts = [ops.head_rope_pages(src[a:a + 53], H, D, G, D, Dv, pos[a:a + 53], slots[a:a + 53], fq, rot, True, *pools[1], unit_eps=1e-4,
+                                 dtype=torch.float32) for a in range(0, T, 53)]
+    assert rel(q, torch.cat(parts)) < 1e-6 and rel(pools[0][0], pools[1][0]) < 1e-6 and rel(pools[0][1], pools[1][1]) == 0.0
+    t = 511
+    want = oracle.unit_rms(oracle.rotate(src[t, :H * D].cpu().double().view(H, D), t, oracle.frequencies(rot, 50.0), True), 1e-4)
+    assert rel(q[t].view(H, D), want) < 1e-4
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_slab_sums_with_a_soft_cap(device):
+    g = torch.Generator().manual_seed(4)
+    for src, val in results(g, 5, 40, device):
+        if isinstance(src, ops.Partial):
+            for dt, tol in ((torch.float32, 1e-6), (torch.bfloat16, 5e-3)):
+                assert rel(ops.reduce(src, dt, softcap=1.5), 1.5 * torch.tanh(val.double() / 1.5)) < tol
+
+
 # ------------------------------------------------------------------------------------------- kept first tokens, a one in the denominator
 def paged(rows_k, rows_v, perm, BS, nb, dt, dev):
     """Pages (leftovers of 50 elsewhere) holding every sequence's keys and values, and the block tables."""
@@ -375,14 +402,15 @@ def test_gla_remembers_over_a_long_run(device, dtype):
 @pytest.mark.parametrize("device,dtype", MODES)
 @pytest.mark.parametrize("E,groups,keep,top,D", [(12, 3, 2, 3, 40), (6, 1, 1, 2, 35), (8, 8, 3, 3, 64), (200, 20, 4, 8, 64), (9, 3, 1, 3, 33), (4, 2, 2, 4, 128),
                                                  (256, 128, 5, 6, 32)])
-def test_router_takes_the_best_groups_first(device, dtype, E, groups, keep, top, D):
+@pytest.mark.parametrize("T", [37, 600])
+def test_router_takes_the_best_groups_first(device, dtype, E, groups, keep, top, D, T):
+    """Few rows (a workgroup each) and many (four a workgroup)."""
     g = torch.Generator().manual_seed(E)
-    T = 37
     x = torch.randn(T, D, generator=g).to(torch.bfloat16).float()
     w = torch.randn(E, D, generator=g)
     ids, wts = ops.router_softmax(x.to(device=device, dtype=getattr(torch, dtype)), w.to(device), None, top, groups, keep, 2.5)
     other = 0
-    for t in range(T):
+    for t in range(0, T, 1 if T < 100 else 13):
         z = w.double() @ x[t].double()
         want_i, want_w = oracle.route(z, top, groups, keep, 2.5)
         assert ids[t].tolist() == want_i
