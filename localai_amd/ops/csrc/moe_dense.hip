@@ -38,13 +38,28 @@ __global__ __launch_bounds__(SPREAD ? 1024 : 256) void router_topk_kernel(const 
 #pragma unroll
     for (int k = 0; k < KE; ++k) a[k] = 0.f;
     if ((D & 3) == 0) {
-#pragma unroll(SPREAD ? 8 : 1)
-      for (int d = lane * 4; d < D; d += 256) {
-        const float x0 = (float)xr[d], x1 = (float)xr[d + 1], x2 = (float)xr[d + 2], x3 = (float)xr[d + 3];
+      // U slices of 256 columns at a time, all their loads before the first sum; past the row's end or the last
+      // expert: some valid element, times 0 or into a sum nobody reads
+      constexpr int U = SPREAD ? 8 : 2;
+      for (int d0 = lane * 4; d0 - lane * 4 < D; d0 += 256 * U) {
+        AT xv[U][4];
+        float4 rv[U][KE];
 #pragma unroll
-        for (int k = 0; k < KE; ++k) {     // past the last expert: its row again, the sum unused (no branch between loads)
-          const float4 r = *(const float4*)(router + (long)min(e0 + k, E - 1) * D + d);
-          a[k] = fmaf(r.x, x0, fmaf(r.y, x1, fmaf(r.z, x2, fmaf(r.w, x3, a[k]))));
+        for (int u = 0; u < U; ++u) {
+          const int d = min(d0 + 256 * u, D - 4);
+#pragma unroll
+          for (int j = 0; j < 4; ++j) xv[u][j] = xr[d + j];
+#pragma unroll
+          for (int k = 0; k < KE; ++k) rv[u][k] = *(const float4*)(router + (long)min(e0 + k, E - 1) * D + d);
+        }
+        __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+          const float in = d0 + 256 * u < D ? 1.f : 0.f;
+          const float x0 = in * (float)xv[u][0], x1 = in * (float)xv[u][1], x2 = in * (float)xv[u][2], x3 = in * (float)xv[u][3];
+#pragma unroll
+          for (int k = 0; k < KE; ++k)
+            a[k] = fmaf(rv[u][k].x, x0, fmaf(rv[u][k].y, x1, fmaf(rv[u][k].z, x2, fmaf(rv[u][k].w, x3, a[k]))));
         }
       }
     } else {
